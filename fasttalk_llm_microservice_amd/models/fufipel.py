@@ -220,16 +220,12 @@ class FufipelModel(StackedModel):
     family = "Fufipel"
     norm_style = "shared_pre"
 
-    def one_plus(self, t: torch.Tensor) -> torch.Tensor:
-        """fp32 weight of a norm stored as an offset from one."""
-        return (1.0 + self.norm_weight(t)).contiguous()
-
     def load_tensors(self, get, has=lambda n: True):
         cfg, dev, dt = self.cfg, self.device, self.dtype
         eps, width = cfg.rms_norm_eps, cfg.hidden_size
         self.load_head(get, lambda n: n != "head" and has(n))     # the embedding table is the head
         self.embed_scale, self.logit_scale, self.residual_mult = cfg.embed_scale, cfg.logit_scale, cfg.residual_mult
-        self.final_norm = self.one_plus(get("final.norm"))
+        self.final_norm = self.offset_norm_weight(get("final.norm"))
         if cfg.bigram:
             buckets, mul_prev, mul_cur = cfg.bigram
             table = get("bigram").to(dev, dt).contiguous()
@@ -259,7 +255,7 @@ class FufipelModel(StackedModel):
                                              b["vdim"], b["tau"], eps, dt, dev)
                 mixer = SideBySide(left, right, get(p + "mix.left.out"), get(p + "mix.right.out"), eps, dev,
                                    PARALLEL_MEAN)
-            L = StackedLayer(l["type"], self.one_plus(get(p + "norm1")), None, mixer)
+            L = StackedLayer(l["type"], self.offset_norm_weight(get(p + "norm1")), None, mixer)
             if l["mlp"] is not None:
                 L.ff = GatedFF(lambda n, p=p: get(p + "mlp." + n), dt, dev, act="relu")
             self.layers.append(L)

@@ -11,6 +11,9 @@ builds the layer list in ``load_tensors``.
 Per run, with x the residual:  x += norm1b(mixer(norm1 x));
 x += norm2b(ff(norm2 x)) (if the layer has a feed-forward);
 x += rms(side(x, token)) * side.norm (if it has a token-side input).
+A layer with a token shift (``StackedLayer.shift``) hands its mixer h + (h' - h) * shift,
+h = norm1 x and h' the h of the token before; every run keeps a sequence's last h in its
+state slot.
 
 A model with ``norm_style = "layer_post"`` has no norm in front of its sublayers: they
 read x itself, and a layer norm with weight and bias sits on each sublayer's output,
@@ -54,6 +57,8 @@ class StackedLayer:
     # biases of the output norms (layer-norm models)
     bias1: Optional[torch.Tensor] = None
     bias2: Optional[torch.Tensor] = None
+    # fp32 [width]: how far the mixer's input moves towards the previous token's
+    shift: Optional[torch.Tensor] = None
 
 
 class StackedCache:
@@ -146,6 +151,10 @@ class StackedModel:
             t = t.reshape(1).expand(self.cfg.hidden_size)
         return t.contiguous()
 
+    def offset_norm_weight(self, t: torch.Tensor) -> torch.Tensor:
+        """fp32 weight of a norm stored as an offset from one."""
+        return (1.0 + self.norm_weight(t)).contiguous()
+
     def load_checkpoint(self, ckpt_dir: str):
         idx = W.SafetensorsIndex(ckpt_dir)
         return self.load_tensors(idx.get, idx.has)
@@ -197,6 +206,10 @@ class StackedModel:
         extra = {}
         if self.pair_embed is not None:
             extra["last_token"] = torch.full((max(num_slots, 1),), -1, dtype=torch.int32, device=self.device)
+        if any(L.shift is not None for L in self.layers):
+            extra["prev_h"] = [torch.zeros(max(num_slots, 1), self.cfg.hidden_size, dtype=torch.float32,
+                                           device=self.device) if self.layers[i].shift is not None else None
+                               for i, _ in self.runs]
         return StackedCache(per_run, extra)
 
     # ------------------------------------------------------------------ forward
@@ -217,11 +230,14 @@ class StackedModel:
         h = None
         nruns = len(self.runs)
         mark = self.mark_at
+        prev_h = caches.extra.get("prev_h")
         for r, (li, step) in enumerate(self.runs):
             if mark is not None and r == mark[0]:
                 mark[1].record()
             L = self.layers[li]
-            if h is None:   # first run, or the step vector was not fused into the last kernel
+            if h is None and L.shift is not None:
+                x, h = M.add_norm_shift_rows(x, None, None, L.norm1, L.shift, eps, dt, prev_h[r], seg)
+            elif h is None:   # first run, or the step vector was not fused into the last kernel
                 vec = self.loop_step[step] if step is not None and (r == 0 or not fuse_step) else None
                 h = M.rms_norm_rows(x, L.norm1, eps, dt, add_vec=vec)
             y = L.mixer(h, ctx, caches.per_run[r])
@@ -229,6 +245,19 @@ class StackedModel:
             nvec = self.loop_step[nxt[1]] if nxt is not None and nxt[1] is not None and fuse_step else None
             nw = self.layers[nxt[0]].norm1 if nxt is not None and (fuse_step or nxt[1] is None) else None
             last = L.ff is None and L.side is None
+            nshift = self.layers[nxt[0]].shift if nxt is not None else None
+            if nshift is not None:
+                # the layer's last add, the next layer's norm and its token shift in one kernel
+                if L.side is not None or nxt[1] is not None:
+                    raise NotImplementedError("a token shift after a token-side input or a loop step")
+                wb = L.norm1b
+                if L.ff is not None:
+                    h, _ = M.add_rms_norm_rows(x, y, L.norm1b, eps, next_w=L.norm2, out_dtype=dt)
+                    y, wb = L.ff(h, ctx), L.norm2b
+                x, h = M.add_norm_shift_rows(x, y, wb, self.layers[nxt[0]].norm1, nshift, eps, dt, prev_h[r + 1], seg)
+                if tap is not None:
+                    tap.append(x.clone())
+                continue
             h, xc = M.add_rms_norm_rows(x, y, L.norm1b, eps,
                                         add_vec=nvec if last else None,
                                         next_w=L.norm2 if L.ff is not None else (nw if last else None),

@@ -1,12 +1,12 @@
 """Sequence-mixer and mixture-of-experts ops: latent (low-rank KV) attention over a
 paged latent cache, windowed attention (softmax or sigmoid weights, distance bias,
 several score maps per head, capped scores, a sink in the softmax) over a paged key /
-value cache, the gated delta-rule recurrence with per-channel decay and the selective
+value cache, attention that mixes its scores across the heads, the gated delta-rule recurrence with per-channel decay and the selective
 state-space scan over state slots, short causal convolutions (alone, or fused with
 per-head norms and the cache write), routing (grouped softmax top-k, or top-k on the
-logits), clamped-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product
-for many), and the fp32-residual norms (RMS pre/post norms, layer norm with bias) that tie
-them together.
+logits with softmax or sigmoid weights), clamped-GLU, silu-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product
+for many), and the fp32-residual norms (RMS pre/post norms, optionally with a token shift, layer
+norm with bias) that tie them together.
 
 GPU tensors run the gfx950 kernels of the ``_C_mixers`` extension (``csrc/mixers``),
 fp32 or bf16 activations with fp32 statistics / scores / state; CPU tensors run the
@@ -160,6 +160,25 @@ def add_scaled_rms_norm_rows(residual: torch.Tensor, y1: Optional[torch.Tensor],
     return ref.add_scaled_rms_norm_rows(residual, y1, y2, mult, next_w, eps, out_dtype)
 
 
+def add_norm_shift_rows(residual: torch.Tensor, y: Optional[torch.Tensor], wb: Optional[torch.Tensor], w: torch.Tensor,
+                        shift: torch.Tensor, eps: float, out_dtype, prev_state: torch.Tensor, seg: "Segments"):
+    """One step between layers with a token shift: x = residual + rms_norm(y) * wb (x =
+    residual without y), h = rms_norm(x) * w, and what the next sublayer reads is
+    h + (h' - h) * shift element by element, h' being the h of the token before in its
+    sequence (zeros for a sequence's first token).  ``prev_state`` [slots, width] fp32
+    holds each sequence's last h and is updated.  Returns (x fp32, shifted h in
+    ``out_dtype``); x may or may not be ``residual`` itself, which must not be read
+    afterwards.  h and the shift are fp32, rounded once."""
+    if residual.is_cuda:
+        h = torch.empty(residual.shape, dtype=out_dtype, device=residual.device)
+        # rows read their predecessor's old residual: in place only if no row has one in this step
+        x = residual if y is None or seg.max_rows <= 1 else torch.empty_like(residual)
+        native_mixers().add_norm_shift(x, residual, y, wb, w, shift, h, prev_state, seg.start, seg.pos0, seg.slot,
+                                       seg.num, seg.max_rows, eps)
+        return x, h
+    return ref.add_norm_shift_rows(residual, y, wb, w, shift, eps, out_dtype, prev_state, seg)
+
+
 def dual_rms_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch.Tensor, eps: float,
                   scale: float = 0.5) -> torch.Tensor:
     """fp32 scale * (rms_norm(a) * wa + rms_norm(b) * wb) of two rows of equal width: the
@@ -284,56 +303,87 @@ def head_rms_gate(o, w, gate_pre, eps: float, heads: int, dv: int, out_dtype, si
 # ---------------------------------------------------------------------------------
 
 def latent_kv_write(dkv, norm_w, eps: float, table, rot_dims: int, positions, slot_mapping, cache,
-                    rank: int):
-    """Cache row = [rms_norm(dkv[:rank]) * norm_w | rope(dkv[rank:])] at each row's slot."""
+                    rank: int, interleaved: bool = False):
+    """Cache row = [rms_norm(dkv[:rank]) * norm_w | rope(dkv[rank:])] at each row's slot
+    (rotary pairs (i, i + rot_dims/2), or (2i, 2i + 1) if ``interleaved``)."""
     if dkv.is_cuda:
         native_mixers().latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping,
-                                        cache, rank)
+                                        cache, rank, bool(interleaved), None, None, None)
     else:
-        ref.latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank)
+        ref.latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank, interleaved)
 
 
-def latent_q_rope(q, table, rot_dims: int, positions, heads: int, dn: int, dr: int):
-    """q rows [heads x (dn unrotated | dr rotated)] -> fp32 ([T, heads, dn], [T, heads, dr] rotated)."""
+def latent_down_prep(dq, q_norm_w, dkv, norm_w, eps: float, table, rot_dims: int, positions, slot_mapping, cache,
+                     rank: int, interleaved: bool = False):
+    """:func:`latent_kv_write` of ``dkv`` and the queries' latent in one launch: returns
+    rms_norm(dq) * q_norm_w in dq's dtype.  ``dq`` and ``dkv`` are adjacent column ranges
+    [q latent | kv latent | rotated part] of one product."""
+    if dkv.is_cuda:
+        cq = torch.empty(dq.shape, dtype=dq.dtype, device=dq.device)
+        native_mixers().latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank,
+                                        bool(interleaved), cq, dq, q_norm_w)
+        return cq
+    return ref.latent_down_prep(dq, q_norm_w, dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank,
+                                interleaved)
+
+
+def latent_q_rope(q, table, rot_dims: int, positions, heads: int, dn: int, dr: int, interleaved: bool = False):
+    """q rows [heads x (dn unrotated | dr rotated)] -> fp32 ([T, heads, dn], [T, heads, dr]
+    rotated: entry i paired with i + rot_dims/2, or 2i with 2i + 1 if ``interleaved``)."""
     if q.is_cuda:
         t = q.shape[0]
         qn = torch.empty(t, heads, dn, dtype=torch.float32, device=q.device)
         qr = torch.empty(t, heads, dr, dtype=torch.float32, device=q.device)
-        native_mixers().latent_q_rope(qn, qr, q, table, rot_dims, positions, heads, dn, dr)
+        native_mixers().latent_q_rope(qn, qr, q, table, rot_dims, positions, heads, dn, dr, bool(interleaved))
         return qn, qr
-    return ref.latent_q_rope(q, table, rot_dims, positions, heads, dn, dr)
+    return ref.latent_q_rope(q, table, rot_dims, positions, heads, dn, dr, interleaved)
 
 
 def latent_attention(qa, qr, cache, seg: Segments, scale: float, rank: int,
-                     skip_from: int = 0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     skip_from: int = 0, out: Optional[torch.Tensor] = None,
+                     sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention over the paged latent cache.  ``qa`` fp32 [heads, T,
     rank]: the unrotated query parts carried into latent space (q W_uk); ``qr`` fp32
     [T, heads, dr]: the rotated parts.  Score = (qa . c + qr . k_rot) * scale; all heads
     share the cached row, whose first ``rank`` entries are also the value.  Returns
     fp32 [heads, T, rank].  ``skip_from`` > 0: segments of that many rows or more are
-    left to the caller (:func:`latent_attention_products`)."""
+    left to the caller (:func:`latent_attention_products`).  ``sink`` fp32 [heads]: the
+    softmax's denominator gains exp(sink[h]), as a key with that score and no value."""
     if qa.is_cuda:
         if out is None:
             out = torch.empty_like(qa)
         native_mixers().latent_attention(out, qa, qr, cache, seg.start, seg.pos0, seg.kv_len,
                                          seg.block_tables, seg.num, seg.max_rows, scale, rank,
-                                         skip_from, seg.max_kv)
+                                         skip_from, seg.max_kv, sink)
         return out
-    r = ref.latent_attention(qa, qr, cache, seg, scale, rank)
+    r = ref.latent_attention(qa, qr, cache, seg, scale, rank, sink)
     if out is not None:
         out.copy_(r)
         return out
     return r
 
 
-def causal_softmax(s, rows_per_head: int, first_pos: int, scale: float, out_dtype):
+def causal_softmax(s, rows_per_head: int, first_pos: int, scale: float, out_dtype,
+                   sink: Optional[torch.Tensor] = None):
     """P = softmax(scale * S) per row over the keys j <= first_pos + (row mod
-    rows_per_head), zeros beyond; S fp32 [heads * rows_per_head, keys]."""
+    rows_per_head), zeros beyond; S fp32 [heads * rows_per_head, keys].  ``sink`` fp32
+    [heads]: exp(sink[head]) joins the denominator."""
     if s.is_cuda:
         p = torch.empty(s.shape, dtype=out_dtype, device=s.device)
-        native_mixers().causal_softmax(p, s, rows_per_head, first_pos, scale)
+        native_mixers().causal_softmax(p, s, rows_per_head, first_pos, scale, sink)
         return p
-    return ref.causal_softmax(s, rows_per_head, first_pos, scale, out_dtype)
+    return ref.causal_softmax(s, rows_per_head, first_pos, scale, out_dtype, sink)
+
+
+def head_gate(o, gate, out_dtype) -> torch.Tensor:
+    """o fp32 [heads, T, dv] times sigmoid(gate[t, h]), one number per row and head, as rows
+    [T, heads*dv] in ``out_dtype``; ``gate`` [T, heads] may be a column range."""
+    if o.is_cuda:
+        heads, t, dv = o.shape
+        out = torch.empty(t, heads * dv, dtype=out_dtype, device=o.device)
+        native_mixers().head_gate(out, o, gate)
+        return out
+    return ref.head_gate(o, gate, out_dtype)
 
 
 _MM_F32_OUT = {}
@@ -360,7 +410,7 @@ PRODUCT_SCORE_BYTES = 1 << 30
 
 
 def latent_attention_products(out, qa, qr, cache, seg: Segments, scale: float, rank: int,
-                              min_rows: int, dtype):
+                              min_rows: int, dtype, sink: Optional[torch.Tensor] = None):
     """Segments of ``min_rows`` rows or more as two matrix products: all heads share
     the cached rows, so with M = heads x rows the scores are Q [M, rank+dr] C^T and the
     sums P [M, keys] C[:, :rank], with a causal softmax (fp32 statistics) in between.
@@ -383,7 +433,7 @@ def latent_attention_products(out, qa, qr, cache, seg: Segments, scale: float, r
             q = torch.cat([qa[:, a + c0:a + c1], qr[a + c0:a + c1].transpose(0, 1)], -1) \
                 .reshape(heads * (c1 - c0), width).to(dtype)
             sc = mm_f32(q, kv[:keys].t())
-            p = causal_softmax(sc, c1 - c0, pos0[s] + c0, scale, dtype)
+            p = causal_softmax(sc, c1 - c0, pos0[s] + c0, scale, dtype, sink)
             out[:, a + c0:a + c1] = mm_f32(p, kv[:keys, :rank]).view(heads, c1 - c0, rank)
     return out
 
@@ -611,6 +661,135 @@ def diff_combine(a, gate, lam: float, post_scale: float, eps: float, heads: int,
 
 
 # ---------------------------------------------------------------------------------
+# attention whose scores are mixed across the heads (paged key cache + paged value cache)
+# ---------------------------------------------------------------------------------
+
+@dataclasses.dataclass
+class TalkSpec:
+    """Constants of an attention that mixes scores across its heads before the softmax.
+    Query head h reads key and value head floor(h / (heads / kv_heads)).  Position i sees
+    j iff 0 <= i - j < window (window 0: every earlier key) or j < keep_first (<= i).
+    With dot products s_g = q_g.k (queries come scaled): s_g <- softcap tanh(s_g /
+    softcap) (softcap 0: as they are), z_h = sum_g talk[h, g] s_g, weights = softmax of
+    z_h over the visible keys."""
+    heads: int
+    kv_heads: int
+    dk: int
+    dv: int
+    window: int
+    keep_first: int
+    softcap: float
+    talk: torch.Tensor          # fp32 [heads, heads]
+
+
+def rot_norm_prep(qk, nq: int, nk: int, head_dim: int, table, rot_dims: int, eps: float, q_scale, positions,
+                  slot_mapping, k_cache, v_cache, interleaved: bool = False) -> torch.Tensor:
+    """Rows [q (nq) | k (nk) | ...] of a fused projection, head by head (``head_dim``
+    entries): rotary positions on the first ``rot_dims`` entries (``table`` =
+    :func:`rope_table`; None: no rotation), then the head divided by its root mean square.
+    Queries are also multiplied by ``q_scale`` fp32 [q heads] and returned in fp32 [T,
+    nq]; keys go to the rows' key-cache slots, and the k rows as projected (neither rotated
+    nor normed) to the value-cache slots."""
+    if qk.is_cuda:
+        q = torch.empty(qk.shape[0], nq, dtype=torch.float32, device=qk.device)
+        native_mixers().rot_norm_prep(q, qk, nq, nk, head_dim, table, rot_dims, bool(interleaved), eps, q_scale,
+                                      positions, slot_mapping, k_cache, v_cache)
+        return q
+    return ref.rot_norm_prep(qk, nq, nk, head_dim, table, rot_dims, interleaved, eps, q_scale, positions,
+                             slot_mapping, k_cache, v_cache)
+
+
+def talk_attention(out, q, gate, k_cache, v_cache, seg: Segments, spec: TalkSpec, skip_from: int = 0):
+    """q fp32 [T, heads*dk] against the paged caches; writes ``out`` [T, heads*dv] (the
+    weighted sums, times sigmoid(gate) element by element when ``gate`` [T, heads*dv] is
+    given).  ``skip_from`` > 0: segments of that many rows or more are left to the caller
+    (:func:`talk_attention_products`)."""
+    sp = spec
+    if q.is_cuda:
+        native_mixers().talk_attention(out, q, gate, k_cache, v_cache, seg.start, seg.pos0, seg.kv_len,
+                                       seg.block_tables, seg.num, seg.max_rows, sp.heads, sp.kv_heads, sp.dk, sp.dv,
+                                       sp.window, sp.keep_first, float(sp.softcap), sp.talk, skip_from, seg.max_kv)
+        return out
+    r = ref.talk_attention(q, k_cache, v_cache, seg, sp.heads, sp.kv_heads, sp.dk, sp.dv, sp.window, sp.keep_first,
+                           sp.softcap, sp.talk)
+    out.copy_(r if gate is None else ref.sigmoid_gate(r, gate, out.dtype))
+    return out
+
+
+def talk_weights(s, first_pos: int, key0: int, ext: int, spec: TalkSpec):
+    """Dot products fp32 [heads, rows, keys] -> unnormalised weights exp(z - max) in place
+    (zeros where a key is not visible) and the reciprocals of their row sums, fp32 [heads,
+    rows]; row r is position first_pos + r, the first ``ext`` columns are the positions
+    0 .. ext-1 and column c >= ext is position key0 + c - ext."""
+    sp = spec
+    if s.is_cuda:
+        inv = torch.empty(s.shape[:2], dtype=torch.float32, device=s.device)
+        native_mixers().talk_weights(s, inv, first_pos, key0, ext, sp.window, sp.keep_first, float(sp.softcap),
+                                     sp.talk)
+        return inv
+    s.copy_(ref.talk_weights(s, s.shape[1], first_pos, key0, ext, sp.window, sp.keep_first, sp.softcap, sp.talk))
+    return torch.ones(s.shape[:2], dtype=torch.float32, device=s.device)
+
+
+def scaled_heads_gate(out, o, inv, gate):
+    """out rows [T, heads*dv] = o [heads, T, dv] * inv [heads, T] (* sigmoid(gate [T, heads*dv]))."""
+    if o.is_cuda:
+        native_mixers().scaled_heads_gate(out, o, inv, gate)
+        return out
+    heads, t, dv = o.shape
+    r = (o * inv[:, :, None]).transpose(0, 1).reshape(t, heads * dv)
+    out.copy_(r if gate is None else ref.sigmoid_gate(r, gate, out.dtype))
+    return out
+
+
+def talk_attention_products(out, q, gate, k_cache, v_cache, seg: Segments, spec: TalkSpec, min_rows: int):
+    """Segments of ``min_rows`` rows or more as banded matrix products in fp32 (see
+    :func:`window_attention_products`), with :func:`talk_weights` between the two and the
+    normalisation and gate in the step that puts the heads back into rows.  Needs the
+    segments' host copies; writes its rows of ``out``."""
+    sp = spec
+    start, pos0, kv_len = seg.host
+    bs = k_cache.shape[1]
+    rep = sp.heads // sp.kv_heads
+    for s in range(seg.num):
+        a, b = start[s], start[s + 1]
+        n = b - a
+        if n < min_rows:
+            continue
+        step = PRODUCT_FULL_CHUNK_ROWS if sp.window <= 0 else max(PRODUCT_CHUNK_ROWS, min(sp.window, 1024))
+        span = sp.window + sp.keep_first if sp.window > 0 else kv_len[s]
+        while step > 32 and 4 * sp.heads * step * (step + span) > PRODUCT_SCORE_BYTES:
+            step //= 2
+        for c0 in range(0, n, step):
+            c1 = min(n, c0 + step)
+            rows = c1 - c0
+            i0 = pos0[s] + c0
+            lo = ref.mask_first_key(i0, sp.window, False)
+            ext = min(sp.keep_first, lo) if sp.window > 0 else 0
+            hi = min(kv_len[s], pos0[s] + c1)
+            k = _band_rows(k_cache, seg.block_tables[s], lo, hi, ext, bs).view(-1, sp.kv_heads, sp.dk)
+            v = _band_rows(v_cache, seg.block_tables[s], lo, hi, ext, bs).view(-1, sp.kv_heads, sp.dv)
+            # q rows [rows, (g, r), dk] -> [g, (r, rows), dk]
+            qc = q[a + c0:a + c1].view(rows, sp.kv_heads, rep, sp.dk).permute(1, 2, 0, 3) \
+                .reshape(sp.kv_heads, rep * rows, sp.dk)
+            sc = torch.bmm(qc, k.permute(1, 2, 0)).view(sp.heads, rows, -1)
+            inv = talk_weights(sc, i0, lo, ext, sp)
+            o = torch.bmm(sc.view(sp.kv_heads, rep * rows, -1), v.transpose(0, 1)).view(sp.heads, rows, sp.dv)
+            scaled_heads_gate(out[a + c0:a + c1], o, inv, None if gate is None else gate[a + c0:a + c1])
+    return out
+
+
+def _band_rows(cache, table, lo: int, hi: int, ext: int, bs: int):
+    """Cached rows (fp32) of positions 0 .. ext-1 followed by lo .. hi-1."""
+    b0, b1 = lo // bs, (hi + bs - 1) // bs
+    r = cache.index_select(0, table[b0:b1].long()).view((b1 - b0) * bs, -1)[lo - b0 * bs:hi - b0 * bs].float()
+    if ext:
+        e = cache.index_select(0, table[:(ext + bs - 1) // bs].long()).view(-1, r.shape[1])[:ext].float()
+        r = torch.cat([e, r], 0)
+    return r
+
+
+# ---------------------------------------------------------------------------------
 # mixture of experts
 # ---------------------------------------------------------------------------------
 
@@ -634,30 +813,48 @@ def moe_top_logits(z, top: int):
         t = z.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=z.device)
         wts = torch.empty(t, top, dtype=torch.float32, device=z.device)
-        native_mixers().moe_top_logits(idx, wts, z, top)
+        native_mixers().moe_top_logits(idx, wts, z, top, False, 1.0)
         return idx, wts
     return ref.moe_top_logits(z, top)
 
 
-def moe_route_top_logits(h, router, bias, top: int):
-    """:func:`moe_top_logits` of z = router h + bias (fp32 router [E, width] and bias, h fp32
+def moe_top_sigmoid(z, top: int, scale: float):
+    """Router: the ``top`` largest logits of each fp32 row (ties to the lower index); the
+    weights are the chosen ones' sigmoids divided by the sum of those, times ``scale``."""
+    if z.is_cuda:
+        t = z.shape[0]
+        idx = torch.empty(t, top, dtype=torch.int32, device=z.device)
+        wts = torch.empty(t, top, dtype=torch.float32, device=z.device)
+        native_mixers().moe_top_logits(idx, wts, z, top, True, float(scale))
+        return idx, wts
+    return ref.moe_top_sigmoid(z, top, scale)
+
+
+def moe_route_top_logits(h, router, bias, top: int, sigmoid: bool = False, scale: float = 1.0):
+    """:func:`moe_top_logits` (or, ``sigmoid``, :func:`moe_top_sigmoid` with ``scale``) of z = router h + bias (fp32 router [E, width] and bias, h fp32
     or bf16, fp32 accumulation) in one launch: the router of few rows (decode steps)."""
     if h.is_cuda:
         t = h.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=h.device)
         wts = torch.empty(t, top, dtype=torch.float32, device=h.device)
-        native_mixers().moe_route_top_logits(idx, wts, h, router, bias, top)
+        native_mixers().moe_route_top_logits(idx, wts, h, router, bias, top, bool(sigmoid), float(scale))
         return idx, wts
-    return ref.moe_top_logits(torch.nn.functional.linear(h.float(), router, bias), top)
+    z = torch.nn.functional.linear(h.float(), router, bias)
+    return ref.moe_top_sigmoid(z, top, scale) if sigmoid else ref.moe_top_logits(z, top)
+
+
+# first matrix and activation of an expert: the code the kernels take
+EXPERT_ACTS = {"clamp_glu": 0, "relu_sq": 1, "silu_glu": 2}
 
 
 def moe_pairs(out, h, idx, wts, wgu, wdown, limit: float = 0.0, act: str = "clamp_glu"):
     """Few rows (decode): out (fp32, in place) += sum_k wts[:, k] * expert_{idx[:, k]}(h),
     every (row, expert) pair streaming its expert's first matrix ([gate | up] with the
-    clamped GLU, ``act`` "clamp_glu"; or up alone with relu(.)^2, ``act`` "relu_sq") and
+    clamped GLU, ``act`` "clamp_glu", or with silu(gate) * up, "silu_glu"; or up alone with
+    relu(.)^2, "relu_sq") and
     its down matrix; no host round trip, so the step can be captured in a hipGraph."""
     if out.is_cuda:
-        native_mixers().moe_pairs(out, h, idx, wts, wgu, wdown, float(limit), act == "relu_sq")
+        native_mixers().moe_pairs(out, h, idx, wts, wgu, wdown, float(limit), EXPERT_ACTS[act])
     else:
         ref.moe_pairs(out, h, idx, wts, wgu, wdown, limit, act)
 
@@ -672,22 +869,25 @@ def clamp_swiglu(gu, limit: float):
     return ref.clamp_swiglu(gu, limit)
 
 
+def _act_glu(gu, code: int):
+    out = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
+    native_mixers().act_glu(out, gu, code)
+    return out
+
+
 def gelu_glu(gu):
     """[gate | up] rows -> gelu_tanh(gate) * up."""
-    if gu.is_cuda:
-        out = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
-        native_mixers().gelu_glu(out, gu, False)
-        return out
-    return ref.gelu_glu(gu)
+    return _act_glu(gu, 0) if gu.is_cuda else ref.gelu_glu(gu)
 
 
 def relu_glu(gu):
     """[gate | up] rows -> relu(gate) * up."""
-    if gu.is_cuda:
-        out = torch.empty(gu.shape[0], gu.shape[1] // 2, dtype=gu.dtype, device=gu.device)
-        native_mixers().gelu_glu(out, gu, True)
-        return out
-    return ref.relu_glu(gu)
+    return _act_glu(gu, 1) if gu.is_cuda else ref.relu_glu(gu)
+
+
+def silu_glu(gu):
+    """[gate | up] rows -> silu(gate) * up."""
+    return _act_glu(gu, 2) if gu.is_cuda else ref.silu_glu(gu)
 
 
 def relu_sq(x):

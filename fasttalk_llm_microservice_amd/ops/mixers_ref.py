@@ -85,6 +85,23 @@ def add_scaled_rms_norm_rows(residual, y1, y2, mult, next_w, eps, out_dtype):
     return (_rms(residual, eps) * next_w.float()).to(out_dtype) if next_w is not None else None
 
 
+def add_norm_shift_rows(residual, y, wb, w, shift, eps, out_dtype, prev_state, seg):
+    x = residual if y is None else residual + _rms(y.float(), eps) * wb.float()
+    h = _rms(x, eps) * w.float()
+    prev = torch.zeros_like(h)
+    prev[1:] = h[:-1]
+    start = seg.start.tolist()
+    for s in range(seg.num):
+        a, b = start[s], start[s + 1]
+        slot = int(seg.slot[s])
+        if b == a:
+            continue
+        prev[a] = prev_state[slot] if int(seg.pos0[s]) > 0 and slot >= 0 else 0.0
+        if slot >= 0:
+            prev_state[slot] = h[b - 1]
+    return x, (h + (prev - h) * shift.float()).to(out_dtype)
+
+
 def dual_rms_mean(a, b, wa, wb, eps, scale):
     return scale * (_rms(a.float(), eps) * wa.float() + _rms(b.float(), eps) * wb.float())
 
@@ -176,10 +193,15 @@ def distance_bias_table(rel, reach: int):
     return rel.float()[torch.tensor(idx, dtype=torch.long, device=rel.device)].contiguous()
 
 
-def _rope(x, cs, dims):
-    """x [..., T, n] fp32 with cs [T, dims]; rotates the first ``dims`` of n."""
+def _rope(x, cs, dims, interleaved=False):
+    """x [..., T, n] fp32 with cs [T, dims]; rotates the first ``dims`` of n, entry i
+    paired with i + dims/2, or (``interleaved``) entry 2i with 2i + 1."""
     half = dims // 2
     cos, sin = cs[:, :half], cs[:, half:]
+    if interleaved:
+        u, v = x[..., 0:dims:2], x[..., 1:dims:2]
+        r = torch.stack([u * cos - v * sin, v * cos + u * sin], -1).flatten(-2)
+        return torch.cat([r, x[..., dims:]], -1)
     u, v = x[..., :half], x[..., half:dims]
     return torch.cat([u * cos - v * sin, v * cos + u * sin, x[..., dims:]], -1)
 
@@ -268,13 +290,19 @@ def head_rms_gate(o, w, gate_pre, eps, heads, dv, out_dtype, silu=False):
     return y.view(t, heads * dv).to(out_dtype)
 
 
-def latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank):
+def latent_down_prep(dq, q_norm_w, dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank,
+                     interleaved):
+    latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank, interleaved)
+    return (_rms(dq.float(), eps) * q_norm_w.float()).to(dq.dtype)
+
+
+def latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, cache, rank, interleaved=False):
     t = dkv.shape[0]
     if t == 0:
         return
     x = dkv.float()
     c = _rms(x[:, :rank], eps) * norm_w.float()
-    kr = _rope(x[:, rank:], table[positions.long()], rot_dims)
+    kr = _rope(x[:, rank:], table[positions[:t].long()], rot_dims, interleaved)
     row = torch.cat([c, kr], -1).to(cache.dtype)
     slots = slot_mapping[:t].long()
     keep = slots >= 0
@@ -282,15 +310,26 @@ def latent_kv_write(dkv, norm_w, eps, table, rot_dims, positions, slot_mapping, 
         cache.view(-1, cache.shape[-1])[slots[keep]] = row[keep]
 
 
-def latent_q_rope(q, table, rot_dims, positions, heads, dn, dr):
+def latent_q_rope(q, table, rot_dims, positions, heads, dn, dr, interleaved=False):
     """q [T, heads*(dn+dr)] -> (q_unrotated fp32 [T, heads, dn], q_rotated fp32 [T, heads, dr])."""
     t = q.shape[0]
     x = q.float().view(t, heads, dn + dr)
-    cs = table[positions.long()]
-    return x[..., :dn].contiguous(), _rope(x[..., dn:].transpose(0, 1), cs, rot_dims).transpose(0, 1).contiguous()
+    cs = table[positions[:t].long()]
+    return x[..., :dn].contiguous(), \
+        _rope(x[..., dn:].transpose(0, 1), cs, rot_dims, interleaved).transpose(0, 1).contiguous()
 
 
-def latent_attention(qa, qr, cache, seg, scale, rank):
+def _softmax_sink(z, sink):
+    """softmax over the last axis of z [heads, ...]; exp(sink[head]) joins the denominator."""
+    if sink is None:
+        return torch.softmax(z, -1)
+    sk = sink.float().view(-1, *([1] * (z.dim() - 1)))
+    m = torch.maximum(z.max(-1, keepdim=True).values, sk)
+    e = torch.exp(z - m)
+    return e / (e.sum(-1, keepdim=True) + torch.exp(sk - m))
+
+
+def latent_attention(qa, qr, cache, seg, scale, rank, sink=None):
     """qa fp32 [heads, T, rank] (queries in latent space) and qr fp32 [T, heads, dr]
     (rotated part) against cache rows [c (rank) | rotated key (dr)]; returns the
     softmax-weighted sums of the c rows, fp32 [heads, T, rank]."""
@@ -310,17 +349,24 @@ def latent_attention(qa, qr, cache, seg, scale, rank):
         qpos = int(seg.pos0[s]) + torch.arange(b - a, device=qa.device)
         mask = torch.arange(n, device=qa.device)[None, :] <= qpos[:, None]
         sc = sc.masked_fill(~mask[None], float("-inf"))
-        p = torch.softmax(sc, -1)
+        p = _softmax_sink(sc, sink)
         out[:, a:b] = torch.einsum("htj,jr->htr", p, kv[:, :rank])
     return out
 
 
-def causal_softmax(s, rows_per_head, first_pos, scale, out_dtype):
+def causal_softmax(s, rows_per_head, first_pos, scale, out_dtype, sink=None):
     rows, keys = s.shape
     qpos = first_pos + torch.arange(rows, device=s.device) % rows_per_head
     mask = torch.arange(keys, device=s.device)[None, :] <= qpos[:, None]
-    p = torch.softmax((s.float() * scale).masked_fill(~mask, float("-inf")), -1)
+    z = (s.float() * scale).masked_fill(~mask, float("-inf"))
+    p = _softmax_sink(z.view(-1, rows_per_head, keys), sink).view(rows, keys)
     return p.masked_fill(~mask, 0.0).to(out_dtype)
+
+
+def head_gate(o, gate, out_dtype):
+    heads, t, dv = o.shape
+    y = o * torch.sigmoid(gate.float()).t()[:, :, None]
+    return y.transpose(0, 1).reshape(t, heads * dv).to(out_dtype)
 
 
 def moe_topk(z, correction, top, groups, keep):
@@ -343,12 +389,20 @@ def moe_top_logits(z, top):
     return idx[:, :top].int(), torch.softmax(val[:, :top], -1)
 
 
+def moe_top_sigmoid(z, top, scale):
+    """The ``top`` largest logits per row (ties to the lower index); weights are their
+    sigmoids divided by the sum of those, times ``scale``."""
+    val, idx = torch.sort(z.float(), dim=-1, descending=True, stable=True)
+    s = torch.sigmoid(val[:, :top])
+    return idx[:, :top].int(), s / (s.sum(-1, keepdim=True) + 1e-20) * scale
+
+
 def moe_pairs(out, h, idx, wts, wgu, wdown, limit, act="clamp_glu"):
     for t in range(h.shape[0]):
         for k in range(idx.shape[1]):
             e = int(idx[t, k])
             u = F.linear(h[t:t + 1], wgu[e])
-            y = clamp_swiglu(u, limit) if act == "clamp_glu" else relu_sq(u)
+            y = clamp_swiglu(u, limit) if act == "clamp_glu" else silu_glu(u) if act == "silu_glu" else relu_sq(u)
             out[t] += wts[t, k] * F.linear(y, wdown[e])[0].float()
 
 
@@ -580,3 +634,73 @@ def relu_glu(gu):
 def gelu_glu(gu):
     ff = gu.shape[1] // 2
     return (gelu_tanh(gu[:, :ff].float()) * gu[:, ff:].float()).to(gu.dtype)
+
+
+def silu_glu(gu):
+    ff = gu.shape[1] // 2
+    g = gu[:, :ff].float()
+    return (g * torch.sigmoid(g) * gu[:, ff:].float()).to(gu.dtype)
+
+
+# ---------------------------------------------------------------------------------
+# attention whose scores are mixed across the heads before the softmax
+# ---------------------------------------------------------------------------------
+
+def rot_norm_prep(qk, nq, nk, head_dim, table, rot_dims, interleaved, eps, q_scale, positions, slot_mapping,
+                  k_cache, v_cache):
+    t = qk.shape[0]
+    x = qk[:, :nq + nk].float().reshape(t, -1, head_dim)
+    raw = x[:, nq // head_dim:]
+    if table is not None and rot_dims > 0:
+        cs = table[positions[:t].long()]
+        x = _rope(x.transpose(0, 1), cs, rot_dims, interleaved).transpose(0, 1)
+    x = _rms(x, eps)
+    q = x[:, :nq // head_dim] * q_scale.float()[None, :, None]
+    slots = slot_mapping[:t].long()
+    keep = slots >= 0
+    if keep.any():
+        k_cache.view(-1, nk)[slots[keep]] = x[:, nq // head_dim:].reshape(t, nk)[keep].to(k_cache.dtype)
+        v_cache.view(-1, nk)[slots[keep]] = raw.reshape(t, nk)[keep].to(v_cache.dtype)
+    return q.reshape(t, nq).contiguous()
+
+
+def talk_weights(s, rows, first_pos, key0, ext, window, keep_first, softcap, talk):
+    """s fp32 [heads, rows, keys] scaled dot products -> weights, columns as in
+    :func:`band_weights`."""
+    heads, _, keys = s.shape
+    col = torch.arange(keys, device=s.device)
+    jpos = torch.where(col < ext, col, key0 + col - ext)
+    dist = first_pos + torch.arange(rows, device=s.device)[:, None] - jpos[None, :]
+    vis = dist >= 0
+    if window > 0:
+        vis = vis & ((dist < window) | (jpos[None, :] < keep_first))
+    z = softcap * torch.tanh(s / softcap) if softcap else s
+    z = torch.einsum("hg,gij->hij", talk.float(), z)
+    return torch.softmax(z.masked_fill(~vis[None], float("-inf")), -1)
+
+
+def talk_attention(q, k_cache, v_cache, seg, heads, kv_heads, dk, dv, window, keep_first, softcap, talk):
+    """q fp32 [T, heads*dk] (already scaled) -> fp32 [T, heads*dv]."""
+    t = q.shape[0]
+    rep = heads // kv_heads
+    out = torch.zeros(t, heads, dv, dtype=torch.float32, device=q.device)
+    bs = k_cache.shape[1]
+    start = seg.start.tolist()
+    kvh = torch.arange(heads) // rep
+    for s in range(seg.num):
+        a, b = start[s], start[s + 1]
+        n = int(seg.kv_len[s])
+        if b == a or n == 0:
+            continue
+        p0 = int(seg.pos0[s])
+        lo = mask_first_key(p0, window, False)
+        ext = min(keep_first, lo) if window > 0 else 0
+        nblk = (n + bs - 1) // bs
+        pages = seg.block_tables[s, :nblk].long()
+        keys = torch.cat([torch.arange(ext), torch.arange(lo, n)]).to(k_cache.device)
+        k = k_cache[pages].reshape(nblk * bs, -1)[keys].float().view(keys.numel(), kv_heads, dk)
+        v = v_cache[pages].reshape(nblk * bs, -1)[keys].float().view(keys.numel(), kv_heads, dv)
+        sc = torch.einsum("thd,jhd->htj", q[a:b].view(b - a, heads, dk), k[:, kvh])
+        w = talk_weights(sc, b - a, p0, lo, ext, window, keep_first, softcap, talk)
+        out[a:b] = torch.einsum("htj,jhd->thd", w, v[:, kvh])
+    return out.view(t, heads * dv)
