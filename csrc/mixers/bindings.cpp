@@ -25,10 +25,31 @@ int mx_conv_attn_prep(float* q_out, const void* qkv, int bf16, long stride, int 
                       int num_segs, int num_state_slots, const float* wq, const float* wk, float eps, int head_dim,
                       const int* slots, void* k_cache, void* v_cache, int cache_bf16, long num_slots, long rows,
                       hipStream_t s);
-int mx_moe_top_logits(int* idx, float* wts, const float* z, long rows, int experts, int top, hipStream_t s);
+int mx_moe_top_logits(int* idx, float* wts, const float* z, long rows, int experts, int top, int sigmoid,
+                      float scale, hipStream_t s);
 int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int bf16, long h_stride, const float* router,
-                            const float* bias, long rows, int experts, int width, int top, hipStream_t s);
-int mx_gelu_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int relu, hipStream_t s);
+                            const float* bias, long rows, int experts, int width, int top, int sigmoid, float scale,
+                            hipStream_t s);
+int mx_act_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int act, hipStream_t s);
+int mx_shift_max_width();
+int mx_add_norm_shift(float* x_out, const float* x_in, const void* y, int y_bf16, long y_stride, const float* wb,
+                      const float* w, const float* shift, void* out, int out_bf16, float* state, int num_slots,
+                      const int* start, const int* pos0, const int* slot, int num_segs, int max_rows, int rows,
+                      int width, float eps, hipStream_t s);
+int mx_rot_norm_prep(float* q_out, const void* qk, int bf16, long stride, int q_heads, int k_heads, int head_dim,
+                     const float* table, int table_rows, int rot_dims, int interleaved, float eps,
+                     const float* q_scale, const int* positions, const int* slots, void* k_cache, void* v_cache,
+                     long num_slots, long rows, hipStream_t s);
+int mx_talk_max_heads();
+int mx_talk_attention(void* out, int out_bf16, float* ws_acc, float* ws_ml, const float* q, const void* gate,
+                      long gate_stride, const void* k_cache, const void* v_cache, int cache_bf16, const int* start,
+                      const int* pos0, const int* kv_len, const int* bt, int bt_stride, int num_segs, long total_rows,
+                      int heads, int kv_heads, int dk, int dv, int window, int keep_first, float softcap,
+                      const float* talk, int block_size, int num_blocks, int skip_from, int splits, hipStream_t s);
+int mx_talk_weights(float* S, float* inv, int heads, int rows, int keys, int first_pos, int key0, int ext, int window,
+                    int keep_first, float softcap, const float* talk, hipStream_t s);
+int mx_heads_to_rows(void* out, int out_bf16, const float* o, const float* inv, const void* gate, long gate_stride,
+                     int per_head, long rows, int heads, int dv, hipStream_t s);
 int mx_gla_max_dk();
 int mx_gla_scan(float* o, const void* qkv, int bf16, long qkv_stride, const void* a, long a_stride,
                 const float* a_bias, float tau, float* state, const int* start, const int* pos0, const int* slot,
@@ -92,26 +113,28 @@ int mx_delta_rule(float* o, const float* qn, const float* kn, const float* g, co
                   hipStream_t s);
 int mx_latent_kv_write(const void* dkv, int bf16, long stride, const float* w, float eps, const float* table,
                        int table_rows, int dims, const int* positions, const int* slots, void* cache,
-                       int cache_bf16, long num_slots, long rows, int rank, int dr, hipStream_t s);
+                       int cache_bf16, long num_slots, long rows, int rank, int dr, int interleaved,
+                       const void* xq, const float* wq, void* cq, int q_rank, hipStream_t s);
 int mx_latent_q_rope(float* qn, float* qr, const void* q, int bf16, long stride, const float* table,
                      int table_rows, int dims, const int* positions, long rows, int heads, int dn, int dr,
-                     hipStream_t s);
+                     int interleaved, hipStream_t s);
 int mx_latent_max_rank();
 int mx_latent_attention(float* out, const float* qa, const float* qr, const void* cache, int cache_bf16,
                         const int* start, const int* pos0, const int* kv_len, const int* bt, int bt_stride,
                         int num_segs, int max_rows, int heads, long total_rows, int rank, int dr,
-                        int block_size, int num_blocks, float scale, int skip_from, hipStream_t s);
+                        int block_size, int num_blocks, float scale, int skip_from, const float* sink,
+                        hipStream_t s);
 long mx_latent_split_ws(int heads, int rank, int dr);
 int mx_latent_attention_split(float* out, float* ws_acc, float* ws_ml, const float* qa, const float* qr,
                               const void* cache, int cache_bf16, const int* start, const int* pos0,
                               const int* kv_len, const int* bt, int bt_stride, int num_segs, int max_rows,
                               int heads, long total_rows, int rank, int dr, int block_size, int num_blocks,
-                              float scale, int skip_from, int splits, hipStream_t s);
+                              float scale, int skip_from, int splits, const float* sink, hipStream_t s);
 int mx_causal_softmax(void* P, int p_bf16, const float* S, long rows, int rows_per_head, int first_pos, int ncols,
-                      float scale, hipStream_t s);
+                      float scale, const float* sink, hipStream_t s);
 int mx_moe_pairs(float* out, void* y, const void* h, int bf16, long h_stride, const int* idx, const float* wts,
                  const void* wgu, const void* wdown, long rows, int top, int experts, int ff, int width,
-                 float limit, int relu_sq, hipStream_t s);
+                 float limit, int act, hipStream_t s);
 int mx_moe_topk(int* idx, float* wts, const float* z, const float* corr, long rows, int experts, int top,
                 int groups, int keep, hipStream_t s);
 }
@@ -477,7 +500,7 @@ void sigmoid_gate(Tensor out, Tensor o, Tensor g) {
 }
 
 void latent_kv_write(Tensor dkv, Tensor w, double eps, Tensor table, int64_t dims, Tensor positions,
-                     Tensor slots, Tensor cache, int64_t rank) {
+                     Tensor slots, Tensor cache, int64_t rank, bool interleaved, OptT cq, OptT dq, OptT wq) {
   check_rows(dkv, "dkv");
   check_f32(w, "norm_w");
   check_f32(table, "rope table");
@@ -488,14 +511,28 @@ void latent_kv_write(Tensor dkv, Tensor w, double eps, Tensor table, int64_t dim
               table.size(1) == dims && positions.numel() >= t && slots.numel() >= t, "latent_kv_write shapes");
   TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 3 && cache.size(2) == rank + dr &&
               cache.scalar_type() == dkv.scalar_type(), "cache");
+  // the queries' latent, a column range of the same product (same row stride) ahead of dkv
+  int64_t q_rank = 0;
+  if (cq) {
+    TORCH_CHECK(dq && wq, "latent_kv_write: the queries' latent needs its rows and weight");
+    check_rows(*dq, "dq");
+    check_f32(*wq, "dq norm");
+    q_rank = dq->size(1);
+    TORCH_CHECK(dq->size(0) == t && dq->scalar_type() == dkv.scalar_type() && wq->numel() == q_rank &&
+                (t <= 1 || dq->stride(0) == dkv.stride(0)) && cq->is_cuda() && cq->is_contiguous() &&
+                cq->scalar_type() == dq->scalar_type() && cq->dim() == 2 && cq->size(0) == t &&
+                cq->size(1) == q_rank, "latent_kv_write: query latent");
+  }
   chk(mx_latent_kv_write(dkv.data_ptr(), bf(dkv), dkv.stride(0), w.data_ptr<float>(), (float)eps,
                          table.data_ptr<float>(), (int)table.size(0), (int)dims, positions.data_ptr<int>(),
                          slots.data_ptr<int>(), cache.data_ptr(), bf(cache), cache.size(0) * cache.size(1), t,
-                         (int)rank, (int)dr, stream()), "latent_kv_write");
+                         (int)rank, (int)dr, interleaved ? 1 : 0, cq ? dq->data_ptr() : nullptr,
+                         cq ? wq->data_ptr<float>() : nullptr, cq ? cq->data_ptr() : nullptr, (int)q_rank, stream()),
+      "latent_kv_write");
 }
 
 void latent_q_rope(Tensor qn, Tensor qr, Tensor q, Tensor table, int64_t dims, Tensor positions, int64_t heads,
-                   int64_t dn, int64_t dr) {
+                   int64_t dn, int64_t dr, bool interleaved) {
   check_f32(qn, "qn");
   check_f32(qr, "qr");
   check_rows(q, "q");
@@ -507,12 +544,13 @@ void latent_q_rope(Tensor qn, Tensor qr, Tensor q, Tensor table, int64_t dims, T
               "latent_q_rope shapes");
   chk(mx_latent_q_rope(qn.data_ptr<float>(), qr.data_ptr<float>(), q.data_ptr(), bf(q), q.stride(0),
                        table.data_ptr<float>(), (int)table.size(0), (int)dims, positions.data_ptr<int>(), t,
-                       (int)heads, (int)dn, (int)dr, stream()), "latent_q_rope");
+                       (int)heads, (int)dn, (int)dr, interleaved ? 1 : 0, stream()), "latent_q_rope");
 }
 
 void latent_attention(Tensor out, Tensor qa, Tensor qr, Tensor cache, Tensor start, Tensor pos0, Tensor kv_len,
                       Tensor bt, int64_t num_segs, int64_t max_rows, double scale, int64_t rank, int64_t skip_from,
-                      int64_t max_kv) {
+                      int64_t max_kv, OptT sink_) {
+  const float* sink = opt_f32(sink_, qa.size(0), "sink");
   check_f32(out, "out");
   check_f32(qa, "qa");
   check_f32(qr, "qr");
@@ -538,23 +576,24 @@ void latent_attention(Tensor out, Tensor qa, Tensor qr, Tensor cache, Tensor sta
                                   start.data_ptr<int>(), pos0.data_ptr<int>(), kv_len.data_ptr<int>(),
                                   bt.data_ptr<int>(), (int)bt.size(1), (int)num_segs, (int)max_rows, (int)heads,
                                   t, (int)rank, (int)dr, (int)cache.size(1), (int)cache.size(0), (float)scale,
-                                  (int)skip_from, (int)splits, stream()), "latent_attention_split");
+                                  (int)skip_from, (int)splits, sink, stream()), "latent_attention_split");
     return;
   }
   chk(mx_latent_attention(out.data_ptr<float>(), qa.data_ptr<float>(), qr.data_ptr<float>(), cache.data_ptr(),
                           bf(cache), start.data_ptr<int>(), pos0.data_ptr<int>(), kv_len.data_ptr<int>(),
                           bt.data_ptr<int>(), (int)bt.size(1), (int)num_segs, (int)max_rows, (int)heads, t,
                           (int)rank, (int)dr, (int)cache.size(1), (int)cache.size(0), (float)scale, (int)skip_from,
-                          stream()),
+                          sink, stream()),
       "latent_attention");
 }
 
-void causal_softmax(Tensor P, Tensor S, int64_t rows_per_head, int64_t first_pos, double scale) {
+void causal_softmax(Tensor P, Tensor S, int64_t rows_per_head, int64_t first_pos, double scale, OptT sink) {
   check_f32(S, "S");
   TORCH_CHECK(S.dim() == 2 && P.is_cuda() && is_act(P) && P.is_contiguous() && P.sizes() == S.sizes() &&
               rows_per_head >= 1 && S.size(0) % rows_per_head == 0 && first_pos >= 0, "causal_softmax shapes");
   chk(mx_causal_softmax(P.data_ptr(), bf(P), S.data_ptr<float>(), S.size(0), (int)rows_per_head, (int)first_pos,
-                        (int)S.size(1), (float)scale, stream()), "causal_softmax");
+                        (int)S.size(1), (float)scale, opt_f32(sink, S.size(0) / rows_per_head, "sink"), stream()),
+      "causal_softmax");
 }
 
 void moe_topk(Tensor idx, Tensor wts, Tensor z, Tensor corr, int64_t top, int64_t groups, int64_t keep) {
@@ -568,17 +607,18 @@ void moe_topk(Tensor idx, Tensor wts, Tensor z, Tensor corr, int64_t top, int64_
                   z.size(0), (int)z.size(1), (int)top, (int)groups, (int)keep, stream()), "moe_topk");
 }
 
-void moe_top_logits(Tensor idx, Tensor wts, Tensor z, int64_t top) {
+void moe_top_logits(Tensor idx, Tensor wts, Tensor z, int64_t top, bool sigmoid, double scale) {
   check_i32(idx, "idx");
   check_f32(wts, "wts");
   check_f32(z, "z");
   TORCH_CHECK(z.dim() == 2 && top >= 1 && top <= z.size(1) && idx.numel() == z.size(0) * top &&
               wts.numel() == z.size(0) * top, "moe_top_logits shapes");
   chk(mx_moe_top_logits(idx.data_ptr<int>(), wts.data_ptr<float>(), z.data_ptr<float>(), z.size(0), (int)z.size(1),
-                        (int)top, stream()), "moe_top_logits");
+                        (int)top, sigmoid ? 1 : 0, (float)scale, stream()), "moe_top_logits");
 }
 
-void moe_route_top_logits(Tensor idx, Tensor wts, Tensor h, Tensor router, OptT bias, int64_t top) {
+void moe_route_top_logits(Tensor idx, Tensor wts, Tensor h, Tensor router, OptT bias, int64_t top,
+                          bool sigmoid, double scale) {
   check_i32(idx, "idx");
   check_f32(wts, "wts");
   check_rows(h, "h");
@@ -591,11 +631,15 @@ void moe_route_top_logits(Tensor idx, Tensor wts, Tensor h, Tensor router, OptT 
   }
   chk(mx_moe_route_top_logits(idx.data_ptr<int>(), wts.data_ptr<float>(), h.data_ptr(), bf(h), h.stride(0),
                               router.data_ptr<float>(), bias ? bias->data_ptr<float>() : nullptr, h.size(0),
-                              (int)router.size(0), (int)router.size(1), (int)top, stream()), "moe_route_top_logits");
+                              (int)router.size(0), (int)router.size(1), (int)top, sigmoid ? 1 : 0, (float)scale,
+                              stream()), "moe_route_top_logits");
 }
 
-// relu_sq: the experts' first matrix is [ff, width] (up alone) instead of [2 ff, width] (gate | up)
-void moe_pairs(Tensor out, Tensor h, Tensor idx, Tensor wts, Tensor wgu, Tensor wdown, double limit, bool relu_sq) {
+// act 0: clamped GLU, 1: relu^2 (the experts' first matrix is [ff, width], up alone, instead of
+// [2 ff, width], gate | up), 2: silu GLU
+void moe_pairs(Tensor out, Tensor h, Tensor idx, Tensor wts, Tensor wgu, Tensor wdown, double limit, int64_t act) {
+  const bool relu_sq = act == 1;
+  TORCH_CHECK(act >= 0 && act <= 2, "moe_pairs: activation");
   check_f32(out, "out");
   check_rows(h, "h");
   check_i32(idx, "idx");
@@ -614,16 +658,17 @@ void moe_pairs(Tensor out, Tensor h, Tensor idx, Tensor wts, Tensor wgu, Tensor 
   Tensor y = at::empty({rows * top, ff}, h.options());
   chk(mx_moe_pairs(out.data_ptr<float>(), y.data_ptr(), h.data_ptr(), bf(h), h.stride(0), idx.data_ptr<int>(),
                    wts.data_ptr<float>(), wgu.data_ptr(), wdown.data_ptr(), rows, (int)top, (int)experts, (int)ff,
-                   (int)width, (float)limit, relu_sq ? 1 : 0, stream()), "moe_pairs");
+                   (int)width, (float)limit, (int)act, stream()), "moe_pairs");
 }
 
-void gelu_glu(Tensor out, Tensor gu, bool relu) {
+void act_glu(Tensor out, Tensor gu, int64_t act) {
   check_rows(gu, "gu");
   const int64_t ff = gu.size(1) / 2;
   TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.scalar_type() == gu.scalar_type() && out.dim() == 2 &&
               out.size(0) == gu.size(0) && out.size(1) == ff && ff >= 1 && gu.size(1) == 2 * ff, "out");
-  chk(mx_gelu_glu(out.data_ptr(), gu.data_ptr(), bf(gu), gu.stride(0), gu.size(0), (int)ff, relu ? 1 : 0, stream()),
-      "gelu_glu");
+  TORCH_CHECK(act >= 0 && act <= 2, "act_glu: activation");
+  chk(mx_act_glu(out.data_ptr(), gu.data_ptr(), bf(gu), gu.stride(0), gu.size(0), (int)ff, (int)act, stream()),
+      "act_glu");
 }
 
 const float* opt_f32(const OptT& t, int64_t n, const char* what) {
@@ -823,6 +868,148 @@ void gate_group_norm(Tensor out, Tensor y, Tensor z, Tensor w, double eps, int64
       "gate_group_norm");
 }
 
+void add_norm_shift(Tensor x_out, Tensor x_in, OptT y, OptT wb, Tensor w, Tensor shift, Tensor out, Tensor state,
+                    Tensor start, Tensor pos0, Tensor slot, int64_t num_segs, int64_t max_rows, double eps) {
+  check_f32(x_in, "residual");
+  check_f32(x_out, "residual out");
+  TORCH_CHECK(x_in.dim() == 2 && x_out.sizes() == x_in.sizes(), "residual 2-D");
+  const int64_t rows = x_in.size(0), width = x_in.size(1);
+  check_f32(w, "norm weight");
+  check_f32(shift, "shift");
+  check_f32(state, "shift state");
+  TORCH_CHECK(w.numel() == width && shift.numel() == width && state.dim() == 2 && state.size(0) >= 1 &&
+              state.size(1) == width && width <= mx_shift_max_width(), "add_norm_shift shapes");
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && is_act(out) && out.sizes() == x_in.sizes(), "out");
+  TORCH_CHECK((bool)y == (bool)wb, "y and its norm weight go together");
+  TORCH_CHECK(max_rows >= 1 && max_rows <= rows + 1, "max_rows");
+  check_segs(start, pos0, slot, num_segs);
+  const void* yp = nullptr;
+  int ybf = 0;
+  long ys = 0;
+  if (y) {
+    check_rows(*y, "y");
+    check_f32(*wb, "post-norm weight");
+    TORCH_CHECK(y->size(0) == rows && y->size(1) == width && wb->numel() == width, "y shape");
+    TORCH_CHECK(max_rows <= 1 || x_out.data_ptr() != x_in.data_ptr(), "segments of several rows need a second buffer");
+    yp = y->data_ptr();
+    ybf = bf(*y);
+    ys = y->stride(0);
+  }
+  chk(mx_add_norm_shift(x_out.data_ptr<float>(), x_in.data_ptr<float>(), yp, ybf, ys,
+                        wb ? wb->data_ptr<float>() : nullptr, w.data_ptr<float>(), shift.data_ptr<float>(),
+                        out.data_ptr(), bf(out), state.data_ptr<float>(), (int)state.size(0), start.data_ptr<int>(),
+                        pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)max_rows, (int)rows,
+                        (int)width, (float)eps, stream()), "add_norm_shift");
+}
+
+void rot_norm_prep(Tensor q, Tensor qk, int64_t nq, int64_t nk, int64_t head_dim, OptT table, int64_t rot_dims,
+                   bool interleaved, double eps, Tensor q_scale, Tensor positions, Tensor slots, Tensor k_cache,
+                   Tensor v_cache) {
+  check_f32(q, "q");
+  check_rows(qk, "qk");
+  check_i32(positions, "positions");
+  check_i32(slots, "slot_mapping");
+  check_f32(q_scale, "q_scale");
+  const int64_t t = qk.size(0);
+  TORCH_CHECK(head_dim >= 1 && head_dim <= 512 && nq >= head_dim && nk >= head_dim && nq % head_dim == 0 &&
+              nk % head_dim == 0 && qk.size(1) >= nq + nk && q.numel() == t * nq && q_scale.numel() * head_dim == nq &&
+              positions.numel() >= t && slots.numel() >= t, "rot_norm_prep shapes");
+  check_cache(k_cache, nk, "k_cache");
+  check_cache(v_cache, nk, "v_cache");
+  TORCH_CHECK(k_cache.scalar_type() == qk.scalar_type() && v_cache.scalar_type() == qk.scalar_type() &&
+              k_cache.size(0) == v_cache.size(0) && k_cache.size(1) == v_cache.size(1), "k / v caches");
+  const float* tp = nullptr;
+  int64_t trows = 0;
+  if (table && rot_dims > 0) {
+    check_f32(*table, "rope table");
+    TORCH_CHECK(table->dim() == 2 && table->size(1) == rot_dims && rot_dims % 2 == 0 && rot_dims <= head_dim,
+                "rope table shape");
+    tp = table->data_ptr<float>();
+    trows = table->size(0);
+  } else {
+    rot_dims = 0;
+  }
+  chk(mx_rot_norm_prep(q.data_ptr<float>(), qk.data_ptr(), bf(qk), qk.stride(0), (int)(nq / head_dim),
+                       (int)(nk / head_dim), (int)head_dim, tp, (int)trows, (int)rot_dims, interleaved ? 1 : 0,
+                       (float)eps, q_scale.data_ptr<float>(), positions.data_ptr<int>(), slots.data_ptr<int>(),
+                       k_cache.data_ptr(), v_cache.data_ptr(), k_cache.size(0) * k_cache.size(1), t, stream()),
+      "rot_norm_prep");
+}
+
+// gate rows beside `out` rows: same dtype as out
+const void* gate_rows(const OptT& gate, const Tensor& out, int64_t rows, int64_t cols, long* stride) {
+  *stride = 0;
+  if (!gate) return nullptr;
+  check_rows(*gate, "gate");
+  TORCH_CHECK(gate->size(0) == rows && gate->size(1) == cols && gate->scalar_type() == out.scalar_type(), "gate rows");
+  *stride = gate->stride(0);
+  return gate->data_ptr();
+}
+
+void talk_attention(Tensor out, Tensor q, OptT gate, Tensor k_cache, Tensor v_cache, Tensor start, Tensor pos0,
+                    Tensor kv_len, Tensor bt, int64_t num_segs, int64_t max_rows, int64_t heads, int64_t kv_heads,
+                    int64_t dk, int64_t dv, int64_t window, int64_t keep_first, double softcap, Tensor talk,
+                    int64_t skip_from, int64_t max_kv) {
+  check_f32(q, "q");
+  check_f32(talk, "head mix");
+  TORCH_CHECK(heads >= 1 && heads <= mx_talk_max_heads() && kv_heads >= 1 && heads % kv_heads == 0 && dk >= 1 &&
+              dv >= 1 && dv <= 512 && keep_first >= 0 && talk.numel() == heads * heads, "talk_attention sizes");
+  const int64_t t = q.size(0);
+  TORCH_CHECK(q.dim() == 2 && q.size(1) == heads * dk && out.is_cuda() && out.is_contiguous() && is_act(out) &&
+              out.dim() == 2 && out.size(0) == t && out.size(1) == heads * dv, "q / out");
+  check_cache(k_cache, kv_heads * dk, "k_cache");
+  check_cache(v_cache, kv_heads * dv, "v_cache");
+  TORCH_CHECK(k_cache.scalar_type() == v_cache.scalar_type() && k_cache.size(0) == v_cache.size(0) &&
+              k_cache.size(1) == v_cache.size(1), "k / v caches differ");
+  check_segs(start, pos0, kv_len, num_segs);
+  check_i32(bt, "block tables");
+  TORCH_CHECK(bt.dim() == 2 && bt.size(0) >= num_segs && max_rows <= t, "block tables / max_rows");
+  long gs = 0;
+  const void* gp = gate_rows(gate, out, t, heads * dv, &gs);
+  // key slices of 64-key tiles: enough workgroups to fill the chip
+  int64_t bound = window > 0 ? window + keep_first : (max_kv > 0 ? max_kv : 4096);
+  if (max_kv > 0) bound = std::min(bound, max_kv);
+  const int64_t per_seg = std::max<int64_t>(1, std::min(max_rows, skip_from > 0 ? skip_from - 1 : max_rows));
+  const int64_t rows = std::max<int64_t>(1, std::min<int64_t>(t, num_segs * per_seg));
+  int64_t splits = std::max<int64_t>(1, std::min<int64_t>({(bound + 63) / 64, 512 / rows, 64}));
+  while (splits > 1 && t * splits * heads * dv * 4 > (256LL << 20)) splits /= 2;
+  Tensor ws_acc = at::empty({t, splits, heads, dv}, q.options()), ws_ml = at::empty({t, splits, heads, 2}, q.options());
+  chk(mx_talk_attention(out.data_ptr(), bf(out), ws_acc.data_ptr<float>(), ws_ml.data_ptr<float>(), q.data_ptr<float>(),
+                        gp, gs, k_cache.data_ptr(), v_cache.data_ptr(), bf(k_cache), start.data_ptr<int>(),
+                        pos0.data_ptr<int>(), kv_len.data_ptr<int>(), bt.data_ptr<int>(), (int)bt.size(1),
+                        (int)num_segs, t, (int)heads, (int)kv_heads, (int)dk, (int)dv, (int)window, (int)keep_first,
+                        (float)softcap, talk.data_ptr<float>(), (int)k_cache.size(1), (int)k_cache.size(0),
+                        (int)skip_from, (int)splits, stream()), "talk_attention");
+}
+
+void talk_weights(Tensor S, Tensor inv, int64_t first_pos, int64_t key0, int64_t ext, int64_t window,
+                  int64_t keep_first, double softcap, Tensor talk) {
+  check_f32(S, "S");
+  check_f32(inv, "inv");
+  check_f32(talk, "head mix");
+  TORCH_CHECK(S.dim() == 3 && S.size(0) >= 1 && S.size(0) <= mx_talk_max_heads() &&
+              inv.numel() == S.size(0) * S.size(1) && talk.numel() == S.size(0) * S.size(0) && first_pos >= 0 &&
+              key0 >= 0 && ext >= 0 && ext <= key0 && ext <= S.size(2) && keep_first >= 0, "talk_weights shapes");
+  chk(mx_talk_weights(S.data_ptr<float>(), inv.data_ptr<float>(), (int)S.size(0), (int)S.size(1), (int)S.size(2),
+                      (int)first_pos, (int)key0, (int)ext, (int)window, (int)keep_first, (float)softcap,
+                      talk.data_ptr<float>(), stream()), "talk_weights");
+}
+
+void heads_to_rows(const Tensor& out, const Tensor& o, const OptT& inv, const OptT& gate, bool per_head) {
+  check_f32(o, "o");
+  TORCH_CHECK(o.dim() == 3, "o [heads, rows, dv]");
+  const int64_t heads = o.size(0), rows = o.size(1), dv = o.size(2);
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && is_act(out) && out.dim() == 2 && out.size(0) == rows &&
+              out.size(1) == heads * dv, "out");
+  long gs = 0;
+  const void* gp = gate_rows(gate, out, rows, per_head ? heads : heads * dv, &gs);
+  chk(mx_heads_to_rows(out.data_ptr(), bf(out), o.data_ptr<float>(), opt_f32(inv, heads * rows, "inv"), gp, gs,
+                       per_head ? 1 : 0, rows, (int)heads, (int)dv, stream()), "heads_to_rows");
+}
+
+void scaled_heads_gate(Tensor out, Tensor o, Tensor inv, OptT gate) { heads_to_rows(out, o, inv, gate, false); }
+void head_gate(Tensor out, Tensor o, Tensor gate) { heads_to_rows(out, o, {}, gate, true); }
+
 }  // namespace
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
@@ -854,7 +1041,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("causal_softmax", &causal_softmax);
   m.def("moe_topk", &moe_topk);
   m.def("moe_pairs", &moe_pairs);
-  m.def("gelu_glu", &gelu_glu);
+  m.def("act_glu", &act_glu);
+  m.def("add_norm_shift", &add_norm_shift);
+  m.def("rot_norm_prep", &rot_norm_prep);
+  m.def("talk_attention", &talk_attention);
+  m.def("talk_weights", &talk_weights);
+  m.def("scaled_heads_gate", &scaled_heads_gate);
+  m.def("head_gate", &head_gate);
+  m.def("talk_max_heads", []() { return (int64_t)mx_talk_max_heads(); });
   m.def("attn_prep", &attn_prep);
   m.def("window_attention", &window_attention);
   m.def("band_weights", &band_weights);

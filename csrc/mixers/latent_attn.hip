@@ -1,10 +1,12 @@
 // Latent attention over a paged cache whose rows are [c (rank) | rotated shared key (dr)]:
 //   * latent_kv_write: c = rms_norm(down-projection[:rank]) * w, key part rotated
-//     (rotate-half pairs over its first `dims` entries, fp32 angles from a table),
+//     (rotate-half or interleaved pairs over its first `dims` entries, fp32 angles from a
+//     table); optionally, in the same launch, the queries' own latent cq = rms_norm(xq) * wq,
 //   * latent_q_rope: splits query rows into unrotated and rotated fp32 parts,
 //   * latent_attention: causal softmax of (qa . c + qr . k_rot) * scale over the paged
 //     rows, returning the weighted sums of the c parts (the value up-projection is
-//     applied by the caller), fp32 scores / weights / sums.
+//     applied by the caller), fp32 scores / weights / sums.  Optionally one learned number
+//     per head, exp(sink[h]), joins the softmax's denominator.
 //
 // The attention kernel runs one workgroup per query row; its waves take the heads in
 // turn.  A wave scores 64 keys at a time (one key per lane), keeps a running max / sum
@@ -19,9 +21,21 @@ __global__ void latent_kv_write_kernel(const T* __restrict__ dkv, long stride, c
                                        float eps, const float* __restrict__ table, int table_rows,
                                        int dims, const int* __restrict__ positions,
                                        const int* __restrict__ slots, TC* __restrict__ cache, long num_slots,
-                                       int rank, int dr) {
+                                       int rank, int dr, int interleaved, const T* __restrict__ xq,
+                                       const float* __restrict__ wq, T* __restrict__ cq, int q_rank) {
   __shared__ float red[NT / 64];
   const long row = blockIdx.x;
+  if (cq != nullptr) {                     // the queries' latent (rows stride apart, like dkv)
+    const T* u = xq + row * stride;
+    float sq = 0.f;
+    for (int i = threadIdx.x; i < q_rank; i += NT) {
+      const float v = ld(u, i);
+      sq += v * v;
+    }
+    sq = block_sum<NT>(sq, red);
+    const float rq = 1.0f / sqrtf(sq / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += NT) st(cq, row * q_rank + i, ld(u, i) * rq * wq[i]);
+  }
   const long sl = slots[row];
   if (sl < 0 || sl >= num_slots) return;
   const T* x = dkv + row * stride;
@@ -37,26 +51,20 @@ __global__ void latent_kv_write_kernel(const T* __restrict__ dkv, long stride, c
   int p = positions[row];
   p = p < 0 ? 0 : (p >= table_rows ? table_rows - 1 : p);
   const float* cs = table + (long)p * dims;
-  const int half = dims / 2;
-  for (int i = threadIdx.x; i < dr; i += NT) {
-    float v;
-    if (i < half) v = ld(x, rank + i) * cs[i] - ld(x, rank + i + half) * cs[half + i];
-    else if (i < dims) v = ld(x, rank + i) * cs[i - half] + ld(x, rank + i - half) * cs[i];
-    else v = ld(x, rank + i);
-    st(dst, rank + i, v);
-  }
+  for (int i = threadIdx.x; i < dr; i += NT)
+    st(dst, rank + i, i < dims ? rope_at(x + rank, i, dims, cs, interleaved) : ld(x, rank + i));
 }
 
 template <typename T>
 __global__ void latent_q_rope_kernel(float* __restrict__ qn, float* __restrict__ qr,
                                      const T* __restrict__ q, long stride, const float* __restrict__ table,
                                      int table_rows, int dims, const int* __restrict__ positions, int heads,
-                                     int dn, int dr) {
+                                     int dn, int dr, int interleaved) {
   const long row = blockIdx.x;
   int p = positions[row];
   p = p < 0 ? 0 : (p >= table_rows ? table_rows - 1 : p);
   const float* cs = table + (long)p * dims;
-  const int half = dims / 2, hd = dn + dr;
+  const int hd = dn + dr;
   const T* x = q + row * stride;
   for (int e = threadIdx.x; e < heads * hd; e += blockDim.x) {
     const int h = e / hd, i = e % hd;
@@ -64,11 +72,7 @@ __global__ void latent_q_rope_kernel(float* __restrict__ qn, float* __restrict__
       qn[(row * heads + h) * dn + i] = ld(x, e);
     } else {
       const int j = i - dn;
-      float v;
-      if (j < half) v = ld(x, e) * cs[j] - ld(x, e + half) * cs[half + j];
-      else if (j < dims) v = ld(x, e) * cs[j - half] + ld(x, e - half) * cs[j];
-      else v = ld(x, e);
-      qr[(row * heads + h) * dr + j] = v;
+      qr[(row * heads + h) * dr + j] = j < dims ? rope_at(x + h * hd + dn, j, dims, cs, interleaved) : ld(x, e);
     }
   }
 }
@@ -80,7 +84,8 @@ latent_attention_kernel(float* __restrict__ out, const float* __restrict__ qa, c
                         const TC* __restrict__ cache, const int* __restrict__ start,
                         const int* __restrict__ pos0, const int* __restrict__ kv_len,
                         const int* __restrict__ bt, int bt_stride, int heads, long total_rows, int rank,
-                        int dr, int block_size, int num_blocks, float scale, int skip_from) {
+                        int dr, int block_size, int num_blocks, float scale, int skip_from,
+                        const float* __restrict__ sink) {
   extern __shared__ float smem[];
   const int s = blockIdx.y;
   const int r0 = start[s], n = start[s + 1] - r0;
@@ -137,7 +142,13 @@ latent_attention_kernel(float* __restrict__ out, const float* __restrict__ qa, c
         }
       }
     }
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float fin = 1.f;
+    if (sink != nullptr && nk > 0) {             // one more term of the denominator
+      const float mn = fmaxf(m, sink[h]);
+      fin = expf(m - mn);
+      l = l * fin + expf(sink[h] - mn);
+    }
+    const float inv = l > 0.f ? fin / l : 0.f;
     float* op = out + ((long)h * total_rows + row) * rank;
 #pragma unroll
     for (int r = 0; r < RPL; ++r) {
@@ -334,16 +345,17 @@ latent_split_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const
 // out[h, row, :] = sum_s exp(m_s - M) acc_s / sum_s exp(m_s - M) l_s over the key slices
 __global__ void latent_combine_kernel(float* __restrict__ out, const float* __restrict__ ws_acc,
                                       const float* __restrict__ ws_ml, const int* __restrict__ start,
-                                      int heads, long total_rows, int rank, int skip_from, int splits) {
+                                      int heads, long total_rows, int rank, int skip_from, int splits,
+                                      const float* __restrict__ sink) {
   const int s = blockIdx.y;
   const int r0 = start[s], n = start[s + 1] - r0;
   const int rel = blockIdx.x;
   if (rel >= n || (skip_from > 0 && n >= skip_from)) return;
   const long row = r0 + rel;
   const int h = blockIdx.z;
-  float M = -INFINITY;
+  float M = sink != nullptr ? sink[h] : -INFINITY;
   for (int sp = 0; sp < splits; ++sp) M = fmaxf(M, ws_ml[((row * splits + sp) * heads + h) * 2]);
-  float L = 0.f;
+  float L = sink != nullptr ? expf(sink[h] - M) : 0.f;
   for (int sp = 0; sp < splits; ++sp) {
     const long b = (row * splits + sp) * heads + h;
     const float m = ws_ml[b * 2];
@@ -366,13 +378,14 @@ __global__ void latent_combine_kernel(float* __restrict__ out, const float* __re
 // 0 beyond (rows r = head * rows_per_head + query row); fp32 statistics, P in TP
 template <typename TP, int NT>
 __global__ void causal_softmax_kernel(TP* __restrict__ P, const float* __restrict__ S, int rows_per_head,
-                                      int first_pos, int ncols, float scale) {
+                                      int first_pos, int ncols, float scale, const float* __restrict__ sink) {
   __shared__ float red[NT / 64];
   __shared__ float bmax;
   const long r = blockIdx.x;
   const int valid = min(first_pos + (int)(r % rows_per_head) + 1, ncols);
   const float* sr = S + r * ncols;
-  float m = -INFINITY;
+  const float sk = sink != nullptr ? sink[r / rows_per_head] : -INFINITY;
+  float m = sk;
   for (int j = threadIdx.x; j < valid; j += NT) m = fmaxf(m, sr[j] * scale);
   m = ft::wave_max(m);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = m;
@@ -387,6 +400,7 @@ __global__ void causal_softmax_kernel(TP* __restrict__ P, const float* __restric
   float sum = 0.f;
   for (int j = threadIdx.x; j < valid; j += NT) sum += expf(sr[j] * scale - m);
   sum = block_sum<NT>(sum, red);
+  if (sink != nullptr) sum += expf(sk - m);
   const float inv = sum > 0.f ? 1.0f / sum : 0.f;
   for (int j = threadIdx.x; j < ncols; j += NT)
     st(P, r * ncols + j, j < valid ? expf(sr[j] * scale - m) * inv : 0.f);
@@ -397,31 +411,32 @@ __global__ void causal_softmax_kernel(TP* __restrict__ P, const float* __restric
 using namespace mx;
 
 extern "C" int mx_causal_softmax(void* P, int p_bf16, const float* S, long rows, int rows_per_head,
-                                 int first_pos, int ncols, float scale, hipStream_t s) {
+                                 int first_pos, int ncols, float scale, const float* sink, hipStream_t s) {
   if (rows <= 0 || ncols <= 0) return 0;
   if (p_bf16)
     hipLaunchKernelGGL((causal_softmax_kernel<bf16_t, 256>), dim3((unsigned)rows), dim3(256), 0, s, (bf16_t*)P, S,
-                       rows_per_head, first_pos, ncols, scale);
+                       rows_per_head, first_pos, ncols, scale, sink);
   else
     hipLaunchKernelGGL((causal_softmax_kernel<float, 256>), dim3((unsigned)rows), dim3(256), 0, s, (float*)P, S,
-                       rows_per_head, first_pos, ncols, scale);
+                       rows_per_head, first_pos, ncols, scale, sink);
   return (int)hipGetLastError();
 }
 
 extern "C" int mx_latent_kv_write(const void* dkv, int bf16, long stride, const float* w, float eps,
                                   const float* table, int table_rows, int dims, const int* positions,
                                   const int* slots, void* cache, int cache_bf16, long num_slots, long rows,
-                                  int rank, int dr, hipStream_t s) {
+                                  int rank, int dr, int interleaved, const void* xq, const float* wq, void* cq,
+                                  int q_rank, hipStream_t s) {
   if (rows <= 0) return 0;
   const dim3 grid((unsigned)rows), block(256);
   if (bf16 && cache_bf16)
     hipLaunchKernelGGL((latent_kv_write_kernel<bf16_t, bf16_t, 256>), grid, block, 0, s, (const bf16_t*)dkv,
                        stride, w, eps, table, table_rows, dims, positions, slots, (bf16_t*)cache, num_slots,
-                       rank, dr);
+                       rank, dr, interleaved, (const bf16_t*)xq, wq, (bf16_t*)cq, q_rank);
   else if (!bf16 && !cache_bf16)
     hipLaunchKernelGGL((latent_kv_write_kernel<float, float, 256>), grid, block, 0, s, (const float*)dkv,
                        stride, w, eps, table, table_rows, dims, positions, slots, (float*)cache, num_slots,
-                       rank, dr);
+                       rank, dr, interleaved, (const float*)xq, wq, (float*)cq, q_rank);
   else
     return -1;
   return (int)hipGetLastError();
@@ -429,11 +444,11 @@ extern "C" int mx_latent_kv_write(const void* dkv, int bf16, long stride, const 
 
 extern "C" int mx_latent_q_rope(float* qn, float* qr, const void* q, int bf16, long stride,
                                 const float* table, int table_rows, int dims, const int* positions,
-                                long rows, int heads, int dn, int dr, hipStream_t s) {
+                                long rows, int heads, int dn, int dr, int interleaved, hipStream_t s) {
   if (rows <= 0) return 0;
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((latent_q_rope_kernel<T>), dim3((unsigned)rows), dim3(256), 0, s,
                                          qn, qr, (const T*)q, stride, table, table_rows, dims, positions,
-                                         heads, dn, dr));
+                                         heads, dn, dr, interleaved));
   return (int)hipGetLastError();
 }
 
@@ -443,17 +458,17 @@ template <typename TC, int RPL>
 static void launch_latent(dim3 grid, size_t lds, hipStream_t s, float* out, const float* qa, const float* qr,
                           const void* cache, const int* start, const int* pos0, const int* kv_len,
                           const int* bt, int bt_stride, int heads, long total_rows, int rank, int dr,
-                          int block_size, int num_blocks, float scale, int skip_from) {
+                          int block_size, int num_blocks, float scale, int skip_from, const float* sink) {
   hipLaunchKernelGGL((latent_attention_kernel<TC, RPL>), grid, dim3(256), lds, s, out, qa, qr,
                      (const TC*)cache, start, pos0, kv_len, bt, bt_stride, heads, total_rows, rank, dr,
-                     block_size, num_blocks, scale, skip_from);
+                     block_size, num_blocks, scale, skip_from, sink);
 }
 
 extern "C" int mx_latent_attention(float* out, const float* qa, const float* qr, const void* cache,
                                    int cache_bf16, const int* start, const int* pos0, const int* kv_len,
                                    const int* bt, int bt_stride, int num_segs, int max_rows, int heads,
                                    long total_rows, int rank, int dr, int block_size, int num_blocks,
-                                   float scale, int skip_from, hipStream_t s) {
+                                   float scale, int skip_from, const float* sink, hipStream_t s) {
   if (num_segs <= 0 || max_rows <= 0) return 0;
   if (rank < 1 || rank > mx_latent_max_rank() || max_rows > 65535 * 32 || num_segs > 65535) return -1;
   const size_t lds = (size_t)4 * (rank + dr) * sizeof(float);
@@ -466,10 +481,12 @@ extern "C" int mx_latent_attention(float* out, const float* qa, const float* qr,
   do {                                                                                                  \
     if (cache_bf16)                                                                                     \
       launch_latent<bf16_t, RPL>(grid, lds, s, out, qa, qr, cache, start, pos0, kv_len, bt, bt_stride,  \
-                                 heads, total_rows, rank, dr, block_size, num_blocks, scale, skip_from); \
+                                 heads, total_rows, rank, dr, block_size, num_blocks, scale, skip_from, \
+                                 sink);                                                                 \
     else                                                                                                \
       launch_latent<float, RPL>(grid, lds, s, out, qa, qr, cache, start, pos0, kv_len, bt, bt_stride,   \
-                                heads, total_rows, rank, dr, block_size, num_blocks, scale, skip_from); \
+                                heads, total_rows, rank, dr, block_size, num_blocks, scale, skip_from, \
+                                sink);                                                                  \
   } while (0)
   if (need <= 1) MX_LAT(1);
   else if (need <= 2) MX_LAT(2);
@@ -518,7 +535,7 @@ extern "C" int mx_latent_attention_split(float* out, float* ws_acc, float* ws_ml
                                          const int* pos0, const int* kv_len, const int* bt, int bt_stride,
                                          int num_segs, int max_rows, int heads, long total_rows, int rank,
                                          int dr, int block_size, int num_blocks, float scale, int skip_from,
-                                         int splits, hipStream_t s) {
+                                         int splits, const float* sink, hipStream_t s) {
   if (num_segs <= 0 || max_rows <= 0) return 0;
   if (skip_from > 0 && max_rows >= skip_from) max_rows = skip_from - 1;
   if (max_rows <= 0) return 0;
@@ -546,6 +563,6 @@ extern "C" int mx_latent_attention_split(float* out, float* ws_acc, float* ws_ml
   else MX_SPLIT(64);
 #undef MX_SPLIT
   hipLaunchKernelGGL(latent_combine_kernel, dim3(max_rows, num_segs, heads), dim3(rank >= 256 ? 256 : 64), 0,
-                     s, out, ws_acc, ws_ml, start, heads, total_rows, rank, skip_from, splits);
+                     s, out, ws_acc, ws_ml, start, heads, total_rows, rank, skip_from, splits, sink);
   return (int)hipGetLastError();
 }

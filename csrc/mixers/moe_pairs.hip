@@ -1,7 +1,7 @@
 // Mixture-of-experts for few rows (decode steps, hipGraph-capturable: nothing is read
 // back on the host): every (row, chosen expert) pair streams its expert's weights.
 //
-//   moe_gu_pairs:   y[pair, c] = glu(W_gate[e] h, W_up[e] h)[c]      (clamped GLU fused)
+//   moe_gu_pairs:   y[pair, c] = glu(W_gate[e] h, W_up[e] h)[c]      (clamped or silu GLU fused)
 //                   or, for experts without a gate, y[pair, c] = relu(W_up[e] h)[c]^2
 //   moe_down_pairs: out[row, c] += sum_k w[row, k] * (W_down[e_k] y[row, k])[c]   (fp32)
 //
@@ -45,12 +45,15 @@ __device__ __forceinline__ float dot_part(const T* a, const T* b, int n, int lan
   return s;
 }
 
+// an expert's activation: clamped GLU, relu^2 of one matrix, silu(gate) * up
+enum { kClampGlu = 0, kReluSq = 1, kSiluGlu = 2 };
+
 // grid (ceil(ff / 4), pairs), 256 threads: wave w -> column 4 * blockIdx.x + w
 template <typename T>
 __global__ void __launch_bounds__(256)
 moe_gu_pairs_kernel(T* __restrict__ y, const T* __restrict__ h, long h_stride, const int* __restrict__ idx,
                     const T* __restrict__ wgu, int top, int experts, int ff, int width, float limit,
-                    int vec, int relu_sq) {
+                    int vec, int act) {
   const int pair = blockIdx.y;
   const int c = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (c >= ff) return;
@@ -58,7 +61,7 @@ moe_gu_pairs_kernel(T* __restrict__ y, const T* __restrict__ h, long h_stride, c
   int e = idx[pair];
   if (e < 0 || e >= experts) e = 0;
   const T* hr = h + (long)(pair / top) * h_stride;
-  if (relu_sq) {
+  if (act == kReluSq) {
     // one matrix [ff, width] per expert
     const float u0 = ft::wave_sum(dot_part(hr, wgu + ((long)e * ff + c) * width, width, lane, vec));
     if (lane == 0) {
@@ -78,9 +81,14 @@ moe_gu_pairs_kernel(T* __restrict__ y, const T* __restrict__ h, long h_stride, c
     T tmp[2];
     st(tmp, 0, g0);
     st(tmp, 1, u0);
-    const float g = fminf(ld(tmp, 0), limit);
-    const float u = fminf(fmaxf(ld(tmp, 1), -limit), limit);
-    st(y, (long)pair * ff + c, g * sigmoidf_(1.702f * g) * (u + 1.0f));
+    if (act == kSiluGlu) {
+      const float g = ld(tmp, 0);
+      st(y, (long)pair * ff + c, g * sigmoidf_(g) * ld(tmp, 1));
+    } else {
+      const float g = fminf(ld(tmp, 0), limit);
+      const float u = fminf(fmaxf(ld(tmp, 1), -limit), limit);
+      st(y, (long)pair * ff + c, g * sigmoidf_(1.702f * g) * (u + 1.0f));
+    }
   }
 }
 
@@ -113,8 +121,9 @@ using namespace mx;
 
 extern "C" int mx_moe_pairs(float* out, void* y, const void* h, int bf16, long h_stride, const int* idx,
                             const float* wts, const void* wgu, const void* wdown, long rows, int top,
-                            int experts, int ff, int width, float limit, int relu_sq, hipStream_t s) {
+                            int experts, int ff, int width, float limit, int act, hipStream_t s) {
   if (rows <= 0) return 0;
+  if (act < kClampGlu || act > kSiluGlu) return -1;
   const long pairs = rows * top;
   if (pairs > 65535 || rows > 65535) return -1;
   const int n = bf16 ? 8 : 4;
@@ -122,7 +131,7 @@ extern "C" int mx_moe_pairs(float* out, void* y, const void* h, int bf16, long h
   const int vec_dn = (ff % n == 0) ? 1 : 0;
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((moe_gu_pairs_kernel<T>), dim3((ff + 3) / 4, (unsigned)pairs), dim3(256),
                                          0, s, (T*)y, (const T*)h, h_stride, idx, (const T*)wgu, top, experts, ff,
-                                         width, limit, vec_gu, relu_sq));
+                                         width, limit, vec_gu, act));
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((moe_down_pairs_kernel<T>), dim3((width + 3) / 4, (unsigned)rows),
                                          dim3(256), 0, s, out, (const T*)y, idx, wts, (const T*)wdown, top,
                                          experts, ff, width, vec_dn));

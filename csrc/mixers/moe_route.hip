@@ -4,8 +4,9 @@
 // is its best biased score; excluded experts count as -infinity), then the `top`
 // eligible experts with the largest biased scores.  Weights = the chosen experts'
 // unbiased softmax scores, not renormalised.  One wave per token; ties go to the lower
-// index.  A second router (moe_top_logits) chooses on the logits and renormalises over
-// the chosen ones.
+// index.  A second router (moe_top_logits) chooses on the logits and weights the chosen ones
+// by the softmax over just those, or by their sigmoids divided by the sum of those, times a
+// factor.
 #include "mx_common.h"
 
 namespace mx {
@@ -91,11 +92,21 @@ moe_topk_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __r
   }
 }
 
+// weights of the chosen logits val[0 .. top) (largest first), one wave
+__device__ __forceinline__ void chosen_weights(float* w, const float* val, int top, int lane, int sigmoid, float scale) {
+  auto f = [&](int k) { return sigmoid ? sigmoidf_(val[k]) : expf(val[k] - val[0]); };
+  float sum = 0.f;
+  for (int k = lane; k < top; k += 64) sum += f(k);
+  sum = ft::wave_sum(sum);
+  if (sigmoid) sum += 1e-20f;
+  for (int k = lane; k < top; k += 64) w[k] = f(k) / sum * scale;
+}
+
 // Routing on the logits themselves: the `top` largest logits of a row are chosen (ties to
-// the lower index) and weighted by the softmax over just those.  One wave per token.
+// the lower index) and weighted by chosen_weights.  One wave per token.
 __global__ void __launch_bounds__(64)
 moe_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ z, int experts,
-                      int top) {
+                      int top, int sigmoid, float scale) {
   extern __shared__ float sm[];
   float* ch = sm;                   // logits, -inf once taken
   float* val = sm + experts;        // the chosen logits, largest first
@@ -116,10 +127,7 @@ moe_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const floa
     }
     __syncthreads();
   }
-  float sum = 0.f;
-  for (int k = lane; k < top; k += 64) sum += expf(val[k] - val[0]);
-  sum = ft::wave_sum(sum);
-  for (int k = lane; k < top; k += 64) wts[row * top + k] = expf(val[k] - val[0]) / sum;
+  chosen_weights(wts + row * top, val, top, lane, sigmoid, scale);
 }
 
 // four consecutive activations as fp32
@@ -145,7 +153,7 @@ template <typename T>
 __global__ void __launch_bounds__(64 * kRouteWaves)
 moe_route_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const T* __restrict__ h, long h_stride,
                             const float* __restrict__ router, const float* __restrict__ bias, int experts,
-                            int width, int top, int vec) {
+                            int width, int top, int vec, int sigmoid, float scale) {
   extern __shared__ float sm[];
   float* ch = sm;
   float* val = sm + experts;
@@ -187,17 +195,14 @@ moe_route_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, cons
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
-  float sum = 0.f;
-  for (int k = lane; k < top; k += 64) sum += expf(val[k] - val[0]);
-  sum = ft::wave_sum(sum);
-  for (int k = lane; k < top; k += 64) wts[row * top + k] = expf(val[k] - val[0]) / sum;
+  chosen_weights(wts + row * top, val, top, lane, sigmoid, scale);
 }
 
 }  // namespace mx
 
 extern "C" int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int bf16, long h_stride,
                                        const float* router, const float* bias, long rows, int experts, int width,
-                                       int top, hipStream_t s) {
+                                       int top, int sigmoid, float scale, hipStream_t s) {
   if (rows <= 0) return 0;
   if (experts < 1 || top < 1 || top > experts || width < 1) return -1;
   const size_t lds = (size_t)(experts + top) * sizeof(float);
@@ -207,17 +212,18 @@ extern "C" int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int 
                   ((uintptr_t)router) % 16 == 0;
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((mx::moe_route_top_logits_kernel<T>), dim3((unsigned)rows),
                                          dim3(64 * mx::kRouteWaves), lds, s, idx, wts, (const T*)h, h_stride, router,
-                                         bias, experts, width, top, vec));
+                                         bias, experts, width, top, vec, sigmoid, scale));
   return (int)hipGetLastError();
 }
 
 extern "C" int mx_moe_top_logits(int* idx, float* wts, const float* z, long rows, int experts, int top,
-                                 hipStream_t s) {
+                                 int sigmoid, float scale, hipStream_t s) {
   if (rows <= 0) return 0;
   if (experts < 1 || top < 1 || top > experts) return -1;
   const size_t lds = (size_t)(experts + top) * sizeof(float);
   if (lds > 60 * 1024) return -2;
-  hipLaunchKernelGGL(mx::moe_top_logits_kernel, dim3((unsigned)rows), dim3(64), lds, s, idx, wts, z, experts, top);
+  hipLaunchKernelGGL(mx::moe_top_logits_kernel, dim3((unsigned)rows), dim3(64), lds, s, idx, wts, z, experts, top,
+                     sigmoid, scale);
   return (int)hipGetLastError();
 }
 

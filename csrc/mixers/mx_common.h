@@ -25,6 +25,18 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf
 // softplus with the usual linear branch for large arguments
 __device__ __forceinline__ float softplusf_(float x) { return x > 20.0f ? x : log1pf(expf(x)); }
 
+// entry d < dims of a head x after rotary positions, cs = [cos | sin] of the position: pairs
+// (i, i + dims/2), or (2i, 2i + 1) if interleaved
+template <typename T>
+__device__ __forceinline__ float rope_at(const T* x, int d, int dims, const float* cs, int interleaved) {
+  const int half = dims / 2;
+  const int i = interleaved ? d >> 1 : (d < half ? d : d - half);
+  const bool second = interleaved ? (d & 1) : d >= half;
+  const int other = interleaved ? d ^ 1 : (second ? d - half : d + half);
+  const float v = ld(x, d), w = ld(x, other), c = cs[i], s = cs[half + i];
+  return second ? v * c + w * s : v * c - w * s;
+}
+
 // sum over a block of NT threads (NT multiple of 64, <= 1024); every thread gets it
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red) {

@@ -1,8 +1,9 @@
 // Row-wise kernels around an fp32 residual stream: embedding rows (optionally with a
-// sinusoidal position vector), the fused "post-norm add + next pre-norm" step, the layer
+// sinusoidal position vector), the fused "post-norm add + next pre-norm" step (also with a
+// token shift of the normed row), the layer
 // norm (weight and bias) that adds a sublayer's output to the residual, the tanh cap of
 // the logits, per-head gated output norm, activations
-// (relu^2, clamped GLU, gelu GLU, gelu * token-side embedding) and the weighted row scatter-add
+// (relu^2, clamped / gelu / relu / silu GLU, gelu * token-side embedding) and the weighted row scatter-add
 // that combines expert outputs.
 #include "mx_common.h"
 
@@ -231,6 +232,173 @@ __global__ void add_rms_norm_kernel(float* __restrict__ x, const TY* __restrict_
     for (int i = threadIdx.x; i < width; i += NT) st(cast, row * width + i, xr[i]);
 }
 
+// ---------------------------------------------------------------------------------
+// the step between layers with a token shift, one workgroup per row:
+//   x_out = x_in + rms_norm(y) * wb (without y: x_out = x_in, not written)
+//   h = rms_norm(x_out) * w;  out = h + (h' - h) * shift
+// with h' the h of the token before: of the row above within a segment (recomputed here from
+// that row's x_in and y, so x_out must be another buffer than x_in when a segment has several
+// rows), of the state slot for a segment's first row, zeros for a sequence's first token.  A
+// one-row segment also leaves its h in the slot; shift_state_kernel does that for longer ones
+// afterwards (a slot may still be read by the segment's first row here).
+// A row lives in registers: 4 C consecutive-by-4 entries per thread, width <= 4 C NT.
+// ---------------------------------------------------------------------------------
+template <typename T, int NT, int C>
+__device__ __forceinline__ void load_row(float (&v)[C][4], const T* p, int width, int vec) {
+#pragma unroll
+  for (int c = 0; c < C; ++c) {
+    const int i = (c * NT + threadIdx.x) * 4;
+    if (vec && i < width) {
+      if constexpr (sizeof(T) == 2) {
+        const uint2 u = *reinterpret_cast<const uint2*>(p + i);
+        ft::unpack2(u.x, v[c][0], v[c][1]);
+        ft::unpack2(u.y, v[c][2], v[c][3]);
+      } else {
+        const float4 u = *reinterpret_cast<const float4*>(p + i);
+        v[c][0] = u.x; v[c][1] = u.y; v[c][2] = u.z; v[c][3] = u.w;
+      }
+    } else {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[c][k] = i + k < width ? ld(p, i + k) : 0.f;
+    }
+  }
+}
+
+template <typename T, int NT, int C>
+__device__ __forceinline__ void store_row(T* p, const float (&v)[C][4], int width, int vec) {
+#pragma unroll
+  for (int c = 0; c < C; ++c) {
+    const int i = (c * NT + threadIdx.x) * 4;
+    if (vec && i < width) {
+      if constexpr (sizeof(T) == 2) {
+        *reinterpret_cast<uint2*>(p + i) = make_uint2(ft::pack2(v[c][0], v[c][1]), ft::pack2(v[c][2], v[c][3]));
+      } else {
+        *reinterpret_cast<float4*>(p + i) = make_float4(v[c][0], v[c][1], v[c][2], v[c][3]);
+      }
+    } else {
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+        if (i + k < width) st(p, i + k, v[c][k]);
+    }
+  }
+}
+
+// sums of two values over a block; every thread gets both
+template <int NT>
+__device__ __forceinline__ void block_sum2(float& a, float& b, float (*red)[2]) {
+  a = ft::wave_sum(a);
+  b = ft::wave_sum(b);
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) {
+    red[threadIdx.x >> 6][0] = a;
+    red[threadIdx.x >> 6][1] = b;
+  }
+  __syncthreads();
+  a = b = 0.f;
+#pragma unroll
+  for (int w = 0; w < NT / 64; ++w) {
+    a += red[w][0];
+    b += red[w][1];
+  }
+}
+
+template <int C>
+__device__ __forceinline__ float sum_sq(const float (&v)[C][4]) {
+  float s = 0.f;
+#pragma unroll
+  for (int c = 0; c < C; ++c)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) s += v[c][k] * v[c][k];
+  return s;
+}
+
+template <typename TY, typename TO, int NT, int C>
+__global__ void __launch_bounds__(NT)
+add_norm_shift_kernel(float* x_out, const float* x_in, const TY* __restrict__ y, long y_stride,
+                      const float* __restrict__ wb, const float* __restrict__ w, const float* __restrict__ shift,
+                      TO* __restrict__ out, float* state, int num_slots, const int* __restrict__ start,
+                      const int* __restrict__ pos0, const int* __restrict__ slot, int num_segs, int width,
+                      float eps, int vec) {
+  __shared__ float red[NT / 64][2];
+  const long row = blockIdx.x;
+  int sl = -1, rel = 0, n = 1;
+  bool old = false;
+  if (row < start[num_segs]) {
+    int lo_s = 0, hi_s = num_segs;
+    while (hi_s - lo_s > 1) {
+      const int mid = (lo_s + hi_s) >> 1;
+      if (start[mid] <= row) lo_s = mid; else hi_s = mid;
+    }
+    rel = (int)row - start[lo_s];
+    n = start[lo_s + 1] - start[lo_s];
+    sl = slot[lo_s];
+    if (sl >= num_slots) sl = -1;
+    old = sl >= 0 && pos0[lo_s] > 0;
+  }
+  float xa[C][4], xp[C][4], t[C][4];
+  load_row<float, NT, C>(xa, x_in + row * width, width, vec);
+  if (rel > 0) load_row<float, NT, C>(xp, x_in + (row - 1) * width, width, vec);
+  if (y != nullptr) {
+    float yp[C][4];
+    load_row<TY, NT, C>(t, y + row * y_stride, width, vec);
+    if (rel > 0) load_row<TY, NT, C>(yp, y + (row - 1) * y_stride, width, vec);
+    float sa = sum_sq<C>(t), sb = rel > 0 ? sum_sq<C>(yp) : 0.f;
+    block_sum2<NT>(sa, sb, red);
+    const float ra = 1.0f / sqrtf(sa / (float)width + eps), rb = 1.0f / sqrtf(sb / (float)width + eps);
+    float wv[C][4];
+    load_row<float, NT, C>(wv, wb, width, vec);
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        xa[c][k] += t[c][k] * ra * wv[c][k];
+        if (rel > 0) xp[c][k] += yp[c][k] * rb * wv[c][k];
+      }
+    store_row<float, NT, C>(x_out + row * width, xa, width, vec);
+  }
+  float sa = sum_sq<C>(xa), sb = rel > 0 ? sum_sq<C>(xp) : 0.f;
+  block_sum2<NT>(sa, sb, red);
+  const float ra = 1.0f / sqrtf(sa / (float)width + eps), rb = 1.0f / sqrtf(sb / (float)width + eps);
+  load_row<float, NT, C>(t, w, width, vec);
+#pragma unroll
+  for (int c = 0; c < C; ++c)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      xa[c][k] *= ra * t[c][k];
+      xp[c][k] = rel > 0 ? xp[c][k] * (rb * t[c][k]) : 0.f;
+    }
+  if (rel == 0 && old) load_row<float, NT, C>(xp, state + (long)sl * width, width, vec);
+  if (sl >= 0 && n == 1) store_row<float, NT, C>(state + (long)sl * width, xa, width, vec);
+  load_row<float, NT, C>(t, shift, width, vec);
+#pragma unroll
+  for (int c = 0; c < C; ++c)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) xa[c][k] += (xp[c][k] - xa[c][k]) * t[c][k];
+  store_row<TO, NT, C>(out + row * width, xa, width, vec);
+}
+
+// the h of each longer segment's last row, from its x, into the segment's slot; grid segments
+template <int NT, int C>
+__global__ void __launch_bounds__(NT)
+shift_state_kernel(float* __restrict__ state, int num_slots, const float* __restrict__ x, const float* __restrict__ w,
+                   const int* __restrict__ start, const int* __restrict__ slot, int width, float eps, int vec) {
+  __shared__ float red[NT / 64][2];
+  const int s = blockIdx.x;
+  const int n = start[s + 1] - start[s], sl = slot[s];
+  if (n < 2 || sl < 0 || sl >= num_slots) return;
+  float xa[C][4], t[C][4];
+  load_row<float, NT, C>(xa, x + (long)(start[s + 1] - 1) * width, width, vec);
+  float sa = sum_sq<C>(xa), sb = 0.f;
+  block_sum2<NT>(sa, sb, red);
+  const float ra = 1.0f / sqrtf(sa / (float)width + eps);
+  load_row<float, NT, C>(t, w, width, vec);
+#pragma unroll
+  for (int c = 0; c < C; ++c)
+#pragma unroll
+    for (int k = 0; k < 4; ++k) xa[c][k] *= ra * t[c][k];
+  store_row<float, NT, C>(state + (long)sl * width, xa, width, vec);
+}
+
 // one wave per (row, head): out = o / rms(o) * w * sigmoid(gate), or * silu(gate)
 template <typename TG, typename TO>
 __global__ void head_rms_gate_kernel(TO* __restrict__ out, const float* __restrict__ o,
@@ -307,16 +475,17 @@ __device__ __forceinline__ float gelu_tanh_(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
-// rows [gate (ff) | up (ff)]: out = gelu_tanh(gate) * up, or relu(gate) * up
+// rows [gate (ff) | up (ff)]: out = act(gate) * up, act = gelu_tanh (0), relu (1) or silu (2)
 template <typename T>
-__global__ void gelu_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, long gu_stride, long rows, int ff,
-                                int relu) {
+__global__ void act_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, long gu_stride, long rows, int ff,
+                               int act) {
   const long n = rows * ff;
   for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
     const long r = i / ff;
     const int c = (int)(i % ff);
     const float g = ld(gu, r * gu_stride + c);
-    st(out, i, (relu ? fmaxf(g, 0.f) : gelu_tanh_(g)) * ld(gu, r * gu_stride + ff + c));
+    const float a = act == 2 ? g * sigmoidf_(g) : act == 1 ? fmaxf(g, 0.f) : gelu_tanh_(g);
+    st(out, i, a * ld(gu, r * gu_stride + ff + c));
   }
 }
 
@@ -464,11 +633,12 @@ extern "C" int mx_clamp_swiglu(void* out, const void* gu, int bf16, long gu_stri
   return (int)hipGetLastError();
 }
 
-extern "C" int mx_gelu_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int relu,
-                           hipStream_t s) {
+extern "C" int mx_act_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int act,
+                          hipStream_t s) {
   if (rows * ff <= 0) return 0;
-  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((gelu_glu_kernel<T>), dim3(ew_grid(rows * ff)), dim3(256), 0, s, (T*)out,
-                                         (const T*)gu, gu_stride, rows, ff, relu));
+  if (act < 0 || act > 2) return -1;
+  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((act_glu_kernel<T>), dim3(ew_grid(rows * ff)), dim3(256), 0, s, (T*)out,
+                                         (const T*)gu, gu_stride, rows, ff, act));
   return (int)hipGetLastError();
 }
 
@@ -549,5 +719,50 @@ extern "C" int mx_sigmoid_gate(void* out, int out_bf16, const float* o, const vo
                        g_stride, rows, n);
   else
     return -1;
+  return (int)hipGetLastError();
+}
+
+template <typename TY, typename TO, int C>
+static void launch_shift(float* x_out, const float* x_in, const void* y, long ys, const float* wb, const float* w,
+                         const float* shift, void* out, float* state, int num_slots, const int* start,
+                         const int* pos0, const int* slot, int num_segs, int max_rows, int rows, int width, float eps,
+                         int vec, hipStream_t s) {
+  constexpr int NT = 512;
+  hipLaunchKernelGGL((add_norm_shift_kernel<TY, TO, NT, C>), dim3(rows), dim3(NT), 0, s, x_out, x_in, (const TY*)y,
+                     ys, wb, w, shift, (TO*)out, state, num_slots, start, pos0, slot, num_segs, width, eps, vec);
+  if (max_rows > 1)
+    hipLaunchKernelGGL((shift_state_kernel<NT, C>), dim3(num_segs), dim3(NT), 0, s, state, num_slots, x_out, w, start,
+                       slot, width, eps, vec);
+}
+
+extern "C" int mx_shift_max_width() { return 512 * 4 * 8; }
+
+extern "C" int mx_add_norm_shift(float* x_out, const float* x_in, const void* y, int y_bf16, long y_stride,
+                                 const float* wb, const float* w, const float* shift, void* out, int out_bf16,
+                                 float* state, int num_slots, const int* start, const int* pos0, const int* slot,
+                                 int num_segs, int max_rows, int rows, int width, float eps, hipStream_t s) {
+  if (rows <= 0 || num_segs <= 0) return 0;
+  if (width < 1 || width > mx_shift_max_width() || (y != nullptr && max_rows > 1 && x_out == x_in)) return -1;
+  const long ye = y_bf16 ? 2 : 4;
+  const int vec = width % 4 == 0 && (y == nullptr || (y_stride % 4 == 0 && ((uintptr_t)y) % (4 * ye) == 0)) &&
+                  ((uintptr_t)x_in | (uintptr_t)x_out | (uintptr_t)w | (uintptr_t)wb | (uintptr_t)shift |
+                   (uintptr_t)state) % 16 == 0 && ((uintptr_t)out) % 8 == 0;
+  const int chunks = (width + 2047) / 2048;
+#define MX_SHIFT(TY, TO, C)                                                                                     \
+  launch_shift<TY, TO, C>(x_out, x_in, y, y_stride, wb, w, shift, out, state, num_slots, start, pos0, slot,     \
+                          num_segs, max_rows, rows, width, eps, vec, s)
+#define MX_SHIFT_C(TY, TO)                     \
+  do {                                         \
+    if (chunks <= 1) MX_SHIFT(TY, TO, 1);      \
+    else if (chunks <= 2) MX_SHIFT(TY, TO, 2); \
+    else if (chunks <= 4) MX_SHIFT(TY, TO, 4); \
+    else MX_SHIFT(TY, TO, 8);                  \
+  } while (0)
+  if (y_bf16 && out_bf16) MX_SHIFT_C(bf16_t, bf16_t);
+  else if (y_bf16) MX_SHIFT_C(bf16_t, float);
+  else if (out_bf16) MX_SHIFT_C(float, bf16_t);
+  else MX_SHIFT_C(float, float);
+#undef MX_SHIFT_C
+#undef MX_SHIFT
   return (int)hipGetLastError();
 }
