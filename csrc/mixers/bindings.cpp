@@ -31,7 +31,7 @@ int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int bf16, long 
                             const float* bias, long rows, int experts, int width, int top, int sigmoid, float scale,
                             hipStream_t s);
 int mx_act_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int act, hipStream_t s);
-int mx_shift_max_width();
+int mx_row_max_width();
 int mx_add_norm_shift(float* x_out, const float* x_in, const void* y, int y_bf16, long y_stride, const float* wb,
                       const float* w, const float* shift, void* out, int out_bf16, float* state, int num_slots,
                       const int* start, const int* pos0, const int* slot, int num_segs, int max_rows, int rows,
@@ -878,7 +878,7 @@ void add_norm_shift(Tensor x_out, Tensor x_in, OptT y, OptT wb, Tensor w, Tensor
   check_f32(shift, "shift");
   check_f32(state, "shift state");
   TORCH_CHECK(w.numel() == width && shift.numel() == width && state.dim() == 2 && state.size(0) >= 1 &&
-              state.size(1) == width && width <= mx_shift_max_width(), "add_norm_shift shapes");
+              state.size(1) == width && width <= mx_row_max_width(), "add_norm_shift shapes");
   TORCH_CHECK(out.is_cuda() && out.is_contiguous() && is_act(out) && out.sizes() == x_in.sizes(), "out");
   TORCH_CHECK((bool)y == (bool)wb, "y and its norm weight go together");
   TORCH_CHECK(max_rows >= 1 && max_rows <= rows + 1, "max_rows");

@@ -166,16 +166,6 @@ latent_attention_kernel(float* __restrict__ out, const float* __restrict__ qa, c
 // is read once per head group instead of once per head.  Each workgroup leaves (max,
 // sum, weighted c sums) per head; latent_combine_kernel merges the slices.
 // ---------------------------------------------------------------------------------
-// sum over the 16 lanes of a row (quad swaps, mirrored half row, mirrored row): every
-// lane gets the total
-__device__ __forceinline__ float sum16(float v) {
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, true));
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, true));
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, true));
-  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, true));
-  return v;
-}
-
 constexpr int kSplitTK = 8;    // keys per staged tile (compile time: the inner loops carry no branches)
 
 // Stages cnt <= kSplitTK cache rows (keys k0..) into LDS as fp32, a wave per key: the wave's
@@ -343,7 +333,10 @@ latent_split_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const
 }
 
 // out[h, row, :] = sum_s exp(m_s - M) acc_s / sum_s exp(m_s - M) l_s over the key slices
-__global__ void latent_combine_kernel(float* __restrict__ out, const float* __restrict__ ws_acc,
+// (plus the sink's term in the sum); one wave per (row, head, 256 columns), four of them per workgroup
+template <bool VEC>
+__global__ void __launch_bounds__(256)
+latent_combine_kernel(float* __restrict__ out, const float* __restrict__ ws_acc,
                                       const float* __restrict__ ws_ml, const int* __restrict__ start,
                                       int heads, long total_rows, int rank, int skip_from, int splits,
                                       const float* __restrict__ sink) {
@@ -352,26 +345,26 @@ __global__ void latent_combine_kernel(float* __restrict__ out, const float* __re
   const int rel = blockIdx.x;
   if (rel >= n || (skip_from > 0 && n >= skip_from)) return;
   const long row = r0 + rel;
-  const int h = blockIdx.z;
-  float M = sink != nullptr ? sink[h] : -INFINITY;
-  for (int sp = 0; sp < splits; ++sp) M = fmaxf(M, ws_ml[((row * splits + sp) * heads + h) * 2]);
-  float L = sink != nullptr ? expf(sink[h] - M) : 0.f;
-  for (int sp = 0; sp < splits; ++sp) {
-    const long b = (row * splits + sp) * heads + h;
-    const float m = ws_ml[b * 2];
-    L += m == -INFINITY ? 0.f : expf(m - M) * ws_ml[b * 2 + 1];
+  const int lane = threadIdx.x & 63, chunks = (rank + 255) / 256;
+  const int unit = blockIdx.z * 4 + (threadIdx.x >> 6);
+  const int h = unit / chunks;
+  if (h >= heads) return;
+  // lane = slice (splits <= 64)
+  const long b0 = row * splits * heads + h;
+  float ms = -INFINITY, ls = 0.f;
+  if (lane < splits) {
+    ms = ws_ml[(b0 + (long)lane * heads) * 2];
+    ls = ws_ml[(b0 + (long)lane * heads) * 2 + 1];
   }
+  float M = ft::wave_max(ms);
+  if (sink != nullptr) M = fmaxf(M, sink[h]);
+  const float w = ms == -INFINITY ? 0.f : expf(ms - M);
+  float L = ft::wave_sum(w * ls);
+  if (sink != nullptr) L += expf(sink[h] - M);
   const float inv = L > 0.f ? 1.0f / L : 0.f;
-  for (int d = threadIdx.x; d < rank; d += blockDim.x) {
-    float v = 0.f;
-    for (int sp = 0; sp < splits; ++sp) {
-      const long b = (row * splits + sp) * heads + h;
-      const float m = ws_ml[b * 2];
-      const float w = m == -INFINITY ? 0.f : expf(m - M);   // an empty slice left zeros
-      v += w * ws_acc[b * rank + d];
-    }
-    out[((long)h * total_rows + row) * rank + d] = v * inv;
-  }
+  float* op = out + ((long)h * total_rows + row) * rank;
+  merge_slices<VEC>(ws_acc + b0 * rank, (long)heads * rank, w, splits, (unit % chunks) * 256, rank, lane,
+                    [&](int c, float v) { op[c] = v * inv; });
 }
 
 // P[r, j] = softmax_j(scale * S[r, j]) over the keys j <= first_pos + (r mod rows_per_head),
@@ -542,7 +535,7 @@ extern "C" int mx_latent_attention_split(float* out, float* ws_acc, float* ws_ml
   int hg, tk;
   size_t lds;
   const int acc = split_plan(heads, rank, dr, &hg, &tk, &lds);
-  if (!acc || splits < 1 || max_rows > 65535 || num_segs > 65535 || heads > 65535) return -1;
+  if (!acc || splits < 1 || splits > 64 || max_rows > 65535 || num_segs > 65535 || heads > 65535) return -1;
   const int groups = (heads + hg - 1) / hg;
   const dim3 grid(splits * groups, max_rows, num_segs);
 #define MX_SPLIT(A)                                                                                      \
@@ -562,7 +555,12 @@ extern "C" int mx_latent_attention_split(float* out, float* ws_acc, float* ws_ml
   else if (acc <= 32) MX_SPLIT(32);
   else MX_SPLIT(64);
 #undef MX_SPLIT
-  hipLaunchKernelGGL(latent_combine_kernel, dim3(max_rows, num_segs, heads), dim3(rank >= 256 ? 256 : 64), 0,
-                     s, out, ws_acc, ws_ml, start, heads, total_rows, rank, skip_from, splits, sink);
+  const dim3 g2(max_rows, num_segs, (heads * ((rank + 255) / 256) + 3) / 4);
+  if (rank % 4 == 0 && ((uintptr_t)ws_acc) % 16 == 0)
+    hipLaunchKernelGGL((latent_combine_kernel<true>), g2, dim3(256), 0, s, out, ws_acc, ws_ml, start, heads,
+                       total_rows, rank, skip_from, splits, sink);
+  else
+    hipLaunchKernelGGL((latent_combine_kernel<false>), g2, dim3(256), 0, s, out, ws_acc, ws_ml, start, heads,
+                       total_rows, rank, skip_from, splits, sink);
   return (int)hipGetLastError();
 }

@@ -37,6 +37,108 @@ __device__ __forceinline__ float rope_at(const T* x, int d, int dims, const floa
   return second ? v * c + w * s : v * c - w * s;
 }
 
+// sum / maximum over the 16 lanes of a row (quad swaps, mirrored half row, mirrored row): every
+// lane gets it
+__device__ __forceinline__ float sum16(float v) {
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, true));
+  v += __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, true));
+  return v;
+}
+__device__ __forceinline__ float max16(float v) {
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xF, 0xF, true)));
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xF, 0xF, true)));
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xF, 0xF, true)));
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x140, 0xF, 0xF, true)));
+  return v;
+}
+
+// v plus the v of the lane 16 / 32 away (row swaps instead of the LDS permute path)
+__device__ __forceinline__ float add_row_pair(float v) {
+  const auto r = __builtin_amdgcn_permlane16_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+__device__ __forceinline__ float add_halves(float v) {
+  const auto r = __builtin_amdgcn_permlane32_swap(__float_as_uint(v), __float_as_uint(v), false, false);
+  return __uint_as_float(r[0]) + __uint_as_float(r[1]);
+}
+
+// tanh without branches: the Taylor polynomial up to |x| = 1/4, (1 - e^-2|x|) / (1 + e^-2|x|) beyond
+__device__ __forceinline__ float tanh_(float x) {
+  const float a = fabsf(x), q = a * a;
+  const float p = a + a * q * (-1.f / 3 + q * (2.f / 15 + q * (-17.f / 315 + q * (62.f / 2835 - q * (1382.f / 155925)))));
+  const float t = __builtin_amdgcn_exp2f(-2.8853900817779268f * a);
+  const float r = (1.f - t) / (1.f + t);
+  return copysignf(a < 0.25f ? p : r, x);
+}
+
+// a wave's own LDS writes, to be read by its other lanes
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// the segment that owns a row: the last s with start[s] <= row.  Decode rows come first in a
+// step, one row each: for them one look at two neighbouring entries is enough.
+__device__ __forceinline__ int segment_of(const int* __restrict__ start, int num_segs, int row) {
+  if (row < num_segs && start[row] == row && start[row + 1] == row + 1) return row;
+  int lo = 0, hi = num_segs;
+  while (hi - lo > 1) {
+    const int mid = (lo + hi) >> 1;
+    if (start[mid] <= row) lo = mid; else hi = mid;
+  }
+  return lo;
+}
+
+// sum_sp w[sp] acc[sp * stride + c] for a wave that owns columns [c0, c0 + 256) of n: w is lane
+// sp's value (slices <= 64; a slice of weight 0 is not read).  VEC (n and stride multiples of 4,
+// 16-byte aligned): several slices per pass, 16-byte loads; out(c, value) is called once per
+// column by one lane.
+template <bool VEC, typename F>
+__device__ __forceinline__ void merge_slices(const float* __restrict__ acc, long stride, float w, int slices, int c0,
+                                             int n, int lane, F out) {
+  const int cols = min(256, n - c0);
+  if constexpr (VEC) {
+    const int pieces = cols / 4;
+    int lpp = 1;
+    while (lpp < pieces) lpp <<= 1;              // lanes per slice
+    const int per = 64 / lpp, sub = lane / lpp, pc = lane & (lpp - 1);
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+    for (int s0 = 0; s0 < slices; s0 += per) {
+      const int sp = s0 + sub;
+      const float ws = __shfl(w, min(sp, 63));
+      if (sp < slices && ws != 0.f && pc < pieces) {
+        const float4 a = *reinterpret_cast<const float4*>(acc + sp * stride + c0 + 4 * pc);
+        v[0] += ws * a.x;
+        v[1] += ws * a.y;
+        v[2] += ws * a.z;
+        v[3] += ws * a.w;
+      }
+    }
+    for (int off = lpp; off < 64; off <<= 1) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[k] += __shfl_xor(v[k], off);
+    }
+    if (sub == 0 && pc < pieces) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) out(c0 + 4 * pc + k, v[k]);
+    }
+  } else {
+    for (int c = lane; c - lane < cols; c += 64) {
+      float v = 0.f;
+#pragma unroll 4
+      for (int sp = 0; sp < slices; ++sp) {
+        const float ws = __shfl(w, sp);
+        if (c < cols && ws != 0.f) v += ws * acc[sp * stride + c0 + c];
+      }
+      if (c < cols) out(c0 + c, v);
+    }
+  }
+}
+
 // sum over a block of NT threads (NT multiple of 64, <= 1024); every thread gets it
 template <int NT>
 __device__ __forceinline__ float block_sum(float v, float* red) {

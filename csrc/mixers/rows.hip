@@ -5,6 +5,8 @@
 // the logits, per-head gated output norm, activations
 // (relu^2, clamped / gelu / relu / silu GLU, gelu * token-side embedding) and the weighted row scatter-add
 // that combines expert outputs.
+#include <type_traits>
+
 #include "mx_common.h"
 
 namespace mx {
@@ -190,59 +192,8 @@ __global__ void tanh_cap_kernel(float* __restrict__ x, long n, float cap) {
   }
 }
 
-// residual (fp32, in place): x += rms_norm(y) * wb (+ add_vec);
-// out = rms_norm(x) * next_w (TO);  cast = x (TO).  Every part is optional.
-template <typename TY, typename TO, int NT>
-__global__ void add_rms_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, long y_stride,
-                                    const float* __restrict__ wb, const float* __restrict__ add_vec,
-                                    const float* __restrict__ next_w, TO* __restrict__ out,
-                                    TO* __restrict__ cast, int width, float eps) {
-  __shared__ float red[NT / 64];
-  const long row = blockIdx.x;
-  float* xr = x + row * width;
-  if (y != nullptr) {
-    const TY* yr = y + row * y_stride;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < width; i += NT) {
-      const float v = ld(yr, i);
-      ss += v * v;
-    }
-    ss = block_sum<NT>(ss, red);
-    const float r = 1.0f / sqrtf(ss / (float)width + eps);
-    for (int i = threadIdx.x; i < width; i += NT) {
-      float v = xr[i] + ld(yr, i) * r * wb[i];
-      if (add_vec != nullptr) v += add_vec[i];
-      xr[i] = v;
-    }
-  } else if (add_vec != nullptr) {
-    for (int i = threadIdx.x; i < width; i += NT) xr[i] += add_vec[i];
-  }
-  // each thread re-reads only what it wrote itself: no barrier needed
-  if (out != nullptr) {
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < width; i += NT) {
-      const float v = xr[i];
-      ss += v * v;
-    }
-    ss = block_sum<NT>(ss, red);
-    const float r = 1.0f / sqrtf(ss / (float)width + eps);
-    for (int i = threadIdx.x; i < width; i += NT) st(out, row * width + i, xr[i] * r * next_w[i]);
-  }
-  if (cast != nullptr)
-    for (int i = threadIdx.x; i < width; i += NT) st(cast, row * width + i, xr[i]);
-}
-
-// ---------------------------------------------------------------------------------
-// the step between layers with a token shift, one workgroup per row:
-//   x_out = x_in + rms_norm(y) * wb (without y: x_out = x_in, not written)
-//   h = rms_norm(x_out) * w;  out = h + (h' - h) * shift
-// with h' the h of the token before: of the row above within a segment (recomputed here from
-// that row's x_in and y, so x_out must be another buffer than x_in when a segment has several
-// rows), of the state slot for a segment's first row, zeros for a sequence's first token.  A
-// one-row segment also leaves its h in the slot; shift_state_kernel does that for longer ones
-// afterwards (a slot may still be read by the segment's first row here).
-// A row lives in registers: 4 C consecutive-by-4 entries per thread, width <= 4 C NT.
-// ---------------------------------------------------------------------------------
+// A row of a workgroup in registers: 4 C entries per thread, four neighbours at a time (16-byte
+// fp32 or 8-byte bf16 accesses when `vec`), width <= 4 C NT.
 template <typename T, int NT, int C>
 __device__ __forceinline__ void load_row(float (&v)[C][4], const T* p, int width, int vec) {
 #pragma unroll
@@ -312,6 +263,56 @@ __device__ __forceinline__ float sum_sq(const float (&v)[C][4]) {
   return s;
 }
 
+// residual (fp32, in place): x += rms_norm(y) * wb (+ add_vec);
+// out = rms_norm(x) * next_w (TO);  cast = x (TO).  Every part is optional.
+template <typename TY, typename TO, int NT, int C>
+__global__ void __launch_bounds__(NT)
+add_rms_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, long y_stride, const float* __restrict__ wb,
+                    const float* __restrict__ add_vec, const float* __restrict__ next_w, TO* __restrict__ out,
+                    TO* __restrict__ cast, int width, float eps, int vec) {
+  __shared__ float red[NT / 64];
+  const long row = blockIdx.x;
+  float v[C][4], t[C][4], w[C][4];
+  load_row<float, NT, C>(v, x + row * width, width, vec);
+  if (y != nullptr) {
+    load_row<TY, NT, C>(t, y + row * y_stride, width, vec);
+    load_row<float, NT, C>(w, wb, width, vec);
+    const float r = 1.0f / sqrtf(block_sum<NT>(sum_sq<C>(t), red) / (float)width + eps);
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[c][k] += t[c][k] * r * w[c][k];
+  }
+  if (add_vec != nullptr) {
+    load_row<float, NT, C>(w, add_vec, width, vec);
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[c][k] += w[c][k];
+  }
+  if (y != nullptr || add_vec != nullptr) store_row<float, NT, C>(x + row * width, v, width, vec);
+  if (cast != nullptr) store_row<TO, NT, C>(cast + row * width, v, width, vec);
+  if (out != nullptr) {
+    load_row<float, NT, C>(w, next_w, width, vec);
+    const float r = 1.0f / sqrtf(block_sum<NT>(sum_sq<C>(v), red) / (float)width + eps);
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+      for (int k = 0; k < 4; ++k) v[c][k] *= r * w[c][k];
+    store_row<TO, NT, C>(out + row * width, v, width, vec);
+  }
+}
+
+// ---------------------------------------------------------------------------------
+// the step between layers with a token shift, one workgroup per row:
+//   x_out = x_in + rms_norm(y) * wb (without y: x_out = x_in, not written)
+//   h = rms_norm(x_out) * w;  out = h + (h' - h) * shift
+// with h' the h of the token before: of the row above within a segment (recomputed here from
+// that row's x_in and y, so x_out must be another buffer than x_in when a segment has several
+// rows), of the state slot for a segment's first row, zeros for a sequence's first token.  A
+// one-row segment also leaves its h in the slot; shift_state_kernel does that for longer ones
+// afterwards (a slot may still be read by the segment's first row here).
+// ---------------------------------------------------------------------------------
 template <typename TY, typename TO, int NT, int C>
 __global__ void __launch_bounds__(NT)
 add_norm_shift_kernel(float* x_out, const float* x_in, const TY* __restrict__ y, long y_stride,
@@ -324,16 +325,12 @@ add_norm_shift_kernel(float* x_out, const float* x_in, const TY* __restrict__ y,
   int sl = -1, rel = 0, n = 1;
   bool old = false;
   if (row < start[num_segs]) {
-    int lo_s = 0, hi_s = num_segs;
-    while (hi_s - lo_s > 1) {
-      const int mid = (lo_s + hi_s) >> 1;
-      if (start[mid] <= row) lo_s = mid; else hi_s = mid;
-    }
-    rel = (int)row - start[lo_s];
-    n = start[lo_s + 1] - start[lo_s];
-    sl = slot[lo_s];
+    const int sg = segment_of(start, num_segs, (int)row);
+    rel = (int)row - start[sg];
+    n = start[sg + 1] - start[sg];
+    sl = slot[sg];
     if (sl >= num_slots) sl = -1;
-    old = sl >= 0 && pos0[lo_s] > 0;
+    old = sl >= 0 && pos0[sg] > 0;
   }
   float xa[C][4], xp[C][4], t[C][4];
   load_row<float, NT, C>(xa, x_in + row * width, width, vec);
@@ -552,18 +549,37 @@ extern "C" int mx_layer_norm(float* x, const void* y, int y_bf16, long y_stride,
   return (int)hipGetLastError();
 }
 
+constexpr int kRowThreads = 512;
+constexpr int kRowMaxWidth = kRowThreads * 4 * 8;
+
+// calls f with the number of register chunks a row of this width takes, as a constant
+template <typename F>
+static void row_chunks(int width, F f) {
+  const int chunks = (width + kRowThreads * 4 - 1) / (kRowThreads * 4);
+  if (chunks <= 1) f(std::integral_constant<int, 1>{});
+  else if (chunks <= 2) f(std::integral_constant<int, 2>{});
+  else if (chunks <= 4) f(std::integral_constant<int, 4>{});
+  else f(std::integral_constant<int, 8>{});
+}
+
 template <typename TY, typename TO>
 static void launch_add_rms(float* x, const void* y, long ys, const float* wb, const float* av,
                            const float* nw, void* out, void* cast, int rows, int width, float eps,
                            hipStream_t s) {
-  hipLaunchKernelGGL((add_rms_norm_kernel<TY, TO, 256>), dim3(rows), dim3(256), 0, s, x, (const TY*)y,
-                     ys, wb, av, nw, (TO*)out, (TO*)cast, width, eps);
+  const int vec = width % 4 == 0 && (y == nullptr || (ys % 4 == 0 && ((uintptr_t)y) % (4 * sizeof(TY)) == 0)) &&
+                  ((uintptr_t)x | (uintptr_t)wb | (uintptr_t)av | (uintptr_t)nw) % 16 == 0 &&
+                  ((uintptr_t)out | (uintptr_t)cast) % (4 * sizeof(TO)) == 0;
+  row_chunks(width, [&](auto c) {
+    hipLaunchKernelGGL((add_rms_norm_kernel<TY, TO, kRowThreads, decltype(c)::value>), dim3(rows), dim3(kRowThreads), 0,
+                       s, x, (const TY*)y, ys, wb, av, nw, (TO*)out, (TO*)cast, width, eps, vec);
+  });
 }
 
 extern "C" int mx_add_rms_norm(float* x, const void* y, int y_bf16, long y_stride, const float* wb,
                                const float* add_vec, const float* next_w, void* out, void* cast,
                                int out_bf16, int rows, int width, float eps, hipStream_t s) {
   if (rows <= 0) return 0;
+  if (width < 1 || width > kRowMaxWidth) return -1;
   if (y_bf16) {
     if (out_bf16) launch_add_rms<bf16_t, bf16_t>(x, y, y_stride, wb, add_vec, next_w, out, cast, rows, width, eps, s);
     else launch_add_rms<bf16_t, float>(x, y, y_stride, wb, add_vec, next_w, out, cast, rows, width, eps, s);
@@ -722,47 +738,40 @@ extern "C" int mx_sigmoid_gate(void* out, int out_bf16, const float* o, const vo
   return (int)hipGetLastError();
 }
 
-template <typename TY, typename TO, int C>
+template <typename TY, typename TO>
 static void launch_shift(float* x_out, const float* x_in, const void* y, long ys, const float* wb, const float* w,
                          const float* shift, void* out, float* state, int num_slots, const int* start,
                          const int* pos0, const int* slot, int num_segs, int max_rows, int rows, int width, float eps,
-                         int vec, hipStream_t s) {
-  constexpr int NT = 512;
-  hipLaunchKernelGGL((add_norm_shift_kernel<TY, TO, NT, C>), dim3(rows), dim3(NT), 0, s, x_out, x_in, (const TY*)y,
-                     ys, wb, w, shift, (TO*)out, state, num_slots, start, pos0, slot, num_segs, width, eps, vec);
-  if (max_rows > 1)
-    hipLaunchKernelGGL((shift_state_kernel<NT, C>), dim3(num_segs), dim3(NT), 0, s, state, num_slots, x_out, w, start,
-                       slot, width, eps, vec);
+                         hipStream_t s) {
+  const int vec = width % 4 == 0 && (y == nullptr || (ys % 4 == 0 && ((uintptr_t)y) % (4 * sizeof(TY)) == 0)) &&
+                  ((uintptr_t)x_in | (uintptr_t)x_out | (uintptr_t)w | (uintptr_t)wb | (uintptr_t)shift |
+                   (uintptr_t)state) % 16 == 0 && ((uintptr_t)out) % (4 * sizeof(TO)) == 0;
+  row_chunks(width, [&](auto c) {
+    constexpr int C = decltype(c)::value;
+    hipLaunchKernelGGL((add_norm_shift_kernel<TY, TO, kRowThreads, C>), dim3(rows), dim3(kRowThreads), 0, s, x_out,
+                       x_in, (const TY*)y, ys, wb, w, shift, (TO*)out, state, num_slots, start, pos0, slot, num_segs,
+                       width, eps, vec);
+    if (max_rows > 1)
+      hipLaunchKernelGGL((shift_state_kernel<kRowThreads, C>), dim3(num_segs), dim3(kRowThreads), 0, s, state,
+                         num_slots, x_out, w, start, slot, width, eps, vec);
+  });
 }
 
-extern "C" int mx_shift_max_width() { return 512 * 4 * 8; }
+extern "C" int mx_row_max_width() { return kRowMaxWidth; }
 
 extern "C" int mx_add_norm_shift(float* x_out, const float* x_in, const void* y, int y_bf16, long y_stride,
                                  const float* wb, const float* w, const float* shift, void* out, int out_bf16,
                                  float* state, int num_slots, const int* start, const int* pos0, const int* slot,
                                  int num_segs, int max_rows, int rows, int width, float eps, hipStream_t s) {
   if (rows <= 0 || num_segs <= 0) return 0;
-  if (width < 1 || width > mx_shift_max_width() || (y != nullptr && max_rows > 1 && x_out == x_in)) return -1;
-  const long ye = y_bf16 ? 2 : 4;
-  const int vec = width % 4 == 0 && (y == nullptr || (y_stride % 4 == 0 && ((uintptr_t)y) % (4 * ye) == 0)) &&
-                  ((uintptr_t)x_in | (uintptr_t)x_out | (uintptr_t)w | (uintptr_t)wb | (uintptr_t)shift |
-                   (uintptr_t)state) % 16 == 0 && ((uintptr_t)out) % 8 == 0;
-  const int chunks = (width + 2047) / 2048;
-#define MX_SHIFT(TY, TO, C)                                                                                     \
-  launch_shift<TY, TO, C>(x_out, x_in, y, y_stride, wb, w, shift, out, state, num_slots, start, pos0, slot,     \
-                          num_segs, max_rows, rows, width, eps, vec, s)
-#define MX_SHIFT_C(TY, TO)                     \
-  do {                                         \
-    if (chunks <= 1) MX_SHIFT(TY, TO, 1);      \
-    else if (chunks <= 2) MX_SHIFT(TY, TO, 2); \
-    else if (chunks <= 4) MX_SHIFT(TY, TO, 4); \
-    else MX_SHIFT(TY, TO, 8);                  \
-  } while (0)
-  if (y_bf16 && out_bf16) MX_SHIFT_C(bf16_t, bf16_t);
-  else if (y_bf16) MX_SHIFT_C(bf16_t, float);
-  else if (out_bf16) MX_SHIFT_C(float, bf16_t);
-  else MX_SHIFT_C(float, float);
-#undef MX_SHIFT_C
+  if (width < 1 || width > kRowMaxWidth || (y != nullptr && max_rows > 1 && x_out == x_in)) return -1;
+#define MX_SHIFT(TY, TO)                                                                                       \
+  launch_shift<TY, TO>(x_out, x_in, y, y_stride, wb, w, shift, out, state, num_slots, start, pos0, slot,       \
+                       num_segs, max_rows, rows, width, eps, s)
+  if (y_bf16 && out_bf16) MX_SHIFT(bf16_t, bf16_t);
+  else if (y_bf16) MX_SHIFT(bf16_t, float);
+  else if (out_bf16) MX_SHIFT(float, bf16_t);
+  else MX_SHIFT(float, float);
 #undef MX_SHIFT
   return (int)hipGetLastError();
 }

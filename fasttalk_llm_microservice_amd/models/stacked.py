@@ -206,7 +206,7 @@ class StackedModel:
         extra = {}
         if self.pair_embed is not None:
             extra["last_token"] = torch.full((max(num_slots, 1),), -1, dtype=torch.int32, device=self.device)
-        if any(L.shift is not None for L in self.layers):
+        if any(self.layers[i].shift is not None for i, _ in self.runs):
             extra["prev_h"] = [torch.zeros(max(num_slots, 1), self.cfg.hidden_size, dtype=torch.float32,
                                            device=self.device) if self.layers[i].shift is not None else None
                                for i, _ in self.runs]
