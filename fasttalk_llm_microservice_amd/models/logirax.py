@@ -95,13 +95,14 @@ def config_from_dict(c: dict, name: str = "logirax") -> LogiraxConfig:
             raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
         mlp = l.get("mlp")
         if mlp is not None:
-            if mlp["kind"] == DENSE:
+            kind = mlp.get("kind", MOE if "router" in mlp else DENSE)
+            if kind == DENSE:
                 mlp = {"kind": DENSE, "ff": int(mlp["ff"]), "limit": float(mlp["limit"])}
-            elif mlp["kind"] == MOE:
+            elif kind == MOE:
                 mlp = {"kind": MOE, "router": dict(mlp["router"]), "expert": dict(mlp["expert"]),
                        "shared": dict(mlp["shared"]) if mlp.get("shared") else None}
             else:
-                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+                raise ValueError(f"layer {i}: unknown feed-forward kind {kind!r}")
         layers.append({"type": l["type"], "mixer": m, "mlp": mlp})
     return LogiraxConfig(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]),
                          rms_norm_eps=float(c.get("norm", {}).get("eps", 1e-6)),
