@@ -110,7 +110,8 @@ def _on(seg, dev):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("H,G,d", [(6, 2, 24), (5, 5, 7), (16, 4, 128), (12, 4, 32), (33, 11, 16)])
+@pytest.mark.parametrize("H,G,d", [(6, 2, 24), (5, 5, 7), (16, 4, 128), (12, 4, 32), (33, 11, 16), (32, 8, 128), (32, 4, 64),
+                                   (24, 3, 40), (20, 20, 72), (16, 1, 160), (8, 1, 264), (64, 4, 32), (64, 8, 128)])
 def test_talking_kernels_multi_segment(dtype, H, G, d):
     """The preparation and the per-row attention kernel on a step of unequal segments (decode
     rows deep in a sequence, a fresh prompt, a later portion, padding) against the PyTorch
