@@ -22,14 +22,40 @@ int mx_gather_add_rows(float* out, const void* y, int y_bf16, const int* idx, co
                        int width, long y_rows, hipStream_t s);
 int mx_conv_attn_prep(float* q_out, const void* qkv, int bf16, long stride, int nq, int nk, int nv,
                       const float* conv_w, int taps, float* hist, const int* start, const int* pos0, const int* slot,
-                      int num_segs, int num_state_slots, const float* wq, const float* wk, float eps, int head_dim,
-                      const int* slots, void* k_cache, void* v_cache, int cache_bf16, long num_slots, long rows,
-                      hipStream_t s);
+                      int num_segs, int max_rows, int num_state_slots, const float* wq, const float* wk, float eps,
+                      int head_dim, const int* slots, void* k_cache, void* v_cache, int cache_bf16, long num_slots,
+                      const float* table, int table_rows, int rot_dims, int interleaved, long rows, hipStream_t s);
 int mx_moe_top_logits(int* idx, float* wts, const float* z, long rows, int experts, int top, int sigmoid,
-                      float scale, hipStream_t s);
+                      float scale, int groups, int keep, hipStream_t s);
 int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int bf16, long h_stride, const float* router,
                             const float* bias, long rows, int experts, int width, int top, int sigmoid, float scale,
-                            hipStream_t s);
+                            int groups, int keep, hipStream_t s);
+int mx_scaled_pair_rows(void* out, int bf16, const float* a, int n, float a_scale, const float* o, const void* gate,
+                        long gate_stride, float o_scale, long rows, int heads, int dv, float eps, hipStream_t s);
+int mx_head_max_dk();
+int mx_conv_delta_prep(float* qn, float* kn, float* vo, float* lg, float* beta, const void* x, int bf16, long x_stride,
+                       const void* a, long a_stride, const void* b, long b_stride, const float* conv_w, int taps,
+                       float* hist, const float* a_log, const float* dt_bias, const int* start, const int* pos0,
+                       const int* slot, int num_segs, int max_rows, long rows, int num_slots, int heads, int kv_heads,
+                       int dk, int dv, hipStream_t s);
+int mx_head_delta_walk(float* o, const float* q, const float* k, const float* v, const float* lg, const float* beta,
+                       float* state, const int* start, const int* pos0, const int* slot, int num_segs, int heads,
+                       int kv_heads, int dk, int dv, int num_slots, int skip_from, hipStream_t s);
+int mx_retention_walk(float* o, const void* p, int bf16, long stride, const float* table, int table_rows, int rot_dims,
+                      int interleaved, const double* log_decay, float* state, const int* start, const int* pos0,
+                      const int* slot, int num_segs, int heads, int dk, int dv, int num_slots, int skip_from,
+                      hipStream_t s);
+int mx_chunk_max_dk();
+int mx_chunk_rows();
+int mx_chunk_key_pad(int dk);
+int mx_head_delta_chunks(float* o, const float* q, const float* k, const float* v, const float* lg, const float* beta,
+                         float* state, float* ws_s, float* ws_w, float* ws_k, float* ws_u, float* ws_g,
+                         const int* start, const int* pos0, const int* slot, int num_segs, int max_rows, int heads,
+                         int kv_heads, int dk, int dv, int num_slots, int min_rows, hipStream_t s);
+int mx_retention_chunks(float* o, const void* p, int bf16, long stride, const float* table, int table_rows,
+                        int rot_dims, int interleaved, const double* log_decay, float* state, float* ws_s,
+                        const int* start, const int* pos0, const int* slot, int num_segs, int max_rows, int heads,
+                        int dk, int dv, int num_slots, int min_rows, hipStream_t s);
 int mx_act_glu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff, int act, hipStream_t s);
 int mx_row_max_width();
 int mx_add_norm_shift(float* x_out, const float* x_in, const void* y, int y_bf16, long y_stride, const float* wb,
@@ -73,12 +99,12 @@ int mx_window_attention(float* out, const float* q, const void* k_cache, const v
                         const int* start, const int* pos0, const int* kv_len, const int* bt, int bt_stride,
                         int num_segs, long total_rows, int heads, int maps, int kv_heads, int dk, int dv, int window,
                         float scale, int sigmoid, const float* r1, const float* r2, const float* pb, int block_size,
-                        int num_blocks, int skip_from, float softcap, int has_sink, float sink, int blocks,
-                        int keep_first, const float* dist_bias, int nd, hipStream_t s);
+                        int num_blocks, int skip_from, float softcap, int has_sink, float sink, const float* sinks,
+                        int blocks, int keep_first, const float* dist_bias, int nd, hipStream_t s);
 int mx_band_weights(float* S, int gk, int rep_rows_total, int rows, int keys, int first_pos, int key0, int heads,
                     int maps, int kv_heads, int window, float scale, int sigmoid, const float* r1, const float* r2,
-                    const float* pb, float softcap, int has_sink, float sink, int blocks, int keep_first, int ext,
-                    const float* dist_bias, int nd, hipStream_t s);
+                    const float* pb, float softcap, int has_sink, float sink, const float* sinks, int blocks,
+                    int keep_first, int ext, const float* dist_bias, int nd, hipStream_t s);
 int mx_diff_combine(void* out, int out_bf16, const float* a, const void* gate, int gate_bf16, long gate_stride,
                     long rows, int heads, int dv, float lam, float post, float eps, hipStream_t s);
 int mx_ssd_max_state();
@@ -173,6 +199,23 @@ void check_segs(const Tensor& start, const Tensor& a, const Tensor& b, int64_t n
   TORCH_CHECK(num >= 0 && start.numel() >= num + 1 && a.numel() >= num && b.numel() >= num, "segment arrays too short");
 }
 
+// an optional rotary table [positions, dims] (none: dims 0)
+struct RopeArg {
+  const float* table = nullptr;
+  int rows = 0, dims = 0;
+};
+RopeArg rope_arg(const OptT& table, int64_t rot_dims, int64_t head_dim) {
+  RopeArg r;
+  if (!table || rot_dims <= 0) return r;
+  check_f32(*table, "rope table");
+  TORCH_CHECK(table->dim() == 2 && table->size(0) >= 1 && table->size(1) == rot_dims && rot_dims % 2 == 0 &&
+              rot_dims <= head_dim, "rope table shape");
+  r.table = table->data_ptr<float>();
+  r.rows = (int)table->size(0);
+  r.dims = (int)rot_dims;
+  return r;
+}
+
 void embed_rows(Tensor out, Tensor ids, Tensor table, double scale, OptT positions, OptT freqs) {
   check_f32(out, "out");
   check_i32(ids, "ids");
@@ -239,9 +282,11 @@ void add_rms_norm(Tensor x, OptT y, OptT wb, OptT add_vec, OptT next_w, OptT out
   long ys = 0;
   if (y) {
     check_rows(*y, "y");
-    TORCH_CHECK(y->size(0) == rows && y->size(1) == width && wb, "y shape / wb");
-    check_f32(*wb, "wb");
-    TORCH_CHECK(wb->numel() == width, "wb size");
+    TORCH_CHECK(y->size(0) == rows && y->size(1) == width, "y shape");
+    if (wb) {
+      check_f32(*wb, "wb");
+      TORCH_CHECK(wb->numel() == width, "wb size");
+    }
     yp = y->data_ptr();
     ybf = bf(*y);
     ys = y->stride(0);
@@ -401,6 +446,109 @@ void gated_delta_rule(Tensor o, Tensor qkv, Tensor a, Tensor b, Tensor a_log, Te
                     beta.data_ptr<float>(), qkv.data_ptr(), bf(qkv), qkv.stride(0), state.data_ptr<float>(),
                     start.data_ptr<int>(), pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)heads,
                     (int)kv_heads, (int)dk, (int)dv, (int)state.size(0), stream()), "delta_rule");
+}
+
+void conv_delta_prep(Tensor qn, Tensor kn, Tensor vo, Tensor lg, Tensor beta, Tensor x, Tensor a, Tensor b,
+                     Tensor conv_w, Tensor hist, Tensor a_log, Tensor dt_bias, Tensor start, Tensor pos0, Tensor slot,
+                     int64_t num_segs, int64_t max_rows) {
+  for (const Tensor* t : {&qn, &kn, &vo, &lg, &beta, &conv_w, &hist, &a_log, &dt_bias}) check_f32(*t, "conv_delta_prep");
+  check_rows(x, "x");
+  check_rows(a, "a");
+  check_rows(b, "b");
+  const int64_t t = x.size(0), c = x.size(1);
+  TORCH_CHECK(qn.dim() == 3 && kn.sizes() == qn.sizes() && vo.dim() == 3 && qn.size(0) == t && vo.size(0) == t, "q / k / v");
+  const int64_t kvh = qn.size(1), dk = qn.size(2), heads = vo.size(1), dv = vo.size(2);
+  TORCH_CHECK(kvh >= 1 && heads % kvh == 0 && dk >= 1 && dk <= mx_head_max_dk() && dv >= 1 &&
+              c == 2 * kvh * dk + heads * dv && lg.numel() == t * heads && beta.numel() == t * heads &&
+              a.size(0) == t && a.size(1) == heads && b.size(0) == t && b.size(1) == heads &&
+              a.scalar_type() == x.scalar_type() && b.scalar_type() == x.scalar_type() && a_log.numel() == heads &&
+              dt_bias.numel() == heads, "conv_delta_prep shapes");
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(0) == c && conv_w.size(1) >= 1 && conv_w.size(1) <= 16 &&
+              hist.dim() == 3 && hist.size(1) == conv_w.size(1) - 1 && hist.size(2) == c, "conv shapes");
+  check_segs(start, pos0, slot, num_segs);
+  chk(mx_conv_delta_prep(qn.data_ptr<float>(), kn.data_ptr<float>(), vo.data_ptr<float>(), lg.data_ptr<float>(),
+                         beta.data_ptr<float>(), x.data_ptr(), bf(x), x.stride(0), a.data_ptr(), a.stride(0),
+                         b.data_ptr(), b.stride(0), conv_w.data_ptr<float>(), (int)conv_w.size(1),
+                         hist.data_ptr<float>(), a_log.data_ptr<float>(), dt_bias.data_ptr<float>(),
+                         start.data_ptr<int>(), pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs,
+                         (int)max_rows, t, (int)hist.size(0), (int)heads, (int)kvh, (int)dk, (int)dv, stream()),
+      "conv_delta_prep");
+}
+
+// chunks of mx_chunk_rows() rows that the segments of a step of t rows are cut into, at most
+int64_t chunk_bound(int64_t t, int64_t num_segs) { return t / mx_chunk_rows() + num_segs; }
+
+void head_delta_rule(Tensor o, Tensor q, Tensor k, Tensor v, Tensor lg, Tensor beta, Tensor state, Tensor start,
+                     Tensor pos0, Tensor slot, int64_t num_segs, int64_t max_rows, bool walk, int64_t chunk_from) {
+  for (const Tensor* t : {&o, &q, &k, &v, &lg, &beta, &state}) check_f32(*t, "head_delta_rule");
+  TORCH_CHECK(q.dim() == 3 && k.sizes() == q.sizes() && v.dim() == 3 && v.size(0) == q.size(0), "q / k / v");
+  const int64_t t = q.size(0), kvh = q.size(1), dk = q.size(2), heads = v.size(1), dv = v.size(2);
+  TORCH_CHECK(kvh >= 1 && heads >= 1 && heads % kvh == 0 && dk >= 1 && dk <= mx_head_max_dk() && dv >= 1 &&
+              o.numel() == t * heads * dv && lg.numel() == t * heads && beta.numel() == t * heads && max_rows <= t &&
+              chunk_from >= 1, "delta rule shapes");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == heads && state.size(2) == dk && state.size(3) == dv, "state");
+  check_segs(start, pos0, slot, num_segs);
+  const bool chunks = max_rows >= chunk_from && dk <= mx_chunk_max_dk();
+  if (walk || !chunks)
+    chk(mx_head_delta_walk(o.data_ptr<float>(), q.data_ptr<float>(), k.data_ptr<float>(), v.data_ptr<float>(),
+                           lg.data_ptr<float>(), beta.data_ptr<float>(), state.data_ptr<float>(), start.data_ptr<int>(),
+                           pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)heads, (int)kvh, (int)dk,
+                           (int)dv, (int)state.size(0), chunks ? (int)chunk_from : 0, stream()), "delta rule walk");
+  if (!chunks) return;
+  const int64_t nc = chunk_bound(t, num_segs), dkp = mx_chunk_key_pad((int)dk), c = mx_chunk_rows();
+  Tensor ws_s = at::empty({nc, heads, dk, dv}, o.options()), ws_w = at::empty({nc, heads, c, dkp}, o.options());
+  Tensor ws_k = at::empty({nc, heads, dkp, c}, o.options()), ws_u = at::empty({t, heads, dv}, o.options());
+  Tensor ws_g = at::empty({nc, heads}, o.options());
+  chk(mx_head_delta_chunks(o.data_ptr<float>(), q.data_ptr<float>(), k.data_ptr<float>(), v.data_ptr<float>(),
+                           lg.data_ptr<float>(), beta.data_ptr<float>(), state.data_ptr<float>(),
+                           ws_s.data_ptr<float>(), ws_w.data_ptr<float>(), ws_k.data_ptr<float>(),
+                           ws_u.data_ptr<float>(), ws_g.data_ptr<float>(), start.data_ptr<int>(), pos0.data_ptr<int>(),
+                           slot.data_ptr<int>(), (int)num_segs, (int)max_rows, (int)heads, (int)kvh, (int)dk, (int)dv,
+                           (int)state.size(0), (int)chunk_from, stream()), "delta rule chunks");
+}
+
+void retention(Tensor o, Tensor p, OptT table, int64_t rot_dims, bool interleaved, Tensor log_decay, Tensor state,
+               Tensor start, Tensor pos0, Tensor slot, int64_t num_segs, int64_t max_rows, int64_t heads, int64_t dk,
+               int64_t dv, bool walk, int64_t chunk_from) {
+  check_f32(o, "o");
+  check_f32(state, "state");
+  check_rows(p, "p");
+  const int64_t t = p.size(0);
+  TORCH_CHECK(heads >= 1 && dk >= 1 && dk <= mx_head_max_dk() && dv >= 1 && p.size(1) >= heads * (2 * dk + dv) &&
+              o.numel() == t * heads * dv && max_rows <= t && chunk_from >= 1, "retention shapes");
+  TORCH_CHECK(log_decay.is_cuda() && log_decay.scalar_type() == at::kDouble && log_decay.is_contiguous() &&
+              log_decay.numel() == heads, "log_decay: fp64 [heads]");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == heads && state.size(2) == dk && state.size(3) == dv, "state");
+  check_segs(start, pos0, slot, num_segs);
+  const RopeArg rope = rope_arg(table, rot_dims, dk);
+  const bool chunks = max_rows >= chunk_from && dk <= mx_chunk_max_dk();
+  if (walk || !chunks)
+    chk(mx_retention_walk(o.data_ptr<float>(), p.data_ptr(), bf(p), p.stride(0), rope.table, rope.rows, rope.dims,
+                          interleaved ? 1 : 0, log_decay.data_ptr<double>(), state.data_ptr<float>(),
+                          start.data_ptr<int>(), pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)heads,
+                          (int)dk, (int)dv, (int)state.size(0), chunks ? (int)chunk_from : 0, stream()),
+        "retention walk");
+  if (!chunks) return;
+  Tensor ws_s = at::empty({chunk_bound(t, num_segs), heads, dk, dv}, o.options());
+  chk(mx_retention_chunks(o.data_ptr<float>(), p.data_ptr(), bf(p), p.stride(0), rope.table, rope.rows, rope.dims,
+                          interleaved ? 1 : 0, log_decay.data_ptr<double>(), state.data_ptr<float>(),
+                          ws_s.data_ptr<float>(), start.data_ptr<int>(), pos0.data_ptr<int>(), slot.data_ptr<int>(),
+                          (int)num_segs, (int)max_rows, (int)heads, (int)dk, (int)dv, (int)state.size(0),
+                          (int)chunk_from, stream()), "retention chunks");
+}
+
+void scaled_pair_rows(Tensor out, Tensor a, double a_scale, Tensor o, Tensor gate, double o_scale, double eps,
+                      int64_t heads, int64_t dv) {
+  check_f32(a, "a");
+  check_f32(o, "o");
+  check_rows(gate, "gate");
+  TORCH_CHECK(a.dim() == 2 && o.dim() == 2 && heads >= 1 && dv >= 1 && o.size(0) == a.size(0) &&
+              o.size(1) == heads * dv && gate.sizes() == o.sizes(), "scaled_pair_rows shapes");
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.scalar_type() == gate.scalar_type() && out.dim() == 2 &&
+              out.size(0) == a.size(0) && out.size(1) == a.size(1) + heads * dv, "out");
+  chk(mx_scaled_pair_rows(out.data_ptr(), bf(out), a.data_ptr<float>(), (int)a.size(1), (float)a_scale,
+                          o.data_ptr<float>(), gate.data_ptr(), gate.stride(0), (float)o_scale, a.size(0), (int)heads,
+                          (int)dv, (float)eps, stream()), "scaled_pair_rows");
 }
 
 void gated_linear_attention(Tensor o, Tensor qkv, Tensor a, Tensor a_bias, double tau, Tensor state, Tensor start,
@@ -607,24 +755,32 @@ void moe_topk(Tensor idx, Tensor wts, Tensor z, Tensor corr, int64_t top, int64_
                   z.size(0), (int)z.size(1), (int)top, (int)groups, (int)keep, stream()), "moe_topk");
 }
 
-void moe_top_logits(Tensor idx, Tensor wts, Tensor z, int64_t top, bool sigmoid, double scale) {
+void check_groups(int64_t experts, int64_t top, bool sigmoid, int64_t groups, int64_t keep) {
+  TORCH_CHECK(groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups && top <= experts / groups * keep &&
+              (keep == groups || sigmoid), "expert groups");
+}
+
+void moe_top_logits(Tensor idx, Tensor wts, Tensor z, int64_t top, bool sigmoid, double scale, int64_t groups,
+                    int64_t keep) {
   check_i32(idx, "idx");
   check_f32(wts, "wts");
   check_f32(z, "z");
   TORCH_CHECK(z.dim() == 2 && top >= 1 && top <= z.size(1) && idx.numel() == z.size(0) * top &&
               wts.numel() == z.size(0) * top, "moe_top_logits shapes");
+  check_groups(z.size(1), top, sigmoid, groups, keep);
   chk(mx_moe_top_logits(idx.data_ptr<int>(), wts.data_ptr<float>(), z.data_ptr<float>(), z.size(0), (int)z.size(1),
-                        (int)top, sigmoid ? 1 : 0, (float)scale, stream()), "moe_top_logits");
+                        (int)top, sigmoid ? 1 : 0, (float)scale, (int)groups, (int)keep, stream()), "moe_top_logits");
 }
 
 void moe_route_top_logits(Tensor idx, Tensor wts, Tensor h, Tensor router, OptT bias, int64_t top,
-                          bool sigmoid, double scale) {
+                          bool sigmoid, double scale, int64_t groups, int64_t keep) {
   check_i32(idx, "idx");
   check_f32(wts, "wts");
   check_rows(h, "h");
   check_f32(router, "router");
   TORCH_CHECK(router.dim() == 2 && router.size(1) == h.size(1) && top >= 1 && top <= router.size(0) &&
               idx.numel() == h.size(0) * top && wts.numel() == h.size(0) * top, "moe_route_top_logits shapes");
+  check_groups(router.size(0), top, sigmoid, groups, keep);
   if (bias) {
     check_f32(*bias, "router bias");
     TORCH_CHECK(bias->numel() == router.size(0), "router bias size");
@@ -632,7 +788,7 @@ void moe_route_top_logits(Tensor idx, Tensor wts, Tensor h, Tensor router, OptT 
   chk(mx_moe_route_top_logits(idx.data_ptr<int>(), wts.data_ptr<float>(), h.data_ptr(), bf(h), h.stride(0),
                               router.data_ptr<float>(), bias ? bias->data_ptr<float>() : nullptr, h.size(0),
                               (int)router.size(0), (int)router.size(1), (int)top, sigmoid ? 1 : 0, (float)scale,
-                              stream()), "moe_route_top_logits");
+                              (int)groups, (int)keep, stream()), "moe_route_top_logits");
 }
 
 // act 0: clamped GLU, 1: relu^2 (the experts' first matrix is [ff, width], up alone, instead of
@@ -733,8 +889,9 @@ void attn_prep(Tensor q, Tensor qkv, int64_t nq, int64_t nk, OptT wq, OptT wk, d
 }
 
 void conv_attn_prep(Tensor q, Tensor qkv, int64_t nq, int64_t nk, Tensor conv_w, Tensor hist, Tensor start,
-                    Tensor pos0, Tensor slot, int64_t num_segs, OptT wq, OptT wk, double eps, int64_t head_dim,
-                    Tensor slots, Tensor k_cache, Tensor v_cache) {
+                    Tensor pos0, Tensor slot, int64_t num_segs, int64_t max_rows, OptT wq, OptT wk, double eps,
+                    int64_t head_dim, Tensor slots, Tensor k_cache, Tensor v_cache, OptT table, int64_t rot_dims,
+                    bool interleaved) {
   check_f32(q, "q");
   check_rows(qkv, "qkv");
   check_i32(slots, "slot_mapping");
@@ -751,18 +908,20 @@ void conv_attn_prep(Tensor q, Tensor qkv, int64_t nq, int64_t nk, Tensor conv_w,
   check_cache(v_cache, nv, "v_cache");
   TORCH_CHECK(k_cache.scalar_type() == v_cache.scalar_type() && k_cache.size(0) == v_cache.size(0) &&
               k_cache.size(1) == v_cache.size(1), "k / v caches differ");
+  const RopeArg rope = rope_arg(table, rot_dims, head_dim);
   chk(mx_conv_attn_prep(q.data_ptr<float>(), qkv.data_ptr(), bf(qkv), qkv.stride(0), (int)nq, (int)nk, (int)nv,
                         conv_w.data_ptr<float>(), (int)taps, hist.data_ptr<float>(), start.data_ptr<int>(),
-                        pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)hist.size(0),
+                        pos0.data_ptr<int>(), slot.data_ptr<int>(), (int)num_segs, (int)max_rows, (int)hist.size(0),
                         opt_f32(wq, head_dim, "q norm"), opt_f32(wk, head_dim, "k norm"), (float)eps, (int)head_dim,
                         slots.data_ptr<int>(), k_cache.data_ptr(), v_cache.data_ptr(), bf(k_cache),
-                        k_cache.size(0) * k_cache.size(1), t, stream()), "conv_attn_prep");
+                        k_cache.size(0) * k_cache.size(1), rope.table, rope.rows, rope.dims, interleaved ? 1 : 0, t,
+                        stream()), "conv_attn_prep");
 }
 
 void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor start, Tensor pos0, Tensor kv_len,
                       Tensor bt, int64_t num_segs, int64_t max_rows, int64_t heads, int64_t maps, int64_t kv_heads,
                       int64_t dk, int64_t dv, int64_t window, double scale, bool sigmoid, OptT r1, OptT r2, OptT pb,
-                      int64_t skip_from, double softcap, c10::optional<double> sink, bool blocks,
+                      int64_t skip_from, double softcap, c10::optional<double> sink, OptT sinks, bool blocks,
                       int64_t keep_first, OptT dist_bias) {
   check_f32(out, "out");
   check_f32(q, "q");
@@ -789,7 +948,8 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache, Tens
                           bt.data_ptr<int>(), (int)bt.size(1), (int)num_segs, t, (int)heads, (int)maps, (int)kv_heads,
                           (int)dk, (int)dv, (int)window, (float)scale, sigmoid ? 1 : 0, opt_f32(r1, hq, "r1"),
                           opt_f32(r2, hq, "r2"), opt_f32(pb, hq, "pb"), (int)k_cache.size(1), (int)k_cache.size(0),
-                          (int)skip_from, (float)softcap, sink ? 1 : 0, sink ? (float)*sink : 0.f, blocks ? 1 : 0,
+                          (int)skip_from, (float)softcap, sink || sinks ? 1 : 0, sink ? (float)*sink : 0.f,
+                          opt_f32(sinks, hq, "sinks"), blocks ? 1 : 0,
                           (int)keep_first, dist_bias ? dist_bias->data_ptr<float>() : nullptr,
                           dist_bias ? (int)dist_bias->size(0) : 0, stream()),
       "window_attention");
@@ -797,8 +957,8 @@ void window_attention(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache, Tens
 
 void band_weights(Tensor S, int64_t rows, int64_t first_pos, int64_t key0, int64_t heads, int64_t maps,
                   int64_t kv_heads, int64_t window, double scale, bool sigmoid, OptT r1, OptT r2, OptT pb,
-                  double softcap, c10::optional<double> sink, bool blocks, int64_t keep_first, int64_t ext,
-                  OptT dist_bias) {
+                  double softcap, c10::optional<double> sink, OptT sinks, bool blocks, int64_t keep_first,
+                  int64_t ext, OptT dist_bias) {
   check_f32(S, "S");
   TORCH_CHECK(keep_first >= 0 && ext >= 0 && ext <= key0 && ext <= S.size(2) && (!blocks || window >= 1),
               "band_weights mask");
@@ -814,8 +974,9 @@ void band_weights(Tensor S, int64_t rows, int64_t first_pos, int64_t key0, int64
   const int64_t hq = heads * maps;
   chk(mx_band_weights(S.data_ptr<float>(), (int)S.size(0), (int)S.size(1), (int)rows, (int)S.size(2), (int)first_pos,
                       (int)key0, (int)heads, (int)maps, (int)kv_heads, (int)window, (float)scale, sigmoid ? 1 : 0,
-                      opt_f32(r1, hq, "r1"), opt_f32(r2, hq, "r2"), opt_f32(pb, hq, "pb"), (float)softcap, sink ? 1 : 0,
-                      sink ? (float)*sink : 0.f, blocks ? 1 : 0, (int)keep_first, (int)ext,
+                      opt_f32(r1, hq, "r1"), opt_f32(r2, hq, "r2"), opt_f32(pb, hq, "pb"), (float)softcap,
+                      sink || sinks ? 1 : 0, sink ? (float)*sink : 0.f, opt_f32(sinks, hq, "sinks"), blocks ? 1 : 0,
+                      (int)keep_first, (int)ext,
                       dist_bias ? dist_bias->data_ptr<float>() : nullptr, dist_bias ? (int)dist_bias->size(0) : 0,
                       stream()), "band_weights");
 }
@@ -1030,6 +1191,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("scale_add_rows", &scale_add_rows);
   m.def("short_conv_silu", &short_conv_silu);
   m.def("gated_delta_rule", &gated_delta_rule);
+  m.def("conv_delta_prep", &conv_delta_prep);
+  m.def("head_delta_rule", &head_delta_rule);
+  m.def("retention", &retention);
+  m.def("scaled_pair_rows", &scaled_pair_rows);
+  m.def("head_max_dk", []() { return (int64_t)mx_head_max_dk(); });
   m.def("gated_linear_attention", &gated_linear_attention);
   m.def("pair_embed_add", &pair_embed_add);
   m.def("add_scaled_rms_norm", &add_scaled_rms_norm);

@@ -54,17 +54,19 @@ __global__ void short_conv_kernel(T* __restrict__ out, const T* __restrict__ x, 
 }
 
 // history <- the segment's last taps-1 inputs (older ones shift out); runs after
-// short_conv_kernel, one thread per (segment, channel)
+// short_conv_kernel, one thread per (segment, channel); segments of fewer than min_rows rows
+// are left alone
 template <typename T>
 __global__ void conv_hist_kernel(const T* __restrict__ x, long x_stride, float* __restrict__ hist,
                                  const int* __restrict__ start, const int* __restrict__ pos0,
-                                 const int* __restrict__ slot, int channels, int taps, int num_slots) {
+                                 const int* __restrict__ slot, int channels, int taps, int num_slots,
+                                 int min_rows) {
   const int s = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= channels) return;
   const int sl = slot[s];
   const int r0 = start[s], n = start[s + 1] - r0;
-  if (sl < 0 || sl >= num_slots || n <= 0) return;
+  if (sl < 0 || sl >= num_slots || n < min_rows) return;
   const bool fresh = pos0[s] <= 0;
   float* h = hist + (long)sl * (taps - 1) * channels;
   float keep[kMaxTaps];
@@ -284,18 +286,19 @@ extern "C" int mx_short_conv_silu(void* out, const void* x, int bf16, long x_str
   if (taps > 1)
     MX_DISPATCH_T(bf16, hipLaunchKernelGGL((conv_hist_kernel<T>), dim3((channels + 255) / 256, num_segs),
                                            block, 0, s, (const T*)x, x_stride, hist, start, pos0, slot,
-                                           channels, taps, num_slots));
+                                           channels, taps, num_slots, 1));
   return (int)hipGetLastError();
 }
 
 // history update alone, for kernels that fuse the convolution into a larger step
 extern "C" int mx_conv_hist(const void* x, int bf16, long x_stride, float* hist, const int* start, const int* pos0,
-                            const int* slot, int num_segs, int channels, int taps, int num_slots, hipStream_t s) {
+                            const int* slot, int num_segs, int channels, int taps, int num_slots, int min_rows,
+                            hipStream_t s) {
   if (num_segs <= 0 || channels <= 0 || taps <= 1) return 0;
   if (taps > kMaxTaps || num_segs > 65535) return -1;
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((conv_hist_kernel<T>), dim3((channels + 255) / 256, num_segs), dim3(256),
                                          0, s, (const T*)x, x_stride, hist, start, pos0, slot, channels, taps,
-                                         num_slots));
+                                         num_slots, min_rows < 1 ? 1 : min_rows));
   return (int)hipGetLastError();
 }
 

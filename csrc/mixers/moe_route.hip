@@ -6,7 +6,8 @@
 // unbiased softmax scores, not renormalised.  One wave per token; ties go to the lower
 // index.  A second router (moe_top_logits) chooses on the logits and weights the chosen ones
 // by the softmax over just those, or by their sigmoids divided by the sum of those, times a
-// factor.
+// factor; there, too, the choice may be limited to the best groups, a group's score being the
+// sum of its two largest sigmoids.
 #include "mx_common.h"
 
 namespace mx {
@@ -92,6 +93,34 @@ moe_topk_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __r
   }
 }
 
+// One wave: the logits ch of every expert outside the `keep` best of `groups` equal groups
+// become -inf.  A group's score is the sum of the sigmoids of its two largest logits (of its
+// only one in a group of one); gs holds `groups` scores.
+__device__ __forceinline__ void limit_to_best_groups(float* ch, float* gs, int experts, int groups, int keep, int lane) {
+  const int gsz = experts / groups;
+  for (int g = lane; g < groups; g += 64) {
+    float a = -INFINITY, b = -INFINITY;
+    for (int e = g * gsz; e < (g + 1) * gsz; ++e) {
+      const float v = ch[e];
+      if (v > a) { b = a; a = v; }
+      else b = fmaxf(b, v);
+    }
+    gs[g] = sigmoidf_(a) + (gsz > 1 ? sigmoidf_(b) : 0.f);
+  }
+  wave_lds_fence();
+  for (int k = 0; k < keep; ++k) {       // a kept group is marked by +inf
+    Best b{-INFINITY, 1 << 30};
+    for (int g = lane; g < groups; g += 64)
+      if (gs[g] != INFINITY) b = better(b, Best{gs[g], g});
+    b = wave_best(b);
+    if (lane == 0 && b.i < groups) gs[b.i] = INFINITY;
+    wave_lds_fence();
+  }
+  for (int e = lane; e < experts; e += 64)
+    if (gs[e / gsz] != INFINITY) ch[e] = -INFINITY;
+  wave_lds_fence();
+}
+
 // weights of the chosen logits val[0 .. top) (largest first), one wave
 __device__ __forceinline__ void chosen_weights(float* w, const float* val, int top, int lane, int sigmoid, float scale) {
   auto f = [&](int k) { return sigmoid ? sigmoidf_(val[k]) : expf(val[k] - val[0]); };
@@ -106,7 +135,7 @@ __device__ __forceinline__ void chosen_weights(float* w, const float* val, int t
 // the lower index) and weighted by chosen_weights.  One wave per token.
 __global__ void __launch_bounds__(64)
 moe_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const float* __restrict__ z, int experts,
-                      int top, int sigmoid, float scale) {
+                      int top, int sigmoid, float scale, int groups, int keep) {
   extern __shared__ float sm[];
   float* ch = sm;                   // logits, -inf once taken
   float* val = sm + experts;        // the chosen logits, largest first
@@ -115,6 +144,7 @@ moe_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const floa
   const float* zr = z + row * experts;
   for (int e = lane; e < experts; e += 64) ch[e] = zr[e];
   __syncthreads();
+  if (keep < groups) limit_to_best_groups(ch, val + top, experts, groups, keep, lane);
   for (int k = 0; k < top; ++k) {
     Best b{-INFINITY, 1 << 30};
     for (int e = lane; e < experts; e += 64) b = better(b, Best{ch[e], e});
@@ -153,7 +183,7 @@ template <typename T>
 __global__ void __launch_bounds__(64 * kRouteWaves)
 moe_route_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, const T* __restrict__ h, long h_stride,
                             const float* __restrict__ router, const float* __restrict__ bias, int experts,
-                            int width, int top, int vec, int sigmoid, float scale) {
+                            int width, int top, int vec, int sigmoid, float scale, int groups, int keep) {
   extern __shared__ float sm[];
   float* ch = sm;
   float* val = sm + experts;
@@ -181,6 +211,7 @@ moe_route_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, cons
   if (wave != 0) return;
   // one wave from here on: lane 0's LDS writes are made visible to the wave's other lanes
   // by a wave-level fence instead of a workgroup barrier
+  if (keep < groups) limit_to_best_groups(ch, val + top, experts, groups, keep, lane);
   for (int k = 0; k < top; ++k) {
     Best b{-INFINITY, 1 << 30};
     for (int e = lane; e < experts; e += 64) b = better(b, Best{ch[e], e});
@@ -202,28 +233,30 @@ moe_route_top_logits_kernel(int* __restrict__ idx, float* __restrict__ wts, cons
 
 extern "C" int mx_moe_route_top_logits(int* idx, float* wts, const void* h, int bf16, long h_stride,
                                        const float* router, const float* bias, long rows, int experts, int width,
-                                       int top, int sigmoid, float scale, hipStream_t s) {
+                                       int top, int sigmoid, float scale, int groups, int keep, hipStream_t s) {
   if (rows <= 0) return 0;
   if (experts < 1 || top < 1 || top > experts || width < 1) return -1;
-  const size_t lds = (size_t)(experts + top) * sizeof(float);
+  if (groups < 1 || experts % groups || keep < 1 || keep > groups || top > experts / groups * keep) return -1;
+  const size_t lds = (size_t)(experts + top + groups) * sizeof(float);
   if (lds > 60 * 1024) return -2;
   const long es = bf16 ? 2 : 4;
   const int vec = width % 4 == 0 && h_stride % 4 == 0 && ((uintptr_t)h) % (4 * es) == 0 &&
                   ((uintptr_t)router) % 16 == 0;
   MX_DISPATCH_T(bf16, hipLaunchKernelGGL((mx::moe_route_top_logits_kernel<T>), dim3((unsigned)rows),
                                          dim3(64 * mx::kRouteWaves), lds, s, idx, wts, (const T*)h, h_stride, router,
-                                         bias, experts, width, top, vec, sigmoid, scale));
+                                         bias, experts, width, top, vec, sigmoid, scale, groups, keep));
   return (int)hipGetLastError();
 }
 
 extern "C" int mx_moe_top_logits(int* idx, float* wts, const float* z, long rows, int experts, int top,
-                                 int sigmoid, float scale, hipStream_t s) {
+                                 int sigmoid, float scale, int groups, int keep, hipStream_t s) {
   if (rows <= 0) return 0;
   if (experts < 1 || top < 1 || top > experts) return -1;
-  const size_t lds = (size_t)(experts + top) * sizeof(float);
+  if (groups < 1 || experts % groups || keep < 1 || keep > groups || top > experts / groups * keep) return -1;
+  const size_t lds = (size_t)(experts + top + groups) * sizeof(float);
   if (lds > 60 * 1024) return -2;
   hipLaunchKernelGGL(mx::moe_top_logits_kernel, dim3((unsigned)rows), dim3(64), lds, s, idx, wts, z, experts, top,
-                     sigmoid, scale);
+                     sigmoid, scale, groups, keep);
   return (int)hipGetLastError();
 }
 

@@ -2,7 +2,7 @@
 // sinusoidal position vector), the fused "post-norm add + next pre-norm" step (also with a
 // token shift of the normed row), the layer
 // norm (weight and bias) that adds a sublayer's output to the residual, the tanh cap of
-// the logits, per-head gated output norm, activations
+// the logits, per-head gated output norm (alone, or beside a second mixer's scaled rows), activations
 // (relu^2, clamped / gelu / relu / silu GLU, gelu * token-side embedding) and the weighted row scatter-add
 // that combines expert outputs.
 #include <type_traits>
@@ -263,7 +263,7 @@ __device__ __forceinline__ float sum_sq(const float (&v)[C][4]) {
   return s;
 }
 
-// residual (fp32, in place): x += rms_norm(y) * wb (+ add_vec);
+// residual (fp32, in place): x += rms_norm(y) * wb (y as it is without wb) (+ add_vec);
 // out = rms_norm(x) * next_w (TO);  cast = x (TO).  Every part is optional.
 template <typename TY, typename TO, int NT, int C>
 __global__ void __launch_bounds__(NT)
@@ -276,12 +276,18 @@ add_rms_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, long y_stri
   load_row<float, NT, C>(v, x + row * width, width, vec);
   if (y != nullptr) {
     load_row<TY, NT, C>(t, y + row * y_stride, width, vec);
-    load_row<float, NT, C>(w, wb, width, vec);
-    const float r = 1.0f / sqrtf(block_sum<NT>(sum_sq<C>(t), red) / (float)width + eps);
+    if (wb != nullptr) {
+      load_row<float, NT, C>(w, wb, width, vec);
+      const float r = 1.0f / sqrtf(block_sum<NT>(sum_sq<C>(t), red) / (float)width + eps);
+#pragma unroll
+      for (int c = 0; c < C; ++c)
+#pragma unroll
+        for (int k = 0; k < 4; ++k) t[c][k] *= r * w[c][k];
+    }
 #pragma unroll
     for (int c = 0; c < C; ++c)
 #pragma unroll
-      for (int k = 0; k < 4; ++k) v[c][k] += t[c][k] * r * w[c][k];
+      for (int k = 0; k < 4; ++k) v[c][k] += t[c][k];
   }
   if (add_vec != nullptr) {
     load_row<float, NT, C>(w, add_vec, width, vec);
@@ -415,6 +421,37 @@ __global__ void head_rms_gate_kernel(TO* __restrict__ out, const float* __restri
     const float gp = ld(gate, row * gate_stride + (long)h * dv + i);
     const float g = silu ? gp * sigmoidf_(gp) : sigmoidf_(gp);
     st(out, (row * heads + h) * dv + i, op[i] * r * w[i] * g);
+  }
+}
+
+// rows [a_scale * a (n) | o_scale * o / rms(o) per head * silu(gate)]: one wave per (row, item),
+// items are the heads of o, then pieces of 256 columns of a
+template <typename T>
+__global__ void scaled_pair_rows_kernel(T* __restrict__ out, const float* __restrict__ a, int n, float a_scale,
+                                        const float* __restrict__ o, const T* __restrict__ gate, long gate_stride,
+                                        float o_scale, long waves, int items, int heads, int dv, float eps) {
+  const long w = (long)blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
+  if (w >= waves) return;
+  const int lane = threadIdx.x & 63;
+  const long row = w / items;
+  const int it = (int)(w % items);
+  T* orow = out + row * (n + (long)heads * dv);
+  if (it >= heads) {
+    const int c0 = (it - heads) * 256;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = c0 + lane + 64 * u;
+      if (c < n) st(orow, c, a[row * n + c] * a_scale);
+    }
+    return;
+  }
+  const float* op = o + (row * heads + it) * dv;
+  float ss = 0.f;
+  for (int i = lane; i < dv; i += 64) ss += op[i] * op[i];
+  const float r = 1.0f / sqrtf(ft::wave_sum(ss) / (float)dv + eps) * o_scale;
+  for (int i = lane; i < dv; i += 64) {
+    const float g = ld(gate, row * gate_stride + (long)it * dv + i);
+    st(orow, n + (long)it * dv + i, op[i] * r * (g * sigmoidf_(g)));
   }
 }
 
@@ -604,6 +641,18 @@ extern "C" int mx_head_rms_gate(void* out, int out_bf16, const float* o, const f
                        (const float*)gate, gate_stride, pairs, heads, dv, eps, silu);
   else
     return -1;
+  return (int)hipGetLastError();
+}
+
+extern "C" int mx_scaled_pair_rows(void* out, int bf16, const float* a, int n, float a_scale, const float* o,
+                                   const void* gate, long gate_stride, float o_scale, long rows, int heads, int dv,
+                                   float eps, hipStream_t s) {
+  const int items = heads + (n + 255) / 256;
+  const long waves = rows * items;
+  if (waves <= 0) return 0;
+  const dim3 grid((unsigned)((waves + 3) / 4)), block(256);
+  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((scaled_pair_rows_kernel<T>), grid, block, 0, s, (T*)out, a, n, a_scale, o,
+                                         (const T*)gate, gate_stride, o_scale, waves, items, heads, dv, eps));
   return (int)hipGetLastError();
 }
 

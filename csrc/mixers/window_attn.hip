@@ -10,11 +10,12 @@
 // s = q.k * scale, capped to softcap tanh(s / softcap) when softcap > 0;
 // score = s - r1[a] ln(1 + r2[a] (i - j)) + dist_bias[min(i - j, nd - 1)][a]; weight =
 // softmax over the visible keys, or sigmoid(score + pb[a]) unnormalised.  A softmax may carry a sink: one more
-// term exp(sink) in its denominator, a key that is always visible and has no value.
+// term exp(sink) (the same for all heads, or sinks[a]) in its denominator, a key that is always
+// visible and has no value.
 // Queries, scores, weights and sums are fp32; the caches hold fp32 or bf16 rows.
 //
 // Kernels: attn_prep (whole-projection RMS norms, rotary positions, cache writes),
-// conv_attn_prep (short causal convolution over time, per-head RMS norms, cache writes),
+// conv_attn_prep (short causal convolution over time, per-head RMS norms, rotary positions, cache writes),
 // window_attn (one workgroup per (row, query head): decode rows and short segments),
 // band_weights (scores -> weights for the banded matrix products of long segments) and
 // diff_combine (two maps -> one gated, normed head output).
@@ -91,19 +92,21 @@ __global__ void attn_prep_kernel(float* __restrict__ q_out, const T* __restrict_
 // of q or k (head_dim channels) or up to head_dim channels of v: a causal convolution
 // over time on every channel (taps along the row axis, the last tap on the row itself;
 // rows before the segment's first come from the state slot's history, zeros at position
-// 0), then, for q and k, the head's RMS norm with one weight vector shared by the heads,
-// fp32 throughout.  The convolved chunk waits in the wave's LDS strip between the two
-// passes.  q leaves as fp32, k and v go to the row's cache slot.  The history is
-// updated afterwards by mx_conv_hist.  grid (rows, ceil(chunks / 4)), 4 waves.
+// 0), then, for q and k, the head's RMS norm with one weight vector shared by the heads and
+// rotary positions (each optional), fp32 throughout.  The convolved chunk waits in the wave's
+// LDS strip between the two passes.  q leaves as fp32, k and v go to the row's cache slot.  A
+// one-row segment shifts its history here (each channel is one lane's own); longer segments'
+// histories are updated afterwards by mx_conv_hist.  grid (rows, ceil(chunks / 4)), 4 waves.
 // ---------------------------------------------------------------------------------
 template <typename T, typename TC>
 __global__ void __launch_bounds__(256)
 conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long stride, int nq, int nk, int nv,
-                      const float* __restrict__ conv_w, int taps, const float* __restrict__ hist,
+                      const float* __restrict__ conv_w, int taps, float* hist,
                       const int* __restrict__ start, const int* __restrict__ pos0, const int* __restrict__ slot,
                       int num_segs, int num_state_slots, const float* __restrict__ wq,
                       const float* __restrict__ wk, float eps, int head_dim, const int* __restrict__ slots,
-                      TC* __restrict__ k_cache, TC* __restrict__ v_cache, long num_slots) {
+                      TC* __restrict__ k_cache, TC* __restrict__ v_cache, long num_slots,
+                      const float* __restrict__ table, int table_rows, int rot_dims, int interleaved) {
   extern __shared__ float smem[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float* y = smem + wave * head_dim;
@@ -113,16 +116,12 @@ conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long
   const int ch = blockIdx.y * 4 + wave;
   const int row = blockIdx.x;
   if (ch >= chunks || row >= start[num_segs]) return;
-  int lo_s = 0, hi_s = num_segs;
-  while (hi_s - lo_s > 1) {
-    const int mid = (lo_s + hi_s) >> 1;
-    if (start[mid] <= row) lo_s = mid; else hi_s = mid;
-  }
-  const int s = lo_s;
-  const int r0 = start[s], rel = row - r0;
+  const int s = segment_of(start, num_segs, row);
+  const int r0 = start[s], n = start[s + 1] - r0, rel = row - r0;
   const int sl = slot[s];
-  const bool old = sl >= 0 && sl < num_state_slots && pos0[s] > 0;   // the slot's history counts
-  const float* h = hist + (long)(old ? sl : 0) * (taps - 1) * channels;
+  const bool mine = sl >= 0 && sl < num_state_slots;
+  const bool old = mine && pos0[s] > 0;                              // the slot's history counts
+  float* h = hist + (long)(mine ? sl : 0) * (taps - 1) * channels;
   const int c0 = ch * head_dim;
   const int len = min(head_dim, channels - c0);
   float ss = 0.f;
@@ -136,7 +135,11 @@ conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long
       else v = old ? h[(long)(taps - 1 + src) * channels + c] : 0.f;
       acc += v * conv_w[(long)c * taps + j];
     }
-    y[i] = acc;                        // each lane re-reads only what it wrote itself
+    if (mine && n == 1) {
+      for (int m = 0; m + 1 < taps - 1; ++m) h[(long)m * channels + c] = old ? h[(long)(m + 1) * channels + c] : 0.f;
+      if (taps > 1) h[(long)(taps - 2) * channels + c] = ld(qkv, (long)row * stride + c);
+    }
+    y[i] = acc;
     ss += acc * acc;
   }
   const long cs = slots[row];
@@ -146,8 +149,18 @@ conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long
     const float* w = is_q ? wq : wk;
     float r = 1.f;
     if (w != nullptr) r = 1.0f / sqrtf(ft::wave_sum(ss) / (float)head_dim + eps);
+    const float* trow = nullptr;
+    if (table != nullptr) {
+      if (w != nullptr)
+        for (int i = lane; i < len; i += 64) y[i] *= r * w[i];
+      int pos = pos0[s] + rel;
+      if (pos < 0 || pos >= table_rows) pos = 0;
+      trow = table + (long)pos * rot_dims;
+      wave_lds_fence();                // rotation pairs cross lanes
+    }
     for (int i = lane; i < len; i += 64) {
-      const float v = w != nullptr ? y[i] * r * w[i] : y[i];
+      const float v = trow != nullptr ? (i < rot_dims ? rope_at(y, i, rot_dims, trow, interleaved) : y[i])
+                                      : w != nullptr ? y[i] * r * w[i] : y[i];
       if (is_q) q_out[(long)row * nq + c0 + i] = v;
       else if (keep) st(k_cache, cs * nk + (c0 - nq) + i, v);
     }
@@ -238,7 +251,7 @@ window_attn_kernel(float* __restrict__ out, const float* __restrict__ q, const T
                    int heads, int maps, int kv_heads, int dk, int dv, int window, float scale, int sigmoid,
                    const float* __restrict__ r1, const float* __restrict__ r2, const float* __restrict__ pb,
                    int block_size, int num_blocks, int skip_from, int vec, int lpk, float softcap, int has_sink,
-                   float sink, int blocks, int keep_first, const float* __restrict__ dist_bias, int nd) {
+                   float sink_all, const float* __restrict__ sinks, int blocks, int keep_first, const float* __restrict__ dist_bias, int nd) {
   extern __shared__ float smem[];
   const int row = blockIdx.x, a = blockIdx.y;
   const int hq = heads * maps;
@@ -366,6 +379,7 @@ window_attn_kernel(float* __restrict__ out, const float* __restrict__ q, const T
 #pragma unroll
       for (int w = 0; w < kWaves; ++w) acc += o_s[w * dv + c];
     } else {
+      const float sink = sinks != nullptr ? sinks[a] : sink_all;
       float mm = has_sink ? sink : -INFINITY;
 #pragma unroll
       for (int w = 0; w < kWaves; ++w) mm = fmaxf(mm, ml_s[2 * w]);
@@ -393,8 +407,8 @@ template <int NT>
 __global__ void band_weights_kernel(float* __restrict__ S, int rows, int keys, int first_pos, int key0,
                                     int heads, int maps, int kv_heads, int window, float scale, int sigmoid,
                                     const float* __restrict__ r1, const float* __restrict__ r2,
-                                    const float* __restrict__ pb, float softcap, int has_sink, float sink,
-                                    int blocks, int keep_first, int ext, const float* __restrict__ dist_bias,
+                                    const float* __restrict__ pb, float softcap, int has_sink, float sink_all,
+                                    const float* __restrict__ sinks, int blocks, int keep_first, int ext, const float* __restrict__ dist_bias,
                                     int nd) {
   __shared__ float red[NT / 64];
   const int rep = heads / kv_heads;
@@ -443,6 +457,7 @@ __global__ void band_weights_kernel(float* __restrict__ S, int rows, int keys, i
   __syncthreads();
 #pragma unroll
   for (int w = 0; w < NT / 64; ++w) mx_ = fmaxf(mx_, red[w]);
+  const float sink = sinks != nullptr ? sinks[a] : sink_all;
   if (has_sink) mx_ = fmaxf(mx_, sink);
   float sum = 0.f;
   for (int u = threadIdx.x; u < nvis; u += NT) {
@@ -506,14 +521,17 @@ extern "C" int mx_attn_prep(float* q_out, const void* qkv, int bf16, long stride
 }
 
 extern "C" int mx_conv_hist(const void* x, int bf16, long x_stride, float* hist, const int* start, const int* pos0,
-                            const int* slot, int num_segs, int channels, int taps, int num_slots, hipStream_t s);
+                            const int* slot, int num_segs, int channels, int taps, int num_slots, int min_rows,
+                            hipStream_t s);
 
 extern "C" int mx_conv_attn_prep(float* q_out, const void* qkv, int bf16, long stride, int nq, int nk, int nv,
                                  const float* conv_w, int taps, float* hist, const int* start, const int* pos0,
-                                 const int* slot, int num_segs, int num_state_slots, const float* wq,
+                                 const int* slot, int num_segs, int max_rows, int num_state_slots, const float* wq,
                                  const float* wk, float eps, int head_dim, const int* slots, void* k_cache,
-                                 void* v_cache, int cache_bf16, long num_slots, long rows, hipStream_t s) {
+                                 void* v_cache, int cache_bf16, long num_slots, const float* table, int table_rows,
+                                 int rot_dims, int interleaved, long rows, hipStream_t s) {
   if (rows <= 0 || num_segs <= 0) return 0;
+  if (rot_dims < 0 || rot_dims % 2 || rot_dims > head_dim || (table != nullptr && table_rows < 1)) return -1;
   if (head_dim < 1 || nq % head_dim || nk % head_dim || taps < 1 || nv < 0) return -1;
   const int channels = nq + nk + nv;
   const size_t shm = (size_t)4 * head_dim * sizeof(float);
@@ -523,15 +541,16 @@ extern "C" int mx_conv_attn_prep(float* q_out, const void* qkv, int bf16, long s
 #define MX_CPREP(T, TC)                                                                                       \
   hipLaunchKernelGGL((conv_attn_prep_kernel<T, TC>), grid, block, shm, s, q_out, (const T*)qkv, stride, nq, nk, \
                      nv, conv_w, taps, hist, start, pos0, slot, num_segs, num_state_slots, wq, wk, eps,         \
-                     head_dim, slots, (TC*)k_cache, (TC*)v_cache, num_slots)
+                     head_dim, slots, (TC*)k_cache, (TC*)v_cache, num_slots, rot_dims > 0 ? table : nullptr, table_rows, \
+                     rot_dims, interleaved)
   if (bf16 && cache_bf16) MX_CPREP(bf16_t, bf16_t);
   else if (bf16) MX_CPREP(bf16_t, float);
   else if (cache_bf16) MX_CPREP(float, bf16_t);
   else MX_CPREP(float, float);
 #undef MX_CPREP
   int rc = (int)hipGetLastError();
-  if (rc == 0 && taps > 1)
-    rc = mx_conv_hist(qkv, bf16, stride, hist, start, pos0, slot, num_segs, channels, taps, num_state_slots, s);
+  if (rc == 0 && taps > 1 && max_rows > 1)
+    rc = mx_conv_hist(qkv, bf16, stride, hist, start, pos0, slot, num_segs, channels, taps, num_state_slots, 2, s);
   return rc;
 }
 
@@ -543,7 +562,8 @@ extern "C" int mx_window_attention(float* out, const float* q, const void* k_cac
                                    int kv_heads, int dk, int dv, int window, float scale, int sigmoid,
                                    const float* r1, const float* r2, const float* pb, int block_size,
                                    int num_blocks, int skip_from, float softcap, int has_sink, float sink,
-                                   int blocks, int keep_first, const float* dist_bias, int nd, hipStream_t s) {
+                                   const float* sinks, int blocks, int keep_first, const float* dist_bias, int nd,
+                                   hipStream_t s) {
   if (num_segs <= 0 || total_rows <= 0) return 0;
   if (dv < 1 || dv > mx_window_max_dv() || dk < 1 || heads % kv_heads || maps < 1) return -1;
   if (keep_first < 0 || (dist_bias != nullptr && nd < 1) || (blocks && window < 1)) return -1;
@@ -566,7 +586,7 @@ extern "C" int mx_window_attention(float* out, const float* q, const void* k_cac
                                                (const T*)k_cache, (const T*)v_cache, start, pos0, kv_len, bt,  \
                                                bt_stride, num_segs, heads, maps, kv_heads, dk, dv, window, scale, \
                                                sigmoid, r1, r2, pb, block_size, num_blocks, skip_from, vec, lpk,  \
-                                               softcap, has_sink, sink, blocks, keep_first, dist_bias, nd))
+                                               softcap, has_sink, sink, sinks, blocks, keep_first, dist_bias, nd))
   if (vecv) MX_WATTN(true);
   else MX_WATTN(false);
 #undef MX_WATTN
@@ -576,8 +596,8 @@ extern "C" int mx_window_attention(float* out, const float* q, const void* k_cac
 extern "C" int mx_band_weights(float* S, int gk, int rep_rows_total, int rows, int keys, int first_pos, int key0,
                                int heads, int maps, int kv_heads, int window, float scale, int sigmoid,
                                const float* r1, const float* r2, const float* pb, float softcap, int has_sink,
-                               float sink, int blocks, int keep_first, int ext, const float* dist_bias, int nd,
-                               hipStream_t s) {
+                               float sink, const float* sinks, int blocks, int keep_first, int ext,
+                               const float* dist_bias, int nd, hipStream_t s) {
   if (gk <= 0 || rep_rows_total <= 0 || keys <= 0) return 0;
   if (heads % kv_heads || gk != kv_heads * maps || rep_rows_total != heads / kv_heads * rows || gk > 65535) return -1;
   if (keep_first < 0 || ext < 0 || ext > keys || ext > key0 || (dist_bias != nullptr && nd < 1) ||
@@ -585,7 +605,7 @@ extern "C" int mx_band_weights(float* S, int gk, int rep_rows_total, int rows, i
     return -1;
   hipLaunchKernelGGL((band_weights_kernel<256>), dim3((unsigned)rep_rows_total, (unsigned)gk), dim3(256), 0, s, S,
                      rows, keys, first_pos, key0, heads, maps, kv_heads, window, scale, sigmoid, r1, r2, pb, softcap,
-                     has_sink, sink, blocks, keep_first, ext, dist_bias, nd);
+                     has_sink, sink, sinks, blocks, keep_first, ext, dist_bias, nd);
   return (int)hipGetLastError();
 }
 

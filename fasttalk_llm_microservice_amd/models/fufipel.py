@@ -228,10 +228,7 @@ class FufipelModel(StackedModel):
         self.final_norm = self.offset_norm_weight(get("final.norm"))
         if cfg.bigram:
             buckets, mul_prev, mul_cur = cfg.bigram
-            table = get("bigram").to(dev, dt).contiguous()
-            if table.shape != (buckets + 1, width):
-                raise ValueError("pair table does not fit its bucket count")
-            self.pair_embed = (table, mul_prev, mul_cur, buckets)
+            self.load_pair_table(get("bigram"), buckets, mul_prev, mul_cur)
         max_pos = max(self.max_model_len, 16) + 1
         self.layers = []
         for i, l in enumerate(cfg.layers):

@@ -1,8 +1,9 @@
 """Reusable sublayers built on :mod:`fasttalk_llm_microservice_amd.ops.mixers`:
 latent attention (paged latent cache), windowed attention with sigmoid weights,
 windowed differential attention, convolved capped attention with a sink and attention that
-mixes its scores across the heads (paged key / value caches), the channel-decay gated
-delta rule and the selective state-space mixer (state slots), dense, gated and
+mixes its scores across the heads (paged key / value caches), the channel-decay and the
+head-decay gated delta rule, retention and the selective state-space mixer (state slots), two
+mixers side by side, dense, gated and
 mixture-of-experts feed-forwards and the per-layer token-side input.
 
 Every mixer owns its cache layout: ``alloc_cache(num_blocks, block_size, dtype,
@@ -18,7 +19,7 @@ in the HIP kernels (GPU) or their PyTorch twins (CPU backend).
 """
 from __future__ import annotations
 
-from typing import Callable, List, Optional
+from typing import Callable, List, Optional, Union
 
 import torch
 import torch.nn.functional as F
@@ -42,6 +43,16 @@ class StepContext:
 def _state_slots(shapes, num_slots: int, device):
     """(recurrent state, convolution history) fp32, one row per state slot."""
     return tuple(torch.zeros((num_slots,) + tuple(sh), dtype=torch.float32, device=device) for sh in shapes)
+
+
+def _product_rows(parts, dtype, device, multiple: int = 8) -> torch.Tensor:
+    """Projections stacked into one product's weight, zero rows up to a multiple of 8 (rows of
+    the product are then whole 16-byte pieces)."""
+    w = torch.cat(list(parts), 0)
+    pad = (-w.shape[0]) % multiple
+    if pad:
+        w = torch.cat([w, torch.zeros(pad, w.shape[1], dtype=w.dtype, device=w.device)], 0)
+    return w.to(device, dtype).contiguous()
 
 
 class LatentAttention:
@@ -187,6 +198,53 @@ class ChannelDelta:
         return F.linear(y, self.wo)
 
 
+class HeadDelta:
+    """Gated delta rule with one decay per head.  q, k (kv_heads x dim) and v (heads x vdim)
+    pass a short causal convolution over time and silu; q and k are made unit vectors; decay
+    exp(-exp(A_log) softplus(W_a h + dt_bias)), step beta = sigmoid(W_b h).  Each head's output
+    is divided by its root mean square, multiplied by one weight vector shared by the heads
+    and by silu(W_g h), then the output projection.  A sequence's slot holds the fp32 state
+    [heads, dim, vdim] and the convolution's last taps - 1 inputs."""
+
+    def __init__(self, get: Get, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float,
+                 dtype, device):
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.heads, self.kvh, self.dk, self.dv, self.taps = heads, kv_heads, dim, vdim, taps
+        self.eps, self.dtype = eps, dtype
+        f32 = lambda n: get(n).to(device, torch.float32).contiguous()   # noqa: E731
+        parts = [get("q"), get("k"), get("v"), get("g"), get("a"), get("b")]
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.win = _product_rows(parts, dtype, device)
+        self.conv_w = torch.cat([f32("q.conv"), f32("k.conv"), f32("v.conv")], 0).contiguous()
+        self.a_log, self.dt_bias, self.norm = f32("A_log"), f32("dt_bias"), f32("norm")
+        self.wo = get("o").to(device, dtype).contiguous()
+        if [p.shape[0] for p in parts] != [kv_heads * dim] * 2 + [heads * vdim] * 2 + [heads] * 2 or \
+                self.conv_w.shape != (self.channels, taps) or self.a_log.numel() != heads or \
+                self.dt_bias.numel() != heads or self.norm.numel() != vdim or self.wo.shape != (width, heads * vdim):
+            raise ValueError("delta-rule projections do not fit the head sizes")
+
+    def state_shapes(self):
+        return (self.heads, self.dk, self.dv), (max(self.taps - 1, 0), self.channels)
+
+    def cache_bytes_per_token(self, elem_bytes: int) -> int:
+        return 0
+
+    def alloc_cache(self, num_blocks, block_size, dtype, num_slots, device):
+        return _state_slots(self.state_shapes(), num_slots, device)
+
+    def __call__(self, h, ctx: StepContext, state) -> torch.Tensor:
+        s_rec, s_conv = state
+        p = F.linear(h, self.win)
+        c, ng, nh = self.channels, self.heads * self.dv, self.heads
+        q, k, v, lg, beta = M.conv_delta_prep(p[:, :c], p[:, c + ng:c + ng + nh], p[:, c + ng + nh:c + ng + 2 * nh],
+                                              self.conv_w, s_conv, self.a_log, self.dt_bias, ctx.seg, nh, self.kvh,
+                                              self.dk, self.dv)
+        o = M.head_delta_rule(q, k, v, lg, beta, s_rec, ctx.seg)
+        y = M.head_rms_gate(o, self.norm, p[:, c:c + ng], self.eps, nh, self.dv, self.dtype, silu=True)
+        return F.linear(y, self.wo)
+
+
 class WindowedAttention:
     """Grouped-query attention over a sliding window of a paged key cache and a paged
     value cache (common part of :class:`SigmoidAttention` and
@@ -306,26 +364,37 @@ class ConvSinkAttention(WindowedAttention):
     """Grouped-query softmax attention over every earlier key (or a window of them) whose
     q, k and v each pass a short per-channel causal convolution over time right after
     their projection (no bias, no activation; the last taps-1 projected rows of a sequence
-    live in its state slot).  Each head's q and k are divided by their root mean square
-    and multiplied by one weight vector shared by all heads.  Positions do not enter the
-    scores: s = softcap tanh(q.k scale / softcap), and the softmax's denominator carries
-    one extra unit, exp(sink) with sink = 0 -- a key that is always visible and has no
-    value, so a row's weights may sum to less than one."""
+    live in its state slot).  ``qk_norm``: each head's q and k are divided by their root mean
+    square and multiplied by one weight vector shared by all heads.  ``rot_dims`` > 0: rotary
+    positions on the first entries of every q and k head (``interleaved`` pairs (2i, 2i + 1),
+    else (i, i + rot_dims/2)); without them positions do not enter the scores.
+    s = q.k scale, with ``softcap`` capped to softcap tanh(s / softcap), and the softmax's
+    denominator carries one extra term exp(sink) (0, another number, or ``sink`` "learned":
+    one per head) -- a key that is always visible and has no value, so a row's weights may
+    sum to less than one."""
 
     def __init__(self, get: Get, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int,
                  scale: float, softcap: float, eps: float, dtype, device, window: int = 0,
-                 sink: Optional[float] = 0.0):
+                 sink: Union[float, str, None] = 0.0, qk_norm: bool = True, rot_dims: int = 0,
+                 rot_base: float = 10000.0, rot_ramp=None, interleaved: bool = False, max_pos: int = 0):
         f32 = lambda n: get(n).to(device, torch.float32).contiguous()   # noqa: E731
+        if sink == "learned":
+            sink = f32("sink")
+            if sink.numel() != heads:
+                raise ValueError("one sink per head")
         spec = M.WindowSpec(heads, kv_heads, dim, vdim, int(window), float(scale), maps=1,
                             softcap=float(softcap or 0.0), sink=sink)
         wqkv = torch.cat([get("q"), get("k"), get("v")], 0).to(device, dtype).contiguous()
         super().__init__(spec, wqkv, None, get("o").to(device, dtype).contiguous(), eps, dtype)
         self.taps = int(taps)
         self.conv_w = torch.cat([f32("q.conv"), f32("k.conv"), f32("v.conv")], 0).contiguous()
-        self.q_norm, self.k_norm = f32("q.norm"), f32("k.norm")
+        self.q_norm, self.k_norm = (f32("q.norm"), f32("k.norm")) if qk_norm else (None, None)
+        self.rot_dims, self.interleaved = int(rot_dims), bool(interleaved)
+        self.table = M.rope_table(max_pos, self.rot_dims, rot_base, device=device, ramp=rot_ramp) if rot_dims else None
         self.channels = self.nq + self.nk + self.nv
         if wqkv.shape != (self.channels, width) or self.conv_w.shape != (self.channels, self.taps) \
-                or self.q_norm.numel() != dim or self.k_norm.numel() != dim:
+                or (qk_norm and (self.q_norm.numel() != dim or self.k_norm.numel() != dim)) \
+                or self.rot_dims % 2 or self.rot_dims > dim:
             raise ValueError("attention projections, convolutions or norms do not fit the head sizes")
 
     def alloc_cache(self, num_blocks, block_size, dtype, num_slots, device):
@@ -333,13 +402,16 @@ class ConvSinkAttention(WindowedAttention):
         return super().alloc_cache(num_blocks, block_size, dtype, num_slots, device) + \
             _state_slots(((max(self.taps - 1, 0), self.channels),), num_slots, device)
 
-    def __call__(self, h, ctx: StepContext, cache) -> torch.Tensor:
+    def rows(self, qkv, ctx: StepContext, cache) -> torch.Tensor:
+        """fp32 [T, heads*vdim] (before the output projection) of projected rows [q | k | v]."""
         kc, vc, hist = cache
-        qkv = F.linear(h, self.wqkv)
         q = M.conv_attn_prep(qkv, self.nq, self.nk, self.conv_w, hist, ctx.seg, self.q_norm, self.k_norm,
-                             self.eps, self.spec.dk, ctx.slot_mapping, kc, vc)
-        o = self.attend(q, ctx, (kc, vc))
-        return F.linear(o.view(h.shape[0], -1).to(self.dtype), self.wo)
+                             self.eps, self.spec.dk, ctx.slot_mapping, kc, vc, self.table, self.rot_dims,
+                             self.interleaved)
+        return self.attend(q, ctx, (kc, vc)).view(qkv.shape[0], -1)
+
+    def __call__(self, h, ctx: StepContext, cache) -> torch.Tensor:
+        return F.linear(self.rows(F.linear(h, self.wqkv), ctx, cache).to(self.dtype), self.wo)
 
 
 class BiasedWindowAttention(WindowedAttention):
@@ -515,6 +587,80 @@ class GatedLinearAttention:
         return F.linear(y, self.wo)
 
 
+class Retention:
+    """Linear attention with one fixed decay per head and no normaliser: S <- d S + k v^T,
+    o = S^T q, with rotary positions on the first ``rot_dims`` entries of every q and k head
+    (entry i paired with i + rot_dims/2) and k scaled by dim^-1/2 after the rotation.  Each
+    head's o is divided by its root mean square, the concatenated heads multiplied by
+    silu(W_g h), then the output projection.  The state [heads, dim, vdim] is fp32 and lives in
+    the sequence's state slot."""
+
+    def __init__(self, get: Get, width: int, heads: int, dim: int, vdim: int, decay, rot_dims: int, rot_base: float,
+                 eps: float, dtype, device, max_pos: int):
+        self.heads, self.dk, self.dv, self.eps, self.dtype = heads, dim, vdim, eps, dtype
+        d = torch.tensor([float(x) for x in decay], dtype=torch.float64)
+        if d.numel() != heads or not bool(((d > 0) & (d <= 1)).all()):
+            raise ValueError("retention needs one decay in (0, 1] per head")
+        self.log_decay = torch.log(d).to(device).contiguous()
+        self.nqkv, self.ng = heads * (2 * dim + vdim), heads * vdim
+        # q | k | v | output gate in one product
+        self.win = torch.cat([get("q"), get("k"), get("v"), get("g")], 0).to(device, dtype).contiguous()
+        self.wo = get("o").to(device, dtype).contiguous()
+        self.rot_dims = int(rot_dims)
+        if self.win.shape != (self.nqkv + self.ng, width) or self.wo.shape != (width, self.ng) or \
+                self.rot_dims % 2 or self.rot_dims > dim:
+            raise ValueError("retention projections do not fit the head sizes")
+        self.table = M.rope_table(max_pos, self.rot_dims, rot_base, device=device) if self.rot_dims else None
+        self.unit = torch.ones(vdim, dtype=torch.float32, device=device)      # the head norm has no weight
+
+    def cache_bytes_per_token(self, elem_bytes: int) -> int:
+        return 0
+
+    def alloc_cache(self, num_blocks, block_size, dtype, num_slots, device):
+        return _state_slots(((self.heads, self.dk, self.dv),), num_slots, device)[0]
+
+    def rows(self, p, ctx: StepContext, state) -> torch.Tensor:
+        """fp32 o [T, heads*vdim] of projected rows [q | k | v | gate]."""
+        return M.retention(p, self.table, self.rot_dims, self.log_decay, state, ctx.seg, self.heads, self.dk, self.dv)
+
+    def __call__(self, h, ctx: StepContext, state) -> torch.Tensor:
+        p = F.linear(h, self.win)
+        y = M.head_rms_gate(self.rows(p, ctx, state), self.unit, p[:, self.nqkv:], self.eps, self.heads, self.dv,
+                            self.dtype, silu=True)
+        return F.linear(y, self.wo)
+
+
+class SideBySideSum:
+    """left_scale * left(h) + right_scale * right(h) of a windowed attention and a retention
+    mixer that read the same input, as two products in all: one input product for both, and
+    one output product over the two mixers' rows side by side (the scales are applied to the
+    rows, in fp32, before they are rounded).  The cache is the pair of the two mixers'."""
+
+    def __init__(self, left: ConvSinkAttention, right: Retention, left_scale: float, right_scale: float, dtype, device):
+        self.left, self.right, self.dtype = left, right, dtype
+        self.left_scale, self.right_scale = float(left_scale), float(right_scale)
+        self.n_left = left.channels
+        self.win = _product_rows([left.wqkv, right.win], dtype, device)
+        self.wo = torch.cat([left.wo, right.wo], 1).contiguous()
+        left.wqkv = left.wo = right.win = right.wo = None        # their weights live here
+
+    def cache_bytes_per_token(self, elem_bytes: int) -> int:
+        return self.left.cache_bytes_per_token(elem_bytes) + self.right.cache_bytes_per_token(elem_bytes)
+
+    def alloc_cache(self, num_blocks, block_size, dtype, num_slots, device):
+        return (self.left.alloc_cache(num_blocks, block_size, dtype, num_slots, device),
+                self.right.alloc_cache(num_blocks, block_size, dtype, num_slots, device))
+
+    def __call__(self, h, ctx: StepContext, cache) -> torch.Tensor:
+        p = F.linear(h, self.win)
+        r = self.right
+        pr = p[:, self.n_left:self.n_left + r.nqkv + r.ng]
+        a = self.left.rows(p[:, :self.n_left], ctx, cache[0])
+        o = r.rows(pr, ctx, cache[1])
+        y = M.scaled_pair_rows(a, self.left_scale, o, pr[:, r.nqkv:], self.right_scale, r.eps, r.heads, r.dv, self.dtype)
+        return F.linear(y, self.wo)
+
+
 class SideBySide:
     """Two mixers that read the same input; each output is divided by its root mean
     square over the model width and multiplied by a weight vector of its own, and the
@@ -635,7 +781,11 @@ class MoEFF:
       W_down relu(W_up h)^2;
     * ``"top_sigmoid"`` + ``"silu_glu"``: the ``top`` largest logits (without a bias) are
       chosen and weighted by their sigmoids, divided by the sum of those, times
-      ``route_scale``; expert out = W_down (silu(W_gate h) * (W_up h)).
+      ``route_scale``; expert out = W_down (silu(W_gate h) * (W_up h)).  With ``keep`` <
+      ``groups`` only the experts of the best groups can be chosen, a group's score being the
+      sum of its two largest sigmoids.
+
+    Routing and expert form can be combined freely.
 
     Router logits are fp32 in all of them."""
 
@@ -688,9 +838,10 @@ class MoEFF:
             return M.moe_topk(z, self.correction, self.top, self.groups, self.keep)
         sg = self.routing == "top_sigmoid"
         if h.shape[0] <= self.PAIR_ROWS:
-            return M.moe_route_top_logits(h, self.router, self.router_bias, self.top, sg, self.route_scale)
+            return M.moe_route_top_logits(h, self.router, self.router_bias, self.top, sg, self.route_scale,
+                                          self.groups if sg else 1, self.keep if sg else 1)
         z = F.linear(h.float(), self.router, self.router_bias)
-        return M.moe_top_sigmoid(z, self.top, self.route_scale) if sg else M.moe_top_logits(z, self.top)
+        return M.moe_top_sigmoid(z, self.top, self.route_scale, self.groups, self.keep) if sg else M.moe_top_logits(z, self.top)
 
     def _act(self, u, limit: Optional[float] = None):
         if self.act == "clamp_glu":

@@ -11,6 +11,8 @@ builds the layer list in ``load_tensors``.
 Per run, with x the residual:  x += norm1b(mixer(norm1 x));
 x += norm2b(ff(norm2 x)) (if the layer has a feed-forward);
 x += rms(side(x, token)) * side.norm (if it has a token-side input).
+A layer without post-norm weights (norm1b / norm2b None) adds its sublayers' outputs as they
+are: x += mixer(norm1 x); x += ff(norm2 x).
 A layer with a token shift (``StackedLayer.shift``) hands its mixer h + (h' - h) * shift,
 h = norm1 x and h' the h of the token before; every run keeps a sequence's last h in its
 state slot.
@@ -48,7 +50,7 @@ from .mixers import StepContext
 class StackedLayer:
     kind: str
     norm1: torch.Tensor
-    norm1b: torch.Tensor
+    norm1b: Optional[torch.Tensor]
     mixer: object
     norm2: Optional[torch.Tensor] = None
     norm2b: Optional[torch.Tensor] = None
@@ -224,7 +226,7 @@ class StackedModel:
             return self._forward_layer_post(input_ids, meta, ctx, caches)
         if self.norm_style == "shared_pre":
             return self._forward_shared_pre(input_ids, meta, ctx, caches)
-        x = M.embed_rows(input_ids, self.embed, self.embed_scale)
+        x = self._embed(input_ids, ctx, caches)
         tap = self.layer_tap
         fuse_step = tap is None
         h = None
@@ -248,8 +250,9 @@ class StackedModel:
             nshift = self.layers[nxt[0]].shift if nxt is not None else None
             if nshift is not None:
                 # the layer's last add, the next layer's norm and its token shift in one kernel
-                if L.side is not None or nxt[1] is not None:
-                    raise NotImplementedError("a token shift after a token-side input or a loop step")
+                if L.side is not None or nxt[1] is not None or L.norm1b is None:
+                    raise NotImplementedError("a token shift after a token-side input, a loop step or a layer "
+                                              "without post-norms")
                 wb = L.norm1b
                 if L.ff is not None:
                     h, _ = M.add_rms_norm_rows(x, y, L.norm1b, eps, next_w=L.norm2, out_dtype=dt)
@@ -280,6 +283,20 @@ class StackedModel:
             return rows.to(dt)
         return M.rms_norm_rows(rows, self.final_norm, eps, dt)
 
+    def _embed(self, input_ids, ctx, caches: StackedCache) -> torch.Tensor:
+        """fp32 residual rows: embedding table, plus the pair table's rows if there is one."""
+        if self.pair_embed is None:
+            return M.embed_rows(input_ids, self.embed, self.embed_scale)
+        table, mul_prev, mul_cur, buckets = self.pair_embed
+        return M.pair_embed_rows(input_ids, self.embed, self.embed_scale, table, mul_prev, mul_cur, buckets, ctx.seg,
+                                 caches.extra["last_token"])
+
+    def load_pair_table(self, table: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int):
+        table = table.to(self.device, self.dtype).contiguous()
+        if table.shape != (buckets + 1, self.cfg.hidden_size):
+            raise ValueError("pair table does not fit its bucket count")
+        self.pair_embed = (table, mul_prev, mul_cur, buckets)
+
     def _forward_layer_post(self, input_ids, meta, ctx, caches: StackedCache) -> torch.Tensor:
         dt, eps = self.dtype, self.cfg.rms_norm_eps
         x = M.embed_rows(input_ids, self.embed, self.embed_scale, meta.positions, self.pos_freqs)
@@ -303,12 +320,7 @@ class StackedModel:
 
     def _forward_shared_pre(self, input_ids, meta, ctx, caches: StackedCache) -> torch.Tensor:
         dt, eps, mult = self.dtype, self.cfg.rms_norm_eps, self.residual_mult
-        if self.pair_embed is not None:
-            table, mul_prev, mul_cur, buckets = self.pair_embed
-            x = M.pair_embed_rows(input_ids, self.embed, self.embed_scale, table, mul_prev, mul_cur, buckets, ctx.seg,
-                                  caches.extra["last_token"])
-        else:
-            x = M.embed_rows(input_ids, self.embed, self.embed_scale)
+        x = self._embed(input_ids, ctx, caches)
         tap, mark = self.layer_tap, self.mark_at
         nruns = len(self.runs)
         h = M.add_scaled_rms_norm_rows(x, None, None, mult, self.layers[self.runs[0][0]].norm1, eps, dt) \

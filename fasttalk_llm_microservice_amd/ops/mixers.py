@@ -1,10 +1,10 @@
 """Sequence-mixer and mixture-of-experts ops: latent (low-rank KV) attention over a
 paged latent cache, windowed attention (softmax or sigmoid weights, distance bias,
-several score maps per head, capped scores, a sink in the softmax) over a paged key /
-value cache, attention that mixes its scores across the heads, the gated delta-rule recurrence with per-channel decay and the selective
-state-space scan over state slots, short causal convolutions (alone, or fused with
-per-head norms and the cache write), routing (grouped softmax top-k, or top-k on the
-logits with softmax or sigmoid weights), clamped-GLU, silu-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product
+several score maps per head, capped scores, a sink in the softmax) over a paged key / value cache, attention that mixes its scores across the heads, the gated delta-rule
+recurrence (a decay per channel or per head), retention and the selective state-space scan
+over state slots, short causal convolutions (alone, or fused with per-head norms, rotation
+and the cache write, or with the delta rule's preparation), routing (grouped softmax top-k,
+or top-k on the logits with softmax or sigmoid weights, optionally limited to the best groups), clamped-GLU, silu-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product
 for many), and the fp32-residual norms (RMS pre/post norms, optionally with a token shift, layer
 norm with bias) that tie them together.
 
@@ -23,7 +23,7 @@ import dataclasses
 import importlib
 import os
 import threading
-from typing import Optional
+from typing import Optional, Union
 
 import torch
 
@@ -133,10 +133,10 @@ def rms_norm_rows(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype,
     return ref.rms_norm_rows(x, w, eps, out_dtype, add_vec)
 
 
-def add_rms_norm_rows(residual: torch.Tensor, y: torch.Tensor, wb: torch.Tensor, eps: float,
+def add_rms_norm_rows(residual: torch.Tensor, y: torch.Tensor, wb: Optional[torch.Tensor], eps: float,
                       add_vec: Optional[torch.Tensor] = None, next_w: Optional[torch.Tensor] = None,
                       out_dtype=None, want_cast: bool = False):
-    """residual (fp32, in place) += rms_norm(y) * wb (+ add_vec); returns
+    """residual (fp32, in place) += rms_norm(y) * wb (y as it is without ``wb``) (+ add_vec); returns
     (rms_norm(residual) * next_w or None, residual cast to out_dtype or None)."""
     out_dtype = out_dtype or y.dtype
     if residual.is_cuda:
@@ -188,6 +188,19 @@ def dual_rms_mean(a: torch.Tensor, b: torch.Tensor, wa: torch.Tensor, wb: torch.
         native_mixers().dual_rms_mean(out, a, b, wa, wb, eps, float(scale))
         return out
     return ref.dual_rms_mean(a, b, wa, wb, eps, scale)
+
+
+def scaled_pair_rows(a: torch.Tensor, a_scale: float, o: torch.Tensor, gate: torch.Tensor, o_scale: float, eps: float,
+                     heads: int, dv: int, out_dtype) -> torch.Tensor:
+    """Rows [a_scale * a | o_scale * head_norm(o) * silu(gate)] in ``out_dtype``: what the
+    joint output product of two side-by-side mixers reads.  a fp32 [T, n]; o fp32 [T,
+    heads*dv], every head divided by its root mean square; gate [T, heads*dv] (may be a
+    column range)."""
+    if o.is_cuda:
+        out = torch.empty(o.shape[0], a.shape[1] + heads * dv, dtype=out_dtype, device=o.device)
+        native_mixers().scaled_pair_rows(out, a, float(a_scale), o, gate, float(o_scale), eps, heads, dv)
+        return out
+    return ref.scaled_pair_rows(a, a_scale, o, gate, o_scale, eps, heads, dv, out_dtype)
 
 
 def pair_embed_add(x: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, mul_prev: int, mul_cur: int,
@@ -269,6 +282,71 @@ def gated_delta_rule(qkv, a, b, a_log, dt_bias, state, seg: Segments, heads: int
                                          seg.slot, seg.num, heads, kv_heads, dk, dv)
         return o
     return ref.gated_delta_rule(qkv, a, b, a_log, dt_bias, state, seg, heads, kv_heads, dk, dv)
+
+
+def conv_delta_prep(qkv, a, b, conv_w, conv_state, a_log, dt_bias, seg: Segments, heads: int, kv_heads: int, dk: int,
+                    dv: int):
+    """What the delta rule with one decay per head reads, in one launch over rows [q
+    (kv_heads*dk) | k (kv_heads*dk) | v (heads*dv)] of a fused projection: per-channel causal
+    convolution over time (as in :func:`conv_attn_prep`) and silu, q and k made unit vectors
+    per head (x / sqrt(sum x^2 + 1e-6); q also * dk^-1/2), the decay's logarithm
+    -exp(a_log) * softplus(a + dt_bias) and beta = sigmoid(b) (a, b [T, heads], may be column
+    ranges).  All fp32: (q [T, kv_heads, dk], k, v [T, heads, dv], log decay [T, heads],
+    beta [T, heads])."""
+    if qkv.is_cuda:
+        t, dev = qkv.shape[0], qkv.device
+        f32 = dict(dtype=torch.float32, device=dev)
+        q, k = torch.empty(t, kv_heads, dk, **f32), torch.empty(t, kv_heads, dk, **f32)
+        v = torch.empty(t, heads, dv, **f32)
+        lg, beta = torch.empty(t, heads, **f32), torch.empty(t, heads, **f32)
+        native_mixers().conv_delta_prep(q, k, v, lg, beta, qkv, a, b, conv_w, conv_state, a_log, dt_bias, seg.start,
+                                        seg.pos0, seg.slot, seg.num, seg.max_rows)
+        return q, k, v, lg, beta
+    return ref.conv_delta_prep(qkv, a, b, conv_w, conv_state, a_log, dt_bias, seg, heads, kv_heads, dk, dv)
+
+
+# rows from which a segment's recurrence runs chunk by chunk as matrix products (per-head
+# decays); shorter segments and decode rows are walked row by row
+CHUNK_ROWS = 32
+
+
+def head_delta_rule(q, k, v, log_decay, beta, state, seg: Segments) -> torch.Tensor:
+    """Gated delta rule with one decay per head, on the outputs of :func:`conv_delta_prep`.
+    Per head and row:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q with g =
+    exp(log_decay).  ``state`` [slots, heads, dk, dv] fp32 is read (zeros at position 0) and
+    left at the segment's last row.  Returns o fp32 [T, heads*dv]."""
+    if v.is_cuda:
+        t, heads, dv = v.shape
+        o = torch.empty(t, heads * dv, dtype=torch.float32, device=v.device)
+        native_mixers().head_delta_rule(o, q, k, v, log_decay, beta, state, seg.start, seg.pos0, seg.slot, seg.num,
+                                        seg.max_rows, _walk_below(seg), CHUNK_ROWS)
+        return o
+    return ref.head_delta_rule(q, k, v, log_decay, beta, state, seg)
+
+
+def retention(qkv, table, rot_dims: int, log_decay, state, seg: Segments, heads: int, dk: int, dv: int,
+              interleaved: bool = False) -> torch.Tensor:
+    """Linear attention with one fixed decay per head.  Rows of ``qkv`` are [q (heads*dk) | k
+    (heads*dk) | v (heads*dv) | ...]; q and k are rotated by position (``table`` =
+    :func:`rope_table` over the first ``rot_dims`` entries of a head, pairs (i, i + rot_dims/2),
+    or (2i, 2i + 1) if ``interleaved``; None: no rotation), k is scaled by dk^-1/2.  Per head
+    and row:  S <- d S + k v^T;  o = S^T q with d = exp(log_decay[head]) (``log_decay`` fp64
+    [heads]: powers of d are formed from it).  ``state`` [slots, heads, dk, dv] fp32 is read
+    (zeros at position 0) and left at the segment's last row.  Returns o fp32 [T, heads*dv]."""
+    if qkv.is_cuda:
+        o = torch.empty(qkv.shape[0], heads * dv, dtype=torch.float32, device=qkv.device)
+        native_mixers().retention(o, qkv, table, rot_dims, bool(interleaved), log_decay, state, seg.start, seg.pos0,
+                                  seg.slot, seg.num, seg.max_rows, heads, dk, dv, _walk_below(seg), CHUNK_ROWS)
+        return o
+    return ref.retention(qkv, table, rot_dims, interleaved, log_decay, state, seg, heads, dk, dv)
+
+
+def _walk_below(seg: Segments) -> bool:
+    """Whether a step may hold segments short enough to be walked row by row."""
+    if seg.max_rows < CHUNK_ROWS or seg.host is None:
+        return True
+    start = seg.host[0]
+    return min(b - a for a, b in zip(start[:-1], start[1:])) < CHUNK_ROWS
 
 
 def gated_linear_attention(qkv, a, a_bias, tau: float, state, seg: Segments, heads: int, dk: int,
@@ -492,22 +570,26 @@ def attn_prep(qkv, nq: int, nk: int, q_norm_w, k_norm_w, eps: float, table, rot_
 
 
 def conv_attn_prep(qkv, nq: int, nk: int, conv_w, conv_state, seg: Segments, q_norm_w, k_norm_w, eps: float,
-                   head_dim: int, slot_mapping, k_cache, v_cache) -> torch.Tensor:
+                   head_dim: int, slot_mapping, k_cache, v_cache, table=None, rot_dims: int = 0,
+                   interleaved: bool = False) -> torch.Tensor:
     """Rows [q (nq) | k (nk) | v] of a fused projection pass a per-channel causal
     convolution over time (``conv_w`` [C, taps] fp32, last column = the current row, no
     bias, no activation; ``conv_state`` [slots, taps-1, C] fp32 holds each sequence's last
     projected rows and is updated; a segment at position 0 starts from zeros), then every
     ``head_dim`` chunk of q and of k is divided by its root mean square and multiplied by
-    ``q_norm_w`` / ``k_norm_w`` ([head_dim], shared by the heads; None: no norm).
-    Convolution and norm are fp32.  Returns fp32 queries [T, nq]; keys and values go to
+    ``q_norm_w`` / ``k_norm_w`` ([head_dim], shared by the heads; None: no norm), then rotated
+    by position on its first ``rot_dims`` entries (``table`` = :func:`rope_table`; pairs
+    (i, i + rot_dims/2), or (2i, 2i + 1) if ``interleaved``; None: no rotation).
+    Convolution, norm and rotation are fp32.  Returns fp32 queries [T, nq]; keys and values go to
     the rows' cache slots."""
     if qkv.is_cuda:
         q = torch.empty(qkv.shape[0], nq, dtype=torch.float32, device=qkv.device)
         native_mixers().conv_attn_prep(q, qkv, nq, nk, conv_w, conv_state, seg.start, seg.pos0, seg.slot, seg.num,
-                                       q_norm_w, k_norm_w, eps, head_dim, slot_mapping, k_cache, v_cache)
+                                       seg.max_rows, q_norm_w, k_norm_w, eps, head_dim, slot_mapping, k_cache, v_cache,
+                                       table, rot_dims, bool(interleaved))
         return q
     return ref.conv_attn_prep(qkv, nq, nk, conv_w, conv_state, seg, q_norm_w, k_norm_w, eps, head_dim,
-                              slot_mapping, k_cache, v_cache)
+                              slot_mapping, k_cache, v_cache, table, rot_dims, interleaved)
 
 
 @dataclasses.dataclass
@@ -521,8 +603,9 @@ class WindowSpec:
     s = q.k * scale; with ``softcap`` c > 0, s <- c tanh(s / c);
     score = s - r1[a] ln(1 + r2[a] (i - j)) + dist_bias[min(i - j, nd - 1), a]; weight =
     softmax over the visible keys, or sigmoid(score + pb[a]) without normalisation.
-    ``sink`` (a score, softmax only): the softmax's denominator gains exp(sink), as if one
-    more key with that score and no value were always visible."""
+    ``sink`` (softmax only; one score, or fp32 [heads * maps], one per query head): the
+    softmax's denominator gains exp(sink), as if one more key with that score and no value
+    were always visible."""
     heads: int
     kv_heads: int
     dk: int
@@ -535,10 +618,15 @@ class WindowSpec:
     r2: Optional[torch.Tensor] = None
     pb: Optional[torch.Tensor] = None     # fp32 [heads * maps] (sigmoid weights only)
     softcap: float = 0.0
-    sink: Optional[float] = None
+    sink: Union[float, torch.Tensor, None] = None
     blocks: bool = False
     keep_first: int = 0
     dist_bias: Optional[torch.Tensor] = None   # fp32 [nd, heads * maps], :func:`distance_bias_table`
+
+
+def _sink_args(sink):
+    """(one score for all heads, scores per head), each None when not given."""
+    return (None, sink) if isinstance(sink, torch.Tensor) else (sink, None)
 
 
 def window_attention(q, k_cache, v_cache, seg: Segments, spec: WindowSpec, skip_from: int = 0,
@@ -553,7 +641,7 @@ def window_attention(q, k_cache, v_cache, seg: Segments, spec: WindowSpec, skip_
         native_mixers().window_attention(out, q, k_cache, v_cache, seg.start, seg.pos0, seg.kv_len,
                                          seg.block_tables, seg.num, seg.max_rows, sp.heads, sp.maps,
                                          sp.kv_heads, sp.dk, sp.dv, sp.window, sp.scale, sp.sigmoid,
-                                         sp.r1, sp.r2, sp.pb, skip_from, float(sp.softcap), sp.sink,
+                                         sp.r1, sp.r2, sp.pb, skip_from, float(sp.softcap), *_sink_args(sp.sink),
                                          bool(sp.blocks), int(sp.keep_first), sp.dist_bias)
         return out
     r = ref.window_attention(q, k_cache, v_cache, seg, sp.heads, sp.maps, sp.kv_heads, sp.dk, sp.dv,
@@ -575,7 +663,7 @@ def band_weights(s, first_pos: int, key0: int, spec: WindowSpec, rep_rows: int, 
     if s.is_cuda:
         native_mixers().band_weights(s, rep_rows, first_pos, key0, sp.heads, sp.maps, sp.kv_heads,
                                      sp.window, sp.scale, sp.sigmoid, sp.r1, sp.r2, sp.pb, float(sp.softcap),
-                                     sp.sink, bool(sp.blocks), int(sp.keep_first), int(ext), sp.dist_bias)
+                                     *_sink_args(sp.sink), bool(sp.blocks), int(sp.keep_first), int(ext), sp.dist_bias)
         return s
     g, rr, keys = s.shape
     rep = sp.heads // sp.kv_heads
@@ -813,34 +901,37 @@ def moe_top_logits(z, top: int):
         t = z.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=z.device)
         wts = torch.empty(t, top, dtype=torch.float32, device=z.device)
-        native_mixers().moe_top_logits(idx, wts, z, top, False, 1.0)
+        native_mixers().moe_top_logits(idx, wts, z, top, False, 1.0, 1, 1)
         return idx, wts
     return ref.moe_top_logits(z, top)
 
 
-def moe_top_sigmoid(z, top: int, scale: float):
+def moe_top_sigmoid(z, top: int, scale: float, groups: int = 1, keep: int = 1):
     """Router: the ``top`` largest logits of each fp32 row (ties to the lower index); the
-    weights are the chosen ones' sigmoids divided by the sum of those, times ``scale``."""
+    weights are the chosen ones' sigmoids divided by the sum of those, times ``scale``.
+    With ``keep`` < ``groups`` only experts of the ``keep`` best of ``groups`` equal groups of
+    neighbours can be chosen; a group's score is the sum of its two largest sigmoids."""
     if z.is_cuda:
         t = z.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=z.device)
         wts = torch.empty(t, top, dtype=torch.float32, device=z.device)
-        native_mixers().moe_top_logits(idx, wts, z, top, True, float(scale))
+        native_mixers().moe_top_logits(idx, wts, z, top, True, float(scale), groups, keep)
         return idx, wts
-    return ref.moe_top_sigmoid(z, top, scale)
+    return ref.moe_top_sigmoid(z, top, scale, groups, keep)
 
 
-def moe_route_top_logits(h, router, bias, top: int, sigmoid: bool = False, scale: float = 1.0):
-    """:func:`moe_top_logits` (or, ``sigmoid``, :func:`moe_top_sigmoid` with ``scale``) of z = router h + bias (fp32 router [E, width] and bias, h fp32
+def moe_route_top_logits(h, router, bias, top: int, sigmoid: bool = False, scale: float = 1.0, groups: int = 1,
+                         keep: int = 1):
+    """:func:`moe_top_logits` (or, ``sigmoid``, :func:`moe_top_sigmoid` with ``scale`` and groups) of z = router h + bias (fp32 router [E, width] and bias, h fp32
     or bf16, fp32 accumulation) in one launch: the router of few rows (decode steps)."""
     if h.is_cuda:
         t = h.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=h.device)
         wts = torch.empty(t, top, dtype=torch.float32, device=h.device)
-        native_mixers().moe_route_top_logits(idx, wts, h, router, bias, top, bool(sigmoid), float(scale))
+        native_mixers().moe_route_top_logits(idx, wts, h, router, bias, top, bool(sigmoid), float(scale), groups, keep)
         return idx, wts
     z = torch.nn.functional.linear(h.float(), router, bias)
-    return ref.moe_top_sigmoid(z, top, scale) if sigmoid else ref.moe_top_logits(z, top)
+    return ref.moe_top_sigmoid(z, top, scale, groups, keep) if sigmoid else ref.moe_top_logits(z, top)
 
 
 # first matrix and activation of an expert: the code the kernels take

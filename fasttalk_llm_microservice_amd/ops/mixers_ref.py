@@ -70,7 +70,7 @@ def rms_norm_rows(x, w, eps, out_dtype, add_vec=None):
 
 
 def add_rms_norm_rows(residual, y, wb, eps, add_vec, next_w, out_dtype, want_cast):
-    residual.add_(_rms(y.float(), eps) * wb.float())
+    residual.add_(y.float() if wb is None else _rms(y.float(), eps) * wb.float())
     if add_vec is not None:
         residual.add_(add_vec.float())
     out = (_rms(residual, eps) * next_w.float()).to(out_dtype) if next_w is not None else None
@@ -100,6 +100,13 @@ def add_norm_shift_rows(residual, y, wb, w, shift, eps, out_dtype, prev_state, s
         if slot >= 0:
             prev_state[slot] = h[b - 1]
     return x, (h + (prev - h) * shift.float()).to(out_dtype)
+
+
+def scaled_pair_rows(a, a_scale, o, gate, o_scale, eps, heads, dv, out_dtype):
+    t = o.shape[0]
+    g = gate.float()
+    r = _rms(o.view(t, heads, dv), eps).view(t, heads * dv) * (g * torch.sigmoid(g)) * o_scale
+    return torch.cat([a.view(t, -1) * a_scale, r], -1).to(out_dtype)
 
 
 def dual_rms_mean(a, b, wa, wb, eps, scale):
@@ -260,6 +267,89 @@ def gated_delta_rule(qkv, a, b, a_log, dt_bias, state, seg, heads, kv_heads, dk,
     return o.view(t, heads * dv)
 
 
+def _conv_fp32(x, conv_w, conv_state, seg):
+    """fp32 short convolution of rows x (no bias, no activation); updates the history."""
+    taps = conv_w.shape[1]
+    w = conv_w.float()
+    y = torch.zeros(x.shape, dtype=torch.float32, device=x.device)
+    start = seg.start.tolist()
+    for s in range(seg.num):
+        a, b = start[s], start[s + 1]
+        slot = int(seg.slot[s])
+        if slot < 0 or b == a:
+            continue
+        hist = conv_state[slot] if int(seg.pos0[s]) > 0 else torch.zeros_like(conv_state[slot])
+        xp = torch.cat([hist, x[a:b].float()], 0)
+        n = b - a
+        y[a:b] = sum(xp[j:j + n] * w[:, j][None] for j in range(taps))
+        if taps > 1:
+            conv_state[slot] = xp[n:]
+    return y
+
+
+def conv_delta_prep(qkv, a, b, conv_w, conv_state, a_log, dt_bias, seg, heads, kv_heads, dk, dv):
+    t = qkv.shape[0]
+    n = kv_heads * dk
+    y = _conv_fp32(qkv, conv_w, conv_state, seg)
+    y = y * torch.sigmoid(y)
+    q, k = y[:, :n].view(t, kv_heads, dk), y[:, n:2 * n].view(t, kv_heads, dk)
+    q = q * torch.rsqrt((q * q).sum(-1, keepdim=True) + 1e-6) * dk ** -0.5
+    k = k * torch.rsqrt((k * k).sum(-1, keepdim=True) + 1e-6)
+    lg = -torch.exp(a_log.float())[None] * F.softplus(a.float() + dt_bias.float(), threshold=1e9)
+    return q.contiguous(), k.contiguous(), y[:, 2 * n:].view(t, heads, dv).contiguous(), lg, torch.sigmoid(b.float())
+
+
+def head_delta_rule(qn, kn, v, lg, beta, state, seg):
+    t, heads, dv = v.shape
+    rep = heads // qn.shape[1]
+    g = torch.exp(lg)
+    o = torch.zeros(t, heads, dv, dtype=torch.float32, device=v.device)
+    start = seg.start.tolist()
+    for s in range(seg.num):
+        slot = int(seg.slot[s])
+        if slot < 0 or start[s + 1] == start[s]:
+            continue
+        S = state[slot] if int(seg.pos0[s]) > 0 else torch.zeros_like(state[slot])
+        for r in range(start[s], start[s + 1]):
+            qt, kt = qn[r].repeat_interleave(rep, 0), kn[r].repeat_interleave(rep, 0)
+            S = g[r][:, None, None] * S
+            u = beta[r][:, None] * (v[r] - torch.einsum("hkv,hk->hv", S, kt))
+            S = S + kt[:, :, None] * u[:, None, :]
+            o[r] = torch.einsum("hkv,hk->hv", S, qt)
+        state[slot] = S
+    return o.view(t, heads * dv)
+
+
+def retention(qkv, table, rot_dims, interleaved, log_decay, state, seg, heads, dk, dv):
+    t = qkv.shape[0]
+    n = heads * dk
+    q = qkv[:, :n].float().view(t, heads, dk)
+    k = qkv[:, n:2 * n].float().view(t, heads, dk)
+    v = qkv[:, 2 * n:2 * n + heads * dv].float().view(t, heads, dv)
+    start = seg.start.tolist()
+    if table is not None and rot_dims > 0:
+        pos = torch.zeros(t, dtype=torch.long, device=qkv.device)
+        for s in range(seg.num):
+            a, b = start[s], start[s + 1]
+            pos[a:b] = int(seg.pos0[s]) + torch.arange(b - a, device=qkv.device)
+        cs = table[pos]
+        q = _rope(q.transpose(0, 1), cs, rot_dims, interleaved).transpose(0, 1)
+        k = _rope(k.transpose(0, 1), cs, rot_dims, interleaved).transpose(0, 1)
+    k = k * dk ** -0.5
+    d = torch.exp(log_decay).float()[:, None, None]
+    o = torch.zeros(t, heads, dv, dtype=torch.float32, device=qkv.device)
+    for s in range(seg.num):
+        slot = int(seg.slot[s])
+        if slot < 0 or start[s + 1] == start[s]:
+            continue
+        S = state[slot] if int(seg.pos0[s]) > 0 else torch.zeros_like(state[slot])
+        for r in range(start[s], start[s + 1]):
+            S = d * S + k[r][:, :, None] * v[r][:, None, :]
+            o[r] = torch.einsum("hkv,hk->hv", S, q[r])
+        state[slot] = S
+    return o.view(t, heads * dv)
+
+
 def gated_linear_attention(qkv, a, a_bias, tau, state, seg, heads, dk, dv):
     t = qkv.shape[0]
     n = heads * dk
@@ -389,9 +479,18 @@ def moe_top_logits(z, top):
     return idx[:, :top].int(), torch.softmax(val[:, :top], -1)
 
 
-def moe_top_sigmoid(z, top, scale):
+def moe_top_sigmoid(z, top, scale, groups=1, keep=1):
     """The ``top`` largest logits per row (ties to the lower index); weights are their
-    sigmoids divided by the sum of those, times ``scale``."""
+    sigmoids divided by the sum of those, times ``scale``.  With ``keep`` < ``groups`` only
+    the experts of the ``keep`` best of ``groups`` equal groups of neighbours can be chosen,
+    a group's score being the sum of its two largest sigmoids."""
+    z = z.float()
+    if keep < groups:
+        s = torch.sigmoid(z).view(z.shape[0], groups, -1)
+        gs = s.topk(min(2, s.shape[2]), -1).values.sum(-1)
+        best = torch.sort(gs, dim=-1, descending=True, stable=True).indices[:, :keep]
+        ok = torch.zeros_like(gs, dtype=torch.bool).scatter_(1, best, True)
+        z = z.masked_fill(~ok.repeat_interleave(s.shape[2], 1), float("-inf"))
     val, idx = torch.sort(z.float(), dim=-1, descending=True, stable=True)
     s = torch.sigmoid(val[:, :top])
     return idx[:, :top].int(), s / (s.sum(-1, keepdim=True) + 1e-20) * scale
@@ -477,28 +576,22 @@ def attn_prep(qkv, nq, nk, q_norm_w, k_norm_w, eps, table, rot_dims, head_dim, p
 
 
 def conv_attn_prep(qkv, nq, nk, conv_w, conv_state, seg, q_norm_w, k_norm_w, eps, head_dim, slot_mapping,
-                   k_cache, v_cache):
+                   k_cache, v_cache, table=None, rot_dims=0, interleaved=False):
     t = qkv.shape[0]
-    taps = conv_w.shape[1]
-    w = conv_w.float()
-    y = torch.zeros(qkv.shape, dtype=torch.float32, device=qkv.device)
-    start = seg.start.tolist()
-    for s in range(seg.num):
-        a, b = start[s], start[s + 1]
-        slot = int(seg.slot[s])
-        if slot < 0 or b == a:
-            continue
-        hist = conv_state[slot] if int(seg.pos0[s]) > 0 else torch.zeros_like(conv_state[slot])
-        xp = torch.cat([hist, qkv[a:b].float()], 0)
-        n = b - a
-        y[a:b] = sum(xp[j:j + n] * w[:, j][None] for j in range(taps))
-        if taps > 1:
-            conv_state[slot] = xp[n:]
+    y = _conv_fp32(qkv, conv_w, conv_state, seg)
     q, k, v = y[:, :nq], y[:, nq:nq + nk], y[:, nq + nk:]
     if q_norm_w is not None:
         q = (_rms(q.reshape(t, -1, head_dim), eps) * q_norm_w.float()).reshape(t, nq)
     if k_norm_w is not None:
         k = (_rms(k.reshape(t, -1, head_dim), eps) * k_norm_w.float()).reshape(t, nk)
+    if table is not None and rot_dims > 0:
+        start = seg.start.tolist()
+        pos = torch.zeros(t, dtype=torch.long, device=qkv.device)
+        for s in range(seg.num):
+            a, b = start[s], start[s + 1]
+            pos[a:b] = int(seg.pos0[s]) + torch.arange(b - a, device=qkv.device)
+        q, k = (_rope(x.reshape(t, -1, head_dim).transpose(0, 1), table[pos], rot_dims, interleaved)
+                .transpose(0, 1).reshape(t, -1) for x in (q, k))
     slots = slot_mapping[:t].long()
     keep = slots >= 0
     if keep.any():
@@ -546,9 +639,10 @@ def band_weights(s, first_pos, key0, window, scale, sigmoid, r1, r2, pb, softcap
         return torch.sigmoid(z) * vis[None]
     z = z.masked_fill(~vis[None], float("-inf"))
     if sink is not None:
-        m = z.max(-1, keepdim=True).values.clamp_min(float(sink))
+        sk = sink.float()[:, None, None] if isinstance(sink, torch.Tensor) else torch.full_like(z[:1, :1, :1], float(sink))
+        m = torch.maximum(z.max(-1, keepdim=True).values, sk)
         e = torch.exp(z - m)
-        return e / (torch.exp(float(sink) - m) + e.sum(-1, keepdim=True))
+        return e / (torch.exp(sk - m) + e.sum(-1, keepdim=True))
     return torch.softmax(z, -1).masked_fill(~vis[None], 0.0)
 
 
