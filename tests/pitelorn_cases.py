@@ -94,9 +94,16 @@ CONFIGS = {
 }
 
 
-def make_model(name, seed, tmp_path, tweak=None):
-    """(checkpoint dir, config dict, fp32 tensors of the bf16 weights)."""
+def make_model(name, seed, tmp_path, tweak=None, dtype="float32"):
+    """(checkpoint dir, config dict, fp32 tensors of the bf16 weights).  For bf16 runs the routers
+    choose every expert: with random weights a choice is often close, and one that rounding
+    turns over moves the logits by as much as a fault would."""
     cfg = copy.deepcopy(CONFIGS[name])
+    if dtype != "float32":
+        for l in cfg["layers"]:
+            if l["mlp"] and l["mlp"]["kind"] == "moe":
+                r = l["mlp"]["router"]
+                r["top"], r["groups"]["keep"] = r["experts"], r["groups"]["count"]
     pcfg = PT.config_from_dict(cfg, name)
     t = PT.random_tensors(pcfg, seed, torch.bfloat16)
     if tweak:
@@ -110,10 +117,9 @@ def close(got, want, dtype="float32"):
     if dtype == "float32":
         torch.testing.assert_close(got, want, rtol=3e-4, atol=4e-4)
         return
-    # bf16: rounding differs from the oracle's everywhere, and a router's close call may go the
-    # other way at single positions (the fp32 runs are the sharp ones)
+    # bf16: rounding differs from the oracle's everywhere (the fp32 runs are the sharp ones)
     err = (got - want).pow(2).mean(-1).sqrt() / want.pow(2).mean(-1).sqrt().clamp_min(1e-3)
-    assert err.median() < 0.06 and float((err > 0.25).float().mean()) <= 0.1, err
+    assert err.median() < 0.06 and float(err.max()) < 0.25, err
 
 
 def oracle(cfg, P, toks):

@@ -9,7 +9,7 @@ from fasttalk_llm_microservice_amd.engine.sampling_params import SamplingParams
 
 
 def whole_prompt(name, device, dtype, tmp):
-    d, cfg, P = C.make_model(name, 11, tmp)
+    d, cfg, P = C.make_model(name, 11, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype)
     for n, seed in ((1, 1), (2, 2), (3, 3), (37, 4), (130, 5)):   # the first tokens, then one and several chunks
         t = C.tokens(n, cfg["vocab"], seed)
@@ -19,7 +19,7 @@ def whole_prompt(name, device, dtype, tmp):
 
 def layers_of_a_prompt(name, device, dtype, tmp):
     """The residual after every layer against the oracle's."""
-    d, cfg, P = C.make_model(name, 18, tmp)
+    d, cfg, P = C.make_model(name, 18, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype)
     t = C.tokens(70, cfg["vocab"], 6)
     eng.runner.model.layer_tap = tap = []
@@ -34,7 +34,7 @@ def layers_of_a_prompt(name, device, dtype, tmp):
 def prefill_then_decode(name, device, dtype, tmp):
     """Windows pass over decoded tokens; the previous token, the convolutions' last inputs and
     both recurrences' states come from the step before."""
-    d, cfg, P = C.make_model(name, 12, tmp)
+    d, cfg, P = C.make_model(name, 12, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype)
     for first in (1, 2, 19, 40):
         t = C.tokens(first + 40, cfg["vocab"], 5 + first)
@@ -43,7 +43,7 @@ def prefill_then_decode(name, device, dtype, tmp):
 
 
 def portions_of_a_prompt(name, device, dtype, tmp):
-    d, cfg, P = C.make_model(name, 13, tmp)
+    d, cfg, P = C.make_model(name, 13, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype)
     t = C.tokens(150, cfg["vocab"], 9)
     want = C.oracle(cfg, P, t)
@@ -59,7 +59,7 @@ def portions_of_a_prompt(name, device, dtype, tmp):
 def mixed_batches_and_reuse(name, device, dtype, tmp):
     """Unequal requests side by side (portions beside single tokens), more requests
     than state slots over time, a page pool smaller than the sum of all requests."""
-    d, cfg, P = C.make_model(name, 14, tmp)
+    d, cfg, P = C.make_model(name, 14, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype, pages=12, seqs=3)          # 192 tokens of cache, 3 slots
     lens = {"a": 110, "b": 9, "c": 41, "d": 1, "e": 55, "f": 40}
     reqs = {i: C.tokens(n, cfg["vocab"], 20 + k) for k, (i, n) in enumerate(lens.items())}
@@ -94,7 +94,7 @@ def peaked_scores(device, dtype, tmp):
             if k.endswith("left.q"):
                 t[k] *= 6.0
     for name in ("a", "c"):
-        d, cfg, P = C.make_model(name, 15, tmp, tweak)
+        d, cfg, P = C.make_model(name, 15, tmp, tweak, dtype)
         eng = C.make_engine(d, device, dtype, pages=24)
         t = C.tokens(200, cfg["vocab"], 31)
         want = C.oracle(cfg, P, t)
@@ -110,7 +110,7 @@ def raised_and_lowered_sinks(device, dtype, tmp):
             if k.endswith("sink"):
                 t[k] = torch.tensor([3.0 if i % 2 else -9.0 for i in range(t[k].numel())]).bfloat16()
     for name in ("a", "b"):
-        d, cfg, P = C.make_model(name, 19, tmp, tweak)
+        d, cfg, P = C.make_model(name, 19, tmp, tweak, dtype)
         eng = C.make_engine(d, device, dtype)
         t = C.tokens(60, cfg["vocab"], 33)
         C.close(C.replay(eng, {"r": t}, [[("r", 34)], [("r", 6)]] + [[("r", 1)]] * 20)["r"], C.oracle(cfg, P, t), dtype)
@@ -124,7 +124,7 @@ def slow_decay_long_decode(device, dtype, tmp):
         for k in t:
             if k.endswith("A_log"):
                 t[k] -= 3.0
-    d, cfg, P = C.make_model("c", 16, tmp, tweak)
+    d, cfg, P = C.make_model("c", 16, tmp, tweak, dtype)
     eng = C.make_engine(d, device, dtype)
     t = C.tokens(123, cfg["vocab"], 41)
     C.close(C.replay(eng, {"r": t}, [[("r", 3)]] + [[("r", 1)]] * 120)["r"], C.oracle(cfg, P, t), dtype)
@@ -133,7 +133,7 @@ def slow_decay_long_decode(device, dtype, tmp):
 def greedy_generation(name, device, dtype, tmp, graphs=False):
     """Through LLMEngine.generate: the scheduler's own batching, the sampler at
     temperature 0, against greedy decoding with the oracle."""
-    d, cfg, P = C.make_model(name, 17, tmp)
+    d, cfg, P = C.make_model(name, 17, tmp, dtype=dtype)
     eng = C.make_engine(d, device, dtype, seqs=2, graphs=graphs)   # three prompts, two slots: one waits
     prompts = [C.tokens(n, cfg["vocab"], 50 + n) for n in (5, 1, 40)]
     outs = eng.generate(prompts, SamplingParams(temperature=0.0, max_tokens=9, ignore_eos=True))
