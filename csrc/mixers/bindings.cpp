@@ -71,7 +71,8 @@ int mx_talk_attention(void* out, int out_bf16, float* ws_acc, float* ws_ml, cons
                       long gate_stride, const void* k_cache, const void* v_cache, int cache_bf16, const int* start,
                       const int* pos0, const int* kv_len, const int* bt, int bt_stride, int num_segs, long total_rows,
                       int heads, int kv_heads, int dk, int dv, int window, int keep_first, float softcap,
-                      const float* talk, int block_size, int num_blocks, int skip_from, int splits, hipStream_t s);
+                      const float* talk, float q_mult, int has_sink, float sink_all, const float* sinks, int block_size,
+                      int num_blocks, int skip_from, int splits, hipStream_t s);
 int mx_talk_weights(float* S, float* inv, int heads, int rows, int keys, int first_pos, int key0, int ext, int window,
                     int keep_first, float softcap, const float* talk, hipStream_t s);
 int mx_heads_to_rows(void* out, int out_bf16, const float* o, const float* inv, const void* gate, long gate_stride,
@@ -1109,12 +1110,11 @@ const void* gate_rows(const OptT& gate, const Tensor& out, int64_t rows, int64_t
 
 void talk_attention(Tensor out, Tensor q, OptT gate, Tensor k_cache, Tensor v_cache, Tensor start, Tensor pos0,
                     Tensor kv_len, Tensor bt, int64_t num_segs, int64_t max_rows, int64_t heads, int64_t kv_heads,
-                    int64_t dk, int64_t dv, int64_t window, int64_t keep_first, double softcap, Tensor talk,
-                    int64_t skip_from, int64_t max_kv) {
+                    int64_t dk, int64_t dv, int64_t window, int64_t keep_first, double softcap, OptT talk,
+                    int64_t skip_from, int64_t max_kv, double q_mult, c10::optional<double> sink, OptT sinks) {
   check_f32(q, "q");
-  check_f32(talk, "head mix");
   TORCH_CHECK(heads >= 1 && heads <= mx_talk_max_heads() && kv_heads >= 1 && heads % kv_heads == 0 && dk >= 1 &&
-              dv >= 1 && dv <= 512 && keep_first >= 0 && talk.numel() == heads * heads, "talk_attention sizes");
+              dv >= 1 && dv <= 512 && keep_first >= 0, "talk_attention sizes");
   const int64_t t = q.size(0);
   TORCH_CHECK(q.dim() == 2 && q.size(1) == heads * dk && out.is_cuda() && out.is_contiguous() && is_act(out) &&
               out.dim() == 2 && out.size(0) == t && out.size(1) == heads * dv, "q / out");
@@ -1139,8 +1139,9 @@ void talk_attention(Tensor out, Tensor q, OptT gate, Tensor k_cache, Tensor v_ca
                         gp, gs, k_cache.data_ptr(), v_cache.data_ptr(), bf(k_cache), start.data_ptr<int>(),
                         pos0.data_ptr<int>(), kv_len.data_ptr<int>(), bt.data_ptr<int>(), (int)bt.size(1),
                         (int)num_segs, t, (int)heads, (int)kv_heads, (int)dk, (int)dv, (int)window, (int)keep_first,
-                        (float)softcap, talk.data_ptr<float>(), (int)k_cache.size(1), (int)k_cache.size(0),
-                        (int)skip_from, (int)splits, stream()), "talk_attention");
+                        (float)softcap, opt_f32(talk, heads * heads, "head mix"), (float)q_mult, sink || sinks ? 1 : 0,
+                        sink ? (float)*sink : 0.f, opt_f32(sinks, heads, "sinks"), (int)k_cache.size(1),
+                        (int)k_cache.size(0), (int)skip_from, (int)splits, stream()), "talk_attention");
 }
 
 void talk_weights(Tensor S, Tensor inv, int64_t first_pos, int64_t key0, int64_t ext, int64_t window,

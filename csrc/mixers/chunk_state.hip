@@ -442,8 +442,8 @@ delta_solve_kernel(float* __restrict__ ws_w, float* __restrict__ ws_k, float* __
 // lane (hi, lo) is row 4 hi + r, column lo, which is also a right-hand operand whose inner index
 // 4 hi + r the left-hand operands (16-byte loads) follow.  Per chunk: every wave's part of
 // -W S for all 64 rows, the parts added through LDS (wave w adds U and owns rows 16 w ..), w left
-// in place of U, then S <- e^{G_last} S + K^T w.  The next chunk's operands are loaded under
-// the current chunk's products.
+// in place of U, then S <- e^{G_last} S + K^T w.  Two register sets keep a chunk's operands
+// on their way while the chunk before is computed.
 // ---------------------------------------------------------------------------------
 template <int DKT>
 __global__ void __launch_bounds__(256)
@@ -470,9 +470,12 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
       const int row = 16 * (wave * IT + ii) + 4 * hi + r;
       S[ii][r] = c.pos > 0 && mine && live && row < dk ? sp[(long)row * dv] : 0.f;
     }
-  f32x4 wf[4][IT], kf[IT][4], uf;
-  float gf = 1.f;
-  auto fetch = [&](int idx) {
+  struct Ops {
+    f32x4 w[4][IT], k[IT][4], u;
+    float g;
+  };
+  auto fetch = [&](Ops& f, int idx) {
+    if (idx >= c.num) return;
     const long cs = (c.ws + idx) * heads + h;
     const float* w = ws_w + cs * kC * DKP;
     const float* k = ws_k + cs * DKP * kC;
@@ -482,19 +485,18 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
 #pragma unroll
         for (int ii = 0; ii < IT; ++ii) {
           const int i = wave * IT + ii;
-          wf[m][ii] = *reinterpret_cast<const f32x4*>(w + (16 * m + lo) * DKP + 16 * i + 4 * hi);
-          kf[ii][m] = *reinterpret_cast<const f32x4*>(k + (16 * i + lo) * kC + 16 * m + 4 * hi);
+          f.w[m][ii] = *reinterpret_cast<const f32x4*>(w + (16 * m + lo) * DKP + 16 * i + 4 * hi);
+          f.k[ii][m] = *reinterpret_cast<const f32x4*>(k + (16 * i + lo) * kC + 16 * m + 4 * hi);
         }
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = idx * kC + 16 * wave + 4 * hi + r;
-      uf[r] = t < n && live ? ws_u[((c.row0 + t) * heads + h) * dv + col] : 0.f;
+      f.u[r] = t < n && live ? ws_u[((c.row0 + t) * heads + h) * dv + col] : 0.f;
     }
-    gf = ws_g[cs];
+    f.g = ws_g[cs];
   };
-  fetch(0);
-  for (int idx = 0; idx < c.num; ++idx) {
+  auto turn = [&](const Ops& f, int idx) {
     float* so = ws_s + (((c.ws + idx) * heads + h) * dk) * (long)dv + col;
     if (mine && live) {
 #pragma unroll
@@ -512,12 +514,12 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
 #pragma unroll
         for (int ii = 0; ii < IT; ++ii)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) a = mma(wf[m][ii][r], S[ii][r], a);
+          for (int r = 0; r < 4; ++r) a = mma(f.w[m][ii][r], S[ii][r], a);
       }
       part[m][wave][lane] = a;
     }
     __syncthreads();
-    f32x4 v = uf;
+    f32x4 v = f.u;
 #pragma unroll
     for (int w = 0; w < 4; ++w) v += part[wave][w][lane];
     whole[wave][lane] = v;
@@ -526,26 +528,29 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
       const int t = idx * kC + 16 * wave + 4 * hi + r;
       if (t < n && live) ws_u[((c.row0 + t) * heads + h) * dv + col] = v[r];
     }
-    f32x4 kc[IT][4];
-    const float g = gf;
-#pragma unroll
-    for (int ii = 0; ii < IT; ++ii)
-#pragma unroll
-      for (int m = 0; m < 4; ++m) kc[ii][m] = kf[ii][m];
-    if (idx + 1 < c.num) fetch(idx + 1);
     __syncthreads();
     if (mine) {
 #pragma unroll
-      for (int ii = 0; ii < IT; ++ii) S[ii] *= g;
+      for (int ii = 0; ii < IT; ++ii) S[ii] *= f.g;
 #pragma unroll
       for (int m = 0; m < 4; ++m) {
         const f32x4 vm = whole[m][lane];
 #pragma unroll
         for (int ii = 0; ii < IT; ++ii)
 #pragma unroll
-          for (int r = 0; r < 4; ++r) S[ii] = mma(kc[ii][m][r], vm[r], S[ii]);
+          for (int r = 0; r < 4; ++r) S[ii] = mma(f.k[ii][m][r], vm[r], S[ii]);
       }
     }
+  };
+  Ops fa, fb;
+  fetch(fa, 0);
+  fetch(fb, 1);
+  for (int idx = 0; idx < c.num; idx += 2) {
+    turn(fa, idx);
+    fetch(fa, idx + 2);
+    if (idx + 1 >= c.num) break;
+    turn(fb, idx + 1);
+    fetch(fb, idx + 3);
   }
   if (mine && live) {
 #pragma unroll

@@ -220,15 +220,14 @@ head_walk_kernel(float* __restrict__ o, HeadIn in, float* __restrict__ state, co
 }
 
 // ---------------------------------------------------------------------------------
-// inputs of the delta rule with one decay per head, one wave per (row, item): items are the
-// 2 kv_heads heads of q and k, then v in pieces of 256 channels, then one item for all heads'
-// decays and steps.  Every channel of q, k and v passes its causal convolution over time
-// (taps along the row axis; rows before the segment's first come from the slot's history,
-// zeros at position 0) and silu, in fp32; a q or k head is then divided by its length.  A
-// one-row segment shifts its history here (each channel is one lane's own); longer ones are
-// left to conv_hist_kernel.
+// inputs of the delta rule with one decay per head, one wave per (RB rows, item): items are the
+// 2 kv_heads heads of q and k, then v in pieces of 64 NU channels, then one item for all heads'
+// decays and steps.  Every channel of q, k and v passes its causal convolution over time (rows
+// before the segment's first come from the slot's history, zeros at position 0) and silu, in
+// fp32; a q or k head is then divided by its length.  A one-row segment leaves its history here
+// (each channel is one lane's own); longer ones are left to conv_hist_kernel.
 // ---------------------------------------------------------------------------------
-template <typename T>
+template <typename T, int TAPS, int NU, int RB>
 __global__ void __launch_bounds__(256)
 conv_delta_prep_kernel(float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ vo, float* __restrict__ lg,
                        float* __restrict__ beta, const T* __restrict__ x, long x_stride, const T* __restrict__ a,
@@ -238,60 +237,68 @@ conv_delta_prep_kernel(float* __restrict__ qn, float* __restrict__ kn, float* __
                        int num_segs, int num_slots, int heads, int kv_heads, int dk, int dv) {
   const int lane = threadIdx.x & 63;
   const int item = blockIdx.y * 4 + (threadIdx.x >> 6);
-  const int row = blockIdx.x;
-  const int qk = 2 * kv_heads, nv = heads * dv, pieces = (nv + 255) / 256;
-  if (item > qk + pieces || row >= start[num_segs]) return;
+  const int row0 = blockIdx.x * RB, rows = start[num_segs];
+  const int qk = 2 * kv_heads, nv = heads * dv, pieces = (nv + 64 * NU - 1) / (64 * NU);
+  if (item > qk + pieces || row0 >= rows) return;
   if (item == qk + pieces) {
-    for (int h = lane; h < heads; h += 64) {
+    for (int e = lane; e < RB * heads; e += 64) {
+      const int row = row0 + e / heads, h = e % heads;
+      if (row >= rows) break;
       const float z = ld(a, (long)row * a_stride + h) + dt_bias[h];
       lg[(long)row * heads + h] = -expf(a_log[h]) * softplusf_(z);
       beta[(long)row * heads + h] = sigmoidf_(ld(b, (long)row * b_stride + h));
     }
     return;
   }
-  const int s = segment_of(start, num_segs, row);
-  const int r0 = start[s], n = start[s + 1] - r0, rel = row - r0;
-  const int sl = slot[s];
-  const bool mine = sl >= 0 && sl < num_slots;
-  const bool old = mine && pos0[s] > 0;
+  const bool is_v = item >= qk, is_q = item < kv_heads;
   const int channels = qk * dk + nv;
-  float* hp = hist + (long)(mine ? sl : 0) * (taps - 1) * channels;
-  auto conv = [&](int c) {
-    float acc = 0.f;
-    for (int j = 0; j < taps; ++j) {
-      const int src = rel - (taps - 1) + j;
-      float v;
-      if (src >= 0) v = ld(x, (long)(r0 + src) * x_stride + c);
-      else v = old ? hp[(long)(taps - 1 + src) * channels + c] : 0.f;
-      acc += v * conv_w[(long)c * taps + j];
-    }
-    if (mine && n == 1) {
-      for (int m = 0; m + 1 < taps - 1; ++m) hp[(long)m * channels + c] = old ? hp[(long)(m + 1) * channels + c] : 0.f;
-      if (taps > 1) hp[(long)(taps - 2) * channels + c] = ld(x, (long)row * x_stride + c);
-    }
-    return acc * sigmoidf_(acc);
-  };
-  if (item < qk) {
-    const bool is_q = item < kv_heads;
-    float* out = (is_q ? qn : kn) + ((long)row * kv_heads + (is_q ? item : item - kv_heads)) * dk;
-    float y[4], ss = 0.f;                          // dk <= 256
+  const int c0 = is_v ? qk * dk + (item - qk) * 64 * NU : item * dk;
+  const int len = is_v ? min(64 * NU, channels - c0) : dk;
+  float xs[RB][NU];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+  for (int r = 0; r < RB; ++r)
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
       const int i = lane + 64 * u;
-      y[u] = i < dk ? conv(item * dk + i) : 0.f;
+      xs[r][u] = ld(x, (long)min(row0 + r, rows - 1) * x_stride + c0 + (i < len ? i : 0));
+    }
+  ConvWalk<TAPS, NU> cv;
+  cv.weights(conv_w, taps, c0, len, lane);
+  int s = segment_of(start, num_segs, row0), at = -1;
+  const float qscale = is_q ? 1.0f / sqrtf((float)dk) : 1.f;
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    const int row = row0 + r;
+    if (row >= rows) break;
+    while (row >= start[s + 1]) ++s;
+    float* h = nullptr;
+    if (s != at) {
+      const int sl = slot[s];
+      const bool mine = sl >= 0 && sl < num_slots;
+      if (mine) h = hist + (long)sl * (taps - 1) * channels;
+      cv.begin(x, x_stride, start[s], row - start[s], mine && pos0[s] > 0 ? h : nullptr, channels, taps, c0, len, lane);
+      at = s;
+    }
+    float y[NU], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const float z = cv.step(u, xs[r][u]);
+      cv.shift(u);
+      y[u] = lane + 64 * u < len ? z * sigmoidf_(z) : 0.f;
       ss += y[u] * y[u];
     }
-    ss = ft::wave_sum(ss);
-    const float r = 1.0f / sqrtf(ss + 1e-6f) * (is_q ? 1.0f / sqrtf((float)dk) : 1.f);
-#pragma unroll
-    for (int u = 0; u < 4; ++u)
-      if (lane + 64 * u < dk) out[lane + 64 * u] = y[u] * r;
-  } else {
-#pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int c = (item - qk) * 256 + lane + 64 * u;
-      if (c < nv) vo[(long)row * nv + c] = conv(qk * dk + c);
+    if (h != nullptr && start[s + 1] - start[s] == 1) cv.store(h, channels, taps, c0, len, lane);
+    float* out;
+    float f = 1.f;
+    if (is_v) {
+      out = vo + (long)row * nv + (item - qk) * 64 * NU;
+    } else {
+      out = (is_q ? qn : kn) + ((long)row * kv_heads + (is_q ? item : item - kv_heads)) * dk;
+      f = 1.0f / sqrtf(ft::wave_sum(ss) + 1e-6f) * qscale;
     }
+#pragma unroll
+    for (int u = 0; u < NU; ++u)
+      if (lane + 64 * u < len) out[lane + 64 * u] = y[u] * f;
   }
 }
 
@@ -312,13 +319,28 @@ extern "C" int mx_conv_delta_prep(float* qn, float* kn, float* vo, float* lg, fl
                                   long rows, int num_slots, int heads, int kv_heads, int dk, int dv, hipStream_t s) {
   if (rows <= 0 || num_segs <= 0) return 0;
   if (taps < 1 || taps > 16 || dk < 1 || dk > mx_head_max_dk() || dv < 1 || kv_heads < 1 || heads % kv_heads) return -1;
-  const int items = 2 * kv_heads + (heads * dv + 255) / 256 + 1;
+  // rows per wave: a few once there are enough of them
+  const int rb = rows >= 256 ? 8 : 1, nu = dk <= 64 ? 1 : dk <= 128 ? 2 : 4;
+  const int items = 2 * kv_heads + (heads * dv + 64 * nu - 1) / (64 * nu) + 1;
   if (rows > 0x7fffffffL || (items + 3) / 4 > 65535) return -2;
-  const dim3 grid((unsigned)rows, (unsigned)((items + 3) / 4));
-  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((conv_delta_prep_kernel<T>), grid, dim3(256), 0, s, qn, kn, vo, lg, beta,
-                                         (const T*)x, x_stride, (const T*)a, a_stride, (const T*)b, b_stride, conv_w,
-                                         taps, hist, a_log, dt_bias, start, pos0, slot, num_segs, num_slots, heads,
-                                         kv_heads, dk, dv));
+  const dim3 grid((unsigned)((rows + rb - 1) / rb), (unsigned)((items + 3) / 4));
+#define MX_CDP(TAPS, NU, RB)                                                                                      \
+  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((conv_delta_prep_kernel<T, TAPS, NU, RB>), grid, dim3(256), 0, s, qn, kn, vo, \
+                                         lg, beta, (const T*)x, x_stride, (const T*)a, a_stride, (const T*)b, b_stride, \
+                                         conv_w, taps, hist, a_log, dt_bias, start, pos0, slot, num_segs, num_slots,  \
+                                         heads, kv_heads, dk, dv))
+#define MX_CDN(TAPS, RB)            \
+  do {                              \
+    if (nu == 1) MX_CDP(TAPS, 1, RB); \
+    else if (nu == 2) MX_CDP(TAPS, 2, RB); \
+    else MX_CDP(TAPS, 4, RB);       \
+  } while (0)
+  if (taps <= 4 && rb == 8) MX_CDN(4, 8);
+  else if (taps <= 4) MX_CDN(4, 1);
+  else if (rb == 8) MX_CDN(16, 8);
+  else MX_CDN(16, 1);
+#undef MX_CDN
+#undef MX_CDP
   int rc = (int)hipGetLastError();
   if (rc == 0 && taps > 1 && max_rows > 1)
     rc = mx_conv_hist(x, bf16, x_stride, hist, start, pos0, slot, num_segs, 2 * kv_heads * dk + heads * dv, taps,

@@ -92,6 +92,74 @@ __device__ __forceinline__ int segment_of(const int* __restrict__ start, int num
   return lo;
 }
 
+// A short causal convolution over time of one wave's channels c0 + lane + 64 u (u < NU, below
+// c0 + len), walked row by row: taps (<= TAPS) weights and the last taps - 1 inputs in
+// registers, fp32.  Missing taps in front count as zeros.
+template <int TAPS, int NU>
+struct ConvWalk {
+  float w[NU][TAPS], win[NU][TAPS];            // win[u][TAPS - 1] is the current row's input
+
+  __device__ __forceinline__ void weights(const float* __restrict__ conv_w, int taps, int c0, int len, int lane) {
+    const int pad = TAPS - taps;
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const int i = lane + 64 * u;
+      const float* p = conv_w + (long)(c0 + (i < len ? i : 0)) * taps;
+      if (TAPS == 4 && pad == 0 && ((uintptr_t)conv_w) % 16 == 0) {
+        const float4 v = *reinterpret_cast<const float4*>(p);
+        w[u][0] = v.x; w[u][1] = v.y; w[u][TAPS == 4 ? 2 : 0] = v.z; w[u][TAPS == 4 ? 3 : 0] = v.w;
+      } else {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[u][j] = j >= pad ? p[j - pad] : 0.f;
+      }
+    }
+  }
+  // the inputs before row rel of the segment that starts at row r0: rows of x, further back the
+  // history h [taps - 1][channels] (null: zeros)
+  template <typename T>
+  __device__ __forceinline__ void begin(const T* __restrict__ x, long stride, long r0, int rel, const float* h,
+                                        int channels, int taps, int c0, int len, int lane) {
+    const int pad = TAPS - taps;
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) {
+      const int src = rel - (TAPS - 1) + j;
+#pragma unroll
+      for (int u = 0; u < NU; ++u) {
+        const int i = lane + 64 * u, c = c0 + (i < len ? i : 0);
+        float v = 0.f;
+        if (j >= pad) {
+          if (src >= 0) v = ld(x, (r0 + src) * stride + c);
+          else if (h != nullptr) v = h[(long)(taps - 1 + src) * channels + c];
+        }
+        win[u][j] = v;
+      }
+    }
+  }
+  __device__ __forceinline__ float step(int u, float v) {
+    win[u][TAPS - 1] = v;
+    float acc = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) acc += win[u][j] * w[u][j];
+    return acc;
+  }
+  // to the next row
+  __device__ __forceinline__ void shift(int u) {
+#pragma unroll
+    for (int j = 0; j + 1 < TAPS; ++j) win[u][j] = win[u][j + 1];
+  }
+  // after shift(): the last taps - 1 inputs, as a history
+  __device__ __forceinline__ void store(float* h, int channels, int taps, int c0, int len, int lane) const {
+    const int pad = TAPS - taps;
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const int i = lane + 64 * u;
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j)
+        if (j >= pad && i < len) h[(long)(j - pad) * channels + c0 + i] = win[u][j];
+    }
+  }
+};
+
 // sum_sp w[sp] acc[sp * stride + c] for a wave that owns columns [c0, c0 + 256) of n: w is lane
 // sp's value (slices <= 64; a slice of weight 0 is not read).  VEC (n and stride multiples of 4,
 // 16-byte aligned): several slices per pass, 16-byte loads; out(c, value) is called once per

@@ -4,7 +4,10 @@
 // Query head h reads key and value head h / rep, rep = heads / kv_heads.  Position i sees
 // key j iff j <= i and (i - j < window, or window == 0, or j < keep_first).  With dot
 // products s_g = q_g . k (queries come scaled): s_g <- softcap tanh(s_g / softcap) when
-// softcap > 0, z_h = sum_g talk[h][g] s_g, weights = softmax of z_h over the visible keys.
+// softcap > 0, z_h = sum_g talk[h][g] s_g, weights = softmax of z_h over the visible keys;
+// optionally with a sink, one more term exp(sink) (sinks[h], or the same for all heads) in the
+// denominator.  Without `talk` the scores are not mixed (z = s): plain grouped-query attention
+// on the same tiles.
 // Every head's weight of a key needs all heads' scores of that key, so the unit of work is
 // a tile of keys for all heads together.
 // Queries, scores, weights and sums are fp32; the caches hold fp32 or bf16 rows.
@@ -190,8 +193,8 @@ talk_attn_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const fl
                  const TC* __restrict__ k_cache, const TC* __restrict__ v_cache, const int* __restrict__ start,
                  const int* __restrict__ pos0, const int* __restrict__ kv_len, const int* __restrict__ bt,
                  int bt_stride, int num_segs, int heads, int kv_heads, int dk, int dv, int window, int keep_first,
-                 float softcap, const float* __restrict__ talk, int block_size, int num_blocks, int skip_from,
-                 int splits, int vec, int lpk) {
+                 float softcap, const float* __restrict__ talk, float q_mult, int block_size, int num_blocks,
+                 int skip_from, int splits, int vec, int lpk) {
   constexpr int CAP = W * HPW;                       // heads there is room for
   constexpr int NB = (CAP + 15) / 16;                // 16-head blocks
   constexpr int RND = (HPW + 3) / 4;                 // softmax rounds of a wave (four heads each)
@@ -236,7 +239,7 @@ talk_attn_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const fl
       for (int x = 0; x < QL; ++x) {
         const int e = e0 + 64 * W * x;
         if (e < total) {
-          const float v[4] = {v4[x].x, v4[x].y, v4[x].z, v4[x].w};
+          const float v[4] = {v4[x].x * q_mult, v4[x].y * q_mult, v4[x].z * q_mult, v4[x].w * q_mult};
           float r1[4], r2[4];
           uint32_t p0[2], p1[2], p2[2];
 #pragma unroll
@@ -269,10 +272,10 @@ talk_attn_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const fl
         }
       }
   } else {
-    for (int d = tid; d < heads * dk; d += 64 * W) q_s[d] = qp[d];
+    for (int d = tid; d < heads * dk; d += 64 * W) q_s[d] = qp[d] * q_mult;
   }
   float tm[NB][NB][4];
-  load_mix<NB>(tm, talk, heads, n, qt);
+  if (talk != nullptr) load_mix<NB>(tm, talk, heads, n, qt);
   const int col = 16 * (wave & 3) + n, half = wave >> 2;   // the key and the share of the heads it scores
   const int h0 = wave * HPW;                         // this wave's heads h0 .. h0 + HPW - 1 (< heads)
   // the key head of each score this lane holds (-1: no such head)
@@ -425,7 +428,8 @@ talk_attn_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const fl
     }
 #pragma unroll
     for (int bb = 0; bb < NB; ++bb) {
-      const f32x4_t z = mix_block<NB>(tm, sc, bb);
+      f32x4_t z = {sc[bb][0], sc[bb][1], sc[bb][2], sc[bb][3]};
+      if (talk != nullptr) z = mix_block<NB>(tm, sc, bb);
 #pragma unroll
       for (int u = 0; u < 4; ++u)
         if (kh[bb][u] >= 0)
@@ -577,13 +581,14 @@ talk_attn_kernel(float* __restrict__ ws_acc, float* __restrict__ ws_ml, const fl
   }
 }
 
-// one wave per (row, head, 256 columns): merges the slices, divides by the sum, applies the
-// element-wise sigmoid gate (optional) and rounds
+// one wave per (row, head, 256 columns): merges the slices, divides by the sum (with the sink's
+// term, if there is one), applies the element-wise sigmoid gate (optional) and rounds
 template <typename TG, typename TO, bool VEC>
 __global__ void __launch_bounds__(256)
 talk_combine_kernel(TO* __restrict__ out, const float* __restrict__ ws_acc, const float* __restrict__ ws_ml,
                     const TG* __restrict__ gate, long gate_stride, const int* __restrict__ start, int num_segs,
-                    long total_rows, int heads, int dv, int skip_from, int splits) {
+                    long total_rows, int heads, int dv, int skip_from, int splits, int has_sink, float sink_all,
+                    const float* __restrict__ sinks) {
   const long pair = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (pair >= total_rows * heads) return;
   const int lane = threadIdx.x & 63;
@@ -601,9 +606,11 @@ talk_combine_kernel(TO* __restrict__ out, const float* __restrict__ ws_acc, cons
     ms = ws_ml[(b0 + (long)lane * heads) * 2];
     ls = ws_ml[(b0 + (long)lane * heads) * 2 + 1];
   }
-  const float M = ft::wave_max(ms);
+  float M = ft::wave_max(ms);
+  const float sink = sinks != nullptr ? sinks[h] : sink_all;
+  if (has_sink) M = fmaxf(M, sink);
   const float w = ms == -INFINITY ? 0.f : expf(ms - M);
-  const float L = ft::wave_sum(w * ls);
+  const float L = ft::wave_sum(w * ls) + (has_sink ? expf(sink - M) : 0.f);
   const float inv = L > 0.f ? 1.0f / L : 0.f;
   merge_slices<VEC>(ws_acc + b0 * dv, (long)heads * dv, w, splits, blockIdx.y * 256, dv, lane, [&](int c, float v) {
     v *= inv;
@@ -757,11 +764,11 @@ static void launch_talk(bool tiled, bool vecv, int ahead, dim3 grid, size_t shm,
                         float* ws_ml, const float* q, const void* k_cache, const void* v_cache, const int* start,
                         const int* pos0, const int* kv_len, const int* bt, int bt_stride, int num_segs, int heads,
                         int kv_heads, int dk, int dv, int window, int keep_first, float softcap, const float* talk,
-                        int block_size, int num_blocks, int skip_from, int splits, int vec, int lpk) {
+                        float q_mult, int block_size, int num_blocks, int skip_from, int splits, int vec, int lpk) {
 #define MX_TALK(T, V, A)                                                                                        \
   hipLaunchKernelGGL((talk_attn_kernel<TC, W, HPW, T, V, A>), grid, dim3(64 * W), shm, s, ws_acc, ws_ml,  \
                      q, (const TC*)k_cache, (const TC*)v_cache, start, pos0, kv_len, bt, bt_stride, num_segs,   \
-                     heads, kv_heads, dk, dv, window, keep_first, softcap, talk, block_size, num_blocks,        \
+                     heads, kv_heads, dk, dv, window, keep_first, softcap, talk, q_mult, block_size, num_blocks, \
                      skip_from, splits, vec, lpk)
   if constexpr (sizeof(TC) == 2) {
     if (tiled && ahead == 16) MX_TALK(true, true, 16);
@@ -779,8 +786,9 @@ extern "C" int mx_talk_attention(void* out, int out_bf16, float* ws_acc, float* 
                                  const void* gate, long gate_stride, const void* k_cache, const void* v_cache,
                                  int cache_bf16, const int* start, const int* pos0, const int* kv_len, const int* bt,
                                  int bt_stride, int num_segs, long total_rows, int heads, int kv_heads, int dk,
-                                 int dv, int window, int keep_first, float softcap, const float* talk,
-                                 int block_size, int num_blocks, int skip_from, int splits, hipStream_t s) {
+                                 int dv, int window, int keep_first, float softcap, const float* talk, float q_mult,
+                                 int has_sink, float sink_all, const float* sinks, int block_size, int num_blocks,
+                                 int skip_from, int splits, hipStream_t s) {
   if (num_segs <= 0 || total_rows <= 0) return 0;
   if (heads < 1 || heads > mx_talk_max_heads() || kv_heads < 1 || heads % kv_heads || dk < 1 || dv < 1 ||
       dv > 64 * kScalarCols || ((uintptr_t)talk) % 16 || ((uintptr_t)q) % 16 || keep_first < 0 || splits < 1 || splits > 64)
@@ -807,7 +815,7 @@ extern "C" int mx_talk_attention(void* out, int out_bf16, float* ws_acc, float* 
 #define MX_TL(W, H)                                                                                                  \
   MX_DISPATCH_T(cache_bf16, (launch_talk<T, W, H>(tiled, vecv, ahead, grid, shm, s, ws_acc, ws_ml, q, k_cache, v_cache, \
                                                start, pos0, kv_len, bt, bt_stride, num_segs, heads, kv_heads, dk,  \
-                                               dv, window, keep_first, softcap, talk, block_size, num_blocks,      \
+                                               dv, window, keep_first, softcap, talk, q_mult, block_size, num_blocks, \
                                                skip_from, splits, vec, lpk)))
   if (waves == 8) MX_TL(8, 4);
   else if (hpw == 1) MX_TL(4, 1);
@@ -819,7 +827,7 @@ extern "C" int mx_talk_attention(void* out, int out_bf16, float* ws_acc, float* 
 #define MX_TC(V)                                                                                                \
   MX_DISPATCH_T(out_bf16, hipLaunchKernelGGL((talk_combine_kernel<T, T, V>), g2, dim3(256), 0, s, (T*)out,      \
                                              ws_acc, ws_ml, (const T*)gate, gate_stride, start, num_segs,       \
-                                             total_rows, heads, dv, skip_from, splits))
+                                             total_rows, heads, dv, skip_from, splits, has_sink, sink_all, sinks))
   if (dv % 4 == 0 && ((uintptr_t)ws_acc) % 16 == 0) MX_TC(true);
   else MX_TC(false);
 #undef MX_TC

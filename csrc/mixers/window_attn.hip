@@ -88,17 +88,17 @@ __global__ void attn_prep_kernel(float* __restrict__ q_out, const T* __restrict_
 }
 
 // ---------------------------------------------------------------------------------
-// one wave per (row, chunk) of the fused [q | k | v] projection, a chunk being one head
+// one wave per (RB rows, chunk) of the fused [q | k | v] projection, a chunk being one head
 // of q or k (head_dim channels) or up to head_dim channels of v: a causal convolution
-// over time on every channel (taps along the row axis, the last tap on the row itself;
-// rows before the segment's first come from the state slot's history, zeros at position
-// 0), then, for q and k, the head's RMS norm with one weight vector shared by the heads and
-// rotary positions (each optional), fp32 throughout.  The convolved chunk waits in the wave's
-// LDS strip between the two passes.  q leaves as fp32, k and v go to the row's cache slot.  A
-// one-row segment shifts its history here (each channel is one lane's own); longer segments'
-// histories are updated afterwards by mx_conv_hist.  grid (rows, ceil(chunks / 4)), 4 waves.
+// over time on every channel (rows before the segment's first come from the state slot's
+// history, zeros at position 0), then, for q and k, the head's RMS norm with one weight
+// vector shared by the heads and rotary positions (each optional), fp32 throughout.  Rotation
+// pairs change lanes through the wave's LDS strip.  q leaves as fp32, k and v go to the row's
+// cache slot.  A one-row segment leaves its history here (each channel is one lane's own);
+// longer segments' histories are updated afterwards by mx_conv_hist.  grid (ceil(rows / RB),
+// ceil(chunks / 4)), 4 waves; head_dim <= 64 NU.
 // ---------------------------------------------------------------------------------
-template <typename T, typename TC>
+template <typename T, typename TC, int TAPS, int NU, int RB>
 __global__ void __launch_bounds__(256)
 conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long stride, int nq, int nk, int nv,
                       const float* __restrict__ conv_w, int taps, float* hist,
@@ -107,65 +107,88 @@ conv_attn_prep_kernel(float* __restrict__ q_out, const T* __restrict__ qkv, long
                       const float* __restrict__ wk, float eps, int head_dim, const int* __restrict__ slots,
                       TC* __restrict__ k_cache, TC* __restrict__ v_cache, long num_slots,
                       const float* __restrict__ table, int table_rows, int rot_dims, int interleaved) {
-  extern __shared__ float smem[];
+  __shared__ float strip[4][64 * NU];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float* y = smem + wave * head_dim;
+  float* y_s = strip[wave];
   const int channels = nq + nk + nv;
   const int qk_chunks = (nq + nk) / head_dim;
   const int chunks = qk_chunks + (nv + head_dim - 1) / head_dim;
   const int ch = blockIdx.y * 4 + wave;
-  const int row = blockIdx.x;
-  if (ch >= chunks || row >= start[num_segs]) return;
-  const int s = segment_of(start, num_segs, row);
-  const int r0 = start[s], n = start[s + 1] - r0, rel = row - r0;
-  const int sl = slot[s];
-  const bool mine = sl >= 0 && sl < num_state_slots;
-  const bool old = mine && pos0[s] > 0;                              // the slot's history counts
-  float* h = hist + (long)(mine ? sl : 0) * (taps - 1) * channels;
+  const int row0 = blockIdx.x * RB, rows = start[num_segs];
+  if (ch >= chunks || row0 >= rows) return;
   const int c0 = ch * head_dim;
   const int len = min(head_dim, channels - c0);
-  float ss = 0.f;
-  for (int i = lane; i < len; i += 64) {
-    const int c = c0 + i;
-    float acc = 0.f;
-    for (int j = 0; j < taps; ++j) {
-      const int src = rel - (taps - 1) + j;
-      float v;
-      if (src >= 0) v = ld(qkv, (long)(r0 + src) * stride + c);
-      else v = old ? h[(long)(taps - 1 + src) * channels + c] : 0.f;
-      acc += v * conv_w[(long)c * taps + j];
+  float xs[RB][NU];
+#pragma unroll
+  for (int r = 0; r < RB; ++r)
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const int i = lane + 64 * u;
+      xs[r][u] = ld(qkv, (long)min(row0 + r, rows - 1) * stride + c0 + (i < len ? i : 0));
     }
-    if (mine && n == 1) {
-      for (int m = 0; m + 1 < taps - 1; ++m) h[(long)m * channels + c] = old ? h[(long)(m + 1) * channels + c] : 0.f;
-      if (taps > 1) h[(long)(taps - 2) * channels + c] = ld(qkv, (long)row * stride + c);
+  ConvWalk<TAPS, NU> cv;
+  cv.weights(conv_w, taps, c0, len, lane);
+  const bool is_q = c0 < nq, is_v = ch >= qk_chunks;
+  const float* w = is_v ? nullptr : is_q ? wq : wk;
+  float wn[NU];
+#pragma unroll
+  for (int u = 0; u < NU; ++u) wn[u] = w != nullptr && lane + 64 * u < len ? w[lane + 64 * u] : 1.f;
+  int s = segment_of(start, num_segs, row0), at = -1;
+#pragma unroll
+  for (int r = 0; r < RB; ++r) {
+    const int row = row0 + r;
+    if (row >= rows) break;
+    while (row >= start[s + 1]) ++s;
+    float* h = nullptr;
+    if (s != at) {
+      const int sl = slot[s];
+      const bool mine = sl >= 0 && sl < num_state_slots;
+      if (mine) h = hist + (long)sl * (taps - 1) * channels;
+      cv.begin(qkv, stride, start[s], row - start[s], mine && pos0[s] > 0 ? h : nullptr, channels, taps, c0, len, lane);
+      at = s;
     }
-    y[i] = acc;
-    ss += acc * acc;
-  }
-  const long cs = slots[row];
-  const bool keep = cs >= 0 && cs < num_slots;
-  if (ch < qk_chunks) {
-    const bool is_q = c0 < nq;
-    const float* w = is_q ? wq : wk;
-    float r = 1.f;
-    if (w != nullptr) r = 1.0f / sqrtf(ft::wave_sum(ss) / (float)head_dim + eps);
-    const float* trow = nullptr;
+    float y[NU], ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      y[u] = cv.step(u, xs[r][u]);
+      cv.shift(u);
+      if (lane + 64 * u < len) ss += y[u] * y[u];
+    }
+    if (h != nullptr && start[s + 1] - start[s] == 1) cv.store(h, channels, taps, c0, len, lane);
+    const long cs = slots[row];
+    const bool keep = cs >= 0 && cs < num_slots;
+    if (is_v) {
+      if (keep) {
+#pragma unroll
+        for (int u = 0; u < NU; ++u)
+          if (lane + 64 * u < len) st(v_cache, cs * nv + (c0 - nq - nk) + lane + 64 * u, y[u]);
+      }
+      continue;
+    }
+    if (w != nullptr) {
+      const float f = 1.0f / sqrtf(ft::wave_sum(ss) / (float)head_dim + eps);
+#pragma unroll
+      for (int u = 0; u < NU; ++u) y[u] *= f * wn[u];
+    }
     if (table != nullptr) {
-      if (w != nullptr)
-        for (int i = lane; i < len; i += 64) y[i] *= r * w[i];
-      int pos = pos0[s] + rel;
+      int pos = pos0[s] + row - start[s];
       if (pos < 0 || pos >= table_rows) pos = 0;
-      trow = table + (long)pos * rot_dims;
-      wave_lds_fence();                // rotation pairs cross lanes
+      const float* trow = table + (long)pos * rot_dims;
+      wave_lds_fence();                // the row before has been read
+#pragma unroll
+      for (int u = 0; u < NU; ++u) y_s[lane + 64 * u] = y[u];
+      wave_lds_fence();
+#pragma unroll
+      for (int u = 0; u < NU; ++u)
+        if (lane + 64 * u < rot_dims) y[u] = rope_at(y_s, lane + 64 * u, rot_dims, trow, interleaved);
     }
-    for (int i = lane; i < len; i += 64) {
-      const float v = trow != nullptr ? (i < rot_dims ? rope_at(y, i, rot_dims, trow, interleaved) : y[i])
-                                      : w != nullptr ? y[i] * r * w[i] : y[i];
-      if (is_q) q_out[(long)row * nq + c0 + i] = v;
-      else if (keep) st(k_cache, cs * nk + (c0 - nq) + i, v);
+#pragma unroll
+    for (int u = 0; u < NU; ++u) {
+      const int i = lane + 64 * u;
+      if (i >= len) continue;
+      if (is_q) q_out[(long)row * nq + c0 + i] = y[u];
+      else if (keep) st(k_cache, cs * nk + (c0 - nq) + i, y[u]);
     }
-  } else if (keep) {
-    for (int i = lane; i < len; i += 64) st(v_cache, cs * nv + (c0 - nq - nk) + i, y[i]);
   }
 }
 
@@ -534,19 +557,36 @@ extern "C" int mx_conv_attn_prep(float* q_out, const void* qkv, int bf16, long s
   if (rot_dims < 0 || rot_dims % 2 || rot_dims > head_dim || (table != nullptr && table_rows < 1)) return -1;
   if (head_dim < 1 || nq % head_dim || nk % head_dim || taps < 1 || nv < 0) return -1;
   const int channels = nq + nk + nv;
-  const size_t shm = (size_t)4 * head_dim * sizeof(float);
   const int chunks = (nq + nk) / head_dim + (nv + head_dim - 1) / head_dim;
-  if (shm > 64 * 1024 || rows > 0x7fffffffL || (chunks + 3) / 4 > 65535) return -3;
-  const dim3 grid((unsigned)rows, (unsigned)((chunks + 3) / 4)), block(256);
-#define MX_CPREP(T, TC)                                                                                       \
-  hipLaunchKernelGGL((conv_attn_prep_kernel<T, TC>), grid, block, shm, s, q_out, (const T*)qkv, stride, nq, nk, \
-                     nv, conv_w, taps, hist, start, pos0, slot, num_segs, num_state_slots, wq, wk, eps,         \
-                     head_dim, slots, (TC*)k_cache, (TC*)v_cache, num_slots, rot_dims > 0 ? table : nullptr, table_rows, \
-                     rot_dims, interleaved)
-  if (bf16 && cache_bf16) MX_CPREP(bf16_t, bf16_t);
-  else if (bf16) MX_CPREP(bf16_t, float);
-  else if (cache_bf16) MX_CPREP(float, bf16_t);
-  else MX_CPREP(float, float);
+  if (head_dim > 512 || rows > 0x7fffffffL || (chunks + 3) / 4 > 65535) return -3;
+  // rows per wave: a few once there are enough of them
+  const int rb = rows >= 256 && head_dim <= 256 && taps <= 4 ? 8 : 1;
+  const int nu = head_dim <= 64 ? 1 : head_dim <= 128 ? 2 : head_dim <= 256 ? 4 : 8;
+  const dim3 grid((unsigned)((rows + rb - 1) / rb), (unsigned)((chunks + 3) / 4)), block(256);
+#define MX_CPREP(T, TC, TAPS, NU, RB)                                                                            \
+  hipLaunchKernelGGL((conv_attn_prep_kernel<T, TC, TAPS, NU, RB>), grid, block, 0, s, q_out, (const T*)qkv, stride, nq, \
+                     nk, nv, conv_w, taps, hist, start, pos0, slot, num_segs, num_state_slots, wq, wk, eps,       \
+                     head_dim, slots, (TC*)k_cache, (TC*)v_cache, num_slots, rot_dims > 0 ? table : nullptr,      \
+                     table_rows, rot_dims, interleaved)
+#define MX_CPN(T, TC)                                  \
+  do {                                                 \
+    if (taps > 4) {                                    \
+      if (nu <= 4) MX_CPREP(T, TC, 16, 4, 1);          \
+      else MX_CPREP(T, TC, 16, 8, 1);                  \
+    } else if (rb == 8) {                              \
+      if (nu == 1) MX_CPREP(T, TC, 4, 1, 8);           \
+      else if (nu == 2) MX_CPREP(T, TC, 4, 2, 8);      \
+      else MX_CPREP(T, TC, 4, 4, 8);                   \
+    } else {                                           \
+      if (nu <= 2) MX_CPREP(T, TC, 4, 2, 1);           \
+      else if (nu == 4) MX_CPREP(T, TC, 4, 4, 1);      \
+      else MX_CPREP(T, TC, 4, 8, 1);                   \
+    }                                                  \
+  } while (0)
+  if (bf16 && cache_bf16) MX_CPN(bf16_t, bf16_t);
+  else if (!bf16 && !cache_bf16) MX_CPN(float, float);
+  else return -4;                        // the cache is kept in the activations' dtype
+#undef MX_CPN
 #undef MX_CPREP
   int rc = (int)hipGetLastError();
   if (rc == 0 && taps > 1 && max_rows > 1)

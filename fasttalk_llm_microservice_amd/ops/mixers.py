@@ -629,6 +629,15 @@ def _sink_args(sink):
     return (None, sink) if isinstance(sink, torch.Tensor) else (sink, None)
 
 
+def _plain_tiles(sp: WindowSpec, k_cache) -> bool:
+    """Softmax attention over a window (or every earlier key) without distance terms, bf16 rows of
+    whole 16-byte pieces, query heads that fit the tile kernel's LDS: all heads of a row share
+    its key tiles there, scores on the matrix units."""
+    return bool(k_cache.dtype == torch.bfloat16 and not sp.sigmoid and sp.maps == 1 and not sp.blocks and sp.r1 is None
+                and sp.dist_bias is None and sp.dk % 8 == 0 and sp.dv % 8 == 0 and sp.dv <= 512
+                and sp.heads <= 64 and sp.heads * sp.dk <= 4096)
+
+
 def window_attention(q, k_cache, v_cache, seg: Segments, spec: WindowSpec, skip_from: int = 0,
                      out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q fp32 [T, heads*maps*dk] against the paged caches; fp32 [T, heads*maps, dv].
@@ -638,6 +647,13 @@ def window_attention(q, k_cache, v_cache, seg: Segments, spec: WindowSpec, skip_
     if q.is_cuda:
         if out is None:
             out = torch.empty(q.shape[0], sp.heads * sp.maps, sp.dv, dtype=torch.float32, device=q.device)
+        if _plain_tiles(sp, k_cache):
+            # the tile kernel of the head-mixing attention, without a mix
+            native_mixers().talk_attention(out.view(q.shape[0], -1), q, None, k_cache, v_cache, seg.start, seg.pos0,
+                                           seg.kv_len, seg.block_tables, seg.num, seg.max_rows, sp.heads, sp.kv_heads,
+                                           sp.dk, sp.dv, sp.window, sp.keep_first, float(sp.softcap), None, skip_from,
+                                           seg.max_kv, float(sp.scale), *_sink_args(sp.sink))
+            return out
         native_mixers().window_attention(out, q, k_cache, v_cache, seg.start, seg.pos0, seg.kv_len,
                                          seg.block_tables, seg.num, seg.max_rows, sp.heads, sp.maps,
                                          sp.kv_heads, sp.dk, sp.dv, sp.window, sp.scale, sp.sigmoid,
@@ -796,7 +812,8 @@ def talk_attention(out, q, gate, k_cache, v_cache, seg: Segments, spec: TalkSpec
     if q.is_cuda:
         native_mixers().talk_attention(out, q, gate, k_cache, v_cache, seg.start, seg.pos0, seg.kv_len,
                                        seg.block_tables, seg.num, seg.max_rows, sp.heads, sp.kv_heads, sp.dk, sp.dv,
-                                       sp.window, sp.keep_first, float(sp.softcap), sp.talk, skip_from, seg.max_kv)
+                                       sp.window, sp.keep_first, float(sp.softcap), sp.talk, skip_from, seg.max_kv,
+                                       1.0, None, None)
         return out
     r = ref.talk_attention(q, k_cache, v_cache, seg, sp.heads, sp.kv_heads, sp.dk, sp.dv, sp.window, sp.keep_first,
                            sp.softcap, sp.talk)
