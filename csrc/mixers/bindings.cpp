@@ -498,7 +498,7 @@ void head_delta_rule(Tensor o, Tensor q, Tensor k, Tensor v, Tensor lg, Tensor b
   if (!chunks) return;
   const int64_t nc = chunk_bound(t, num_segs), dkp = mx_chunk_key_pad((int)dk), c = mx_chunk_rows();
   Tensor ws_s = at::empty({nc, heads, dk, dv}, o.options()), ws_w = at::empty({nc, heads, c, dkp}, o.options());
-  Tensor ws_k = at::empty({nc, heads, dkp, c}, o.options()), ws_u = at::empty({t, heads, dv}, o.options());
+  Tensor ws_k = at::empty({nc, heads, dkp, c}, o.options()), ws_u = at::empty({nc, heads, c, (dv + 15) / 16 * 16}, o.options());
   Tensor ws_g = at::empty({nc, heads}, o.options());
   chk(mx_head_delta_chunks(o.data_ptr<float>(), q.data_ptr<float>(), k.data_ptr<float>(), v.data_ptr<float>(),
                            lg.data_ptr<float>(), beta.data_ptr<float>(), state.data_ptr<float>(),

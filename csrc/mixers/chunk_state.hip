@@ -12,8 +12,10 @@
 // beta_t e^{G_t - G_j} (k_t.k_j) for j < t.
 //
 // Kernels:
-//   delta_solve   per (chunk, head), parallel: A on the matrix units, forward substitution with
-//                 one column of [U | W] per thread; leaves U, -W and e^{G_63 - G_j} k_j
+//   delta_solve   per (chunk, head), parallel: A, (I + A)^-1 (16-row diagonal blocks by
+//                 substitution, the rest by block products) and [U | W] on the matrix units;
+//                 leaves U, -W and e^{G_63 - G_j} k_j.  (The inverse is harmless numerically:
+//                 its entries are -beta k^T (products of I - beta k k^T) k, at most one in size.)
 //   delta_carry   per (head, 16 columns of the state), chunk after chunk: the state stays in the
 //                 accumulators of four waves (16-row tiles dealt out), whose register layout is
 //                 that of a right-hand operand; leaves w and every chunk's incoming state
@@ -22,6 +24,12 @@
 //   chunk_out     both, per (chunk, head, 64 columns), parallel: o from the incoming state
 // Sums of log decays are formed in double precision and only their differences are rounded, so
 // a chunk's decay ratios are as exact as a row-by-row walk's.
+//
+// delta_solve leaves -W, the keys and U as fragments: for every 16 x 16 tile one 16-byte piece per
+// lane (hi, lo) = (lane / 16, lane % 16), in the lanes' order, so that delta_carry's operand
+// loads are whole kilobytes: -W tile (m, i) holds rows 16 m + lo, columns 16 i + 4 hi + r; key
+// tile (i, m) columns 16 i + lo, rows 16 m + 4 hi + r; U tile (ct, m) rows 16 m + 4 hi + r, column
+// 16 ct + lo (r = 0 .. 3 the piece's entries).
 //
 // A chunk's workspace index is start[s] / 64 + s + its number within the segment: distinct
 // for all chunks of a step, below rows / 64 + segments.  Rows of a last, partial chunk past the
@@ -41,6 +49,18 @@ __device__ __forceinline__ f32x4 mma(float a, float b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
+// a product over N inner steps of 4, a(s) and b(s) the operands of step s: four sums in turn, so
+// that no product waits for the one before
+template <int N, typename A, typename B>
+__device__ __forceinline__ f32x4 dot_steps(A a, B b) {
+  f32x4 p[4];
+#pragma unroll
+  for (int u = 0; u < 4; ++u) p[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int s = 0; s < N; ++s) p[s & 3] = mma(a(s), b(s), p[s & 3]);
+  return (p[0] + p[1]) + (p[2] + p[3]);
+}
+
 struct ChunkIn {
   const void* q;
   const void* k;
@@ -52,6 +72,7 @@ struct ChunkIn {
   const float* table;                  // rotation of q and k, null: none
   int table_rows, rot_dims, interleaved;
   float k_scale;
+  int v_frags;                         // v: fragments by workspace chunk (below) instead of rows
 };
 
 // four consecutive entries as fp32 (16- or 8-byte load)
@@ -72,24 +93,26 @@ __device__ __forceinline__ void stage_head(float* dst, int LDK, const T* src, lo
                                            const float* table, int table_rows, int rot, int interleaved, int pos,
                                            float scale, int vec) {
   const int tid = threadIdx.x;
+  const int t0 = tid >> 5, l0 = tid & 31;   // without 16-byte pieces: 32 lanes per row, 8 rows at a time
   int d0 = 0;                       // entries below are rotated pairs
   if (table != nullptr && rot > 0) {
     d0 = rot;
     const int half = rot / 2;
-    for (int e = tid; e < kC * half; e += 256) {
-      const int t = e / half, i = e % half;
-      float u = 0.f, w = 0.f;
-      const int a = interleaved ? 2 * i : i, b = interleaved ? 2 * i + 1 : i + half;
-      if (t < cnt) {
-        int p = pos + t;
-        if (p < 0 || p >= table_rows) p = 0;
-        const float c = table[(long)p * rot + i], sn = table[(long)p * rot + half + i];
-        const float x = ld(src, t * stride + a), y = ld(src, t * stride + b);
-        u = (x * c - y * sn) * scale;
-        w = (y * c + x * sn) * scale;
+#pragma unroll 4
+    for (int t = t0; t < kC; t += 8) {
+      // rows past cnt read the last row and count as zeros
+      const int tt = min(t, cnt - 1);
+      int p = pos + tt;
+      if (p < 0 || p >= table_rows) p = 0;
+      const float* cs = table + (long)p * rot;
+      const float f = t < cnt ? scale : 0.f;
+      for (int i = l0; i < half; i += 32) {
+        const int a = interleaved ? 2 * i : i, b = interleaved ? 2 * i + 1 : i + half;
+        const float c = cs[i], sn = cs[half + i];
+        const float x = ld(src, tt * stride + a), y = ld(src, tt * stride + b);
+        dst[t * LDK + a] = (x * c - y * sn) * f;
+        dst[t * LDK + b] = (y * c + x * sn) * f;
       }
-      dst[t * LDK + a] = u;
-      dst[t * LDK + b] = w;
     }
   }
   if (vec && d0 == 0) {
@@ -102,12 +125,8 @@ __device__ __forceinline__ void stage_head(float* dst, int LDK, const T* src, lo
     }
     return;
   }
-  const int rest = DKP - d0;
-  if (rest <= 0) return;
-  for (int e = tid; e < kC * rest; e += 256) {
-    const int t = e / rest, i = d0 + e % rest;
-    dst[t * LDK + i] = t < cnt && i < dk ? ld(src, t * stride + i) * scale : 0.f;
-  }
+  for (int t = t0; t < kC; t += 8)
+    for (int i = d0 + l0; i < DKP; i += 32) dst[t * LDK + i] = t < cnt && i < dk ? ld(src, t * stride + i) * scale : 0.f;
 }
 
 // rows [0, cnt) x 64 columns from col0 of a [., dv] array into LDS [kC][kVLD], zeros elsewhere
@@ -295,7 +314,22 @@ chunk_out_kernel(float* __restrict__ o, ChunkIn in, const float* __restrict__ ws
   }
   stage_head<T, DKP>(kb, LDK, (const T*)in.k + c.row0 * in.k_stride + hoff, in.k_stride, c.cnt, dk, in.table,
                      in.table_rows, in.rot_dims, in.interleaved, c.pos, in.k_scale, vec);
-  stage_cols<T>(vb, (const T*)in.v + c.row0 * in.v_stride + (long)h * dv, in.v_stride, c.cnt, col0, dv, vec);
+  if (in.v_frags) {
+    const int tiles = (dv + 15) / 16;
+    const float4* fp = (const float4*)in.v + (c.ws * heads + h) * (long)tiles * 256;
+    for (int ct = wave; ct < 4; ct += 4) {
+      const int tile = min(col0 / 16 + ct, tiles - 1);       // columns past dv are not stored
+#pragma unroll
+      for (int m = 0; m < 4; ++m) {
+        const float4 u = fp[(tile * 4 + m) * 64 + lane];
+        const float v[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vb[(16 * m + 4 * hi + r) * kVLD + 16 * ct + lo] = v[r];
+      }
+    }
+  } else {
+    stage_cols<T>(vb, (const T*)in.v + c.row0 * in.v_stride + (long)h * dv, in.v_stride, c.cnt, col0, dv, vec);
+  }
   double gr[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
@@ -309,9 +343,8 @@ chunk_out_kernel(float* __restrict__ o, ChunkIn in, const float* __restrict__ ws
 #pragma unroll
   for (int jt = 0; jt < 4; ++jt) {
     if (jt > wave) continue;                                 // keys behind every row of this wave
-    f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int s = 0; s < 4 * DKT; ++s) a = mma(qf[s], kb[(16 * jt + lo) * LDK + 4 * s + hi], a);
+    const float* kr = kb + (16 * jt + lo) * LDK + hi;
+    f32x4 a = dot_steps<4 * DKT>([&](int s) { return qf[s]; }, [&](int s) { return kr[4 * s]; });
     const double gj = G[16 * jt + lo];
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -349,8 +382,8 @@ chunk_out_kernel(float* __restrict__ o, ChunkIn in, const float* __restrict__ ws
 }
 
 // ---------------------------------------------------------------------------------
-// grid (chunks, heads, segments), 256 threads.  Leaves per chunk and head: -W [64][DKP],
-// (e^{G_last - G_j} k_j)^T [DKP][64], e^{G_last}; and U in rows [T, heads, dv].
+// grid (chunks, heads, segments), 256 threads.  Leaves per chunk and head, as fragments: -W,
+// e^{G_last - G_j} k_j and U; and e^{G_last}.
 // ---------------------------------------------------------------------------------
 template <int DKT>
 __global__ void __launch_bounds__(256)
@@ -359,8 +392,8 @@ delta_solve_kernel(float* __restrict__ ws_w, float* __restrict__ ws_k, float* __
                    const int* __restrict__ pos0, const int* __restrict__ slot, int heads, int dk, int dv, int num_slots,
                    int min_rows, int vec) {
   constexpr int DKP = 16 * DKT, LDK = DKP + 4;
-  // A transposed: at[j][i] = A_ij, so that the substitution reads the rows below j together
-  __shared__ __attribute__((aligned(16))) float kb[kC * LDK], at[kC * kPLD];
+  // ab: A, block by block replaced by T = (I + A)^-1 (blocks above the diagonal are never read)
+  __shared__ __attribute__((aligned(16))) float kb[kC * LDK], ab[kC * kPLD];
   __shared__ double G[kC];
   __shared__ float bs[kC], eg[kC], el[kC];
   Chunk c;
@@ -373,7 +406,7 @@ delta_solve_kernel(float* __restrict__ ws_w, float* __restrict__ ws_k, float* __
                          dk, nullptr, 0, 0, 0, 0, 1.f, vec);
   __syncthreads();
   if (tid < kC) {
-    eg[tid] = expf((float)G[tid]);
+    eg[tid] = expf((float)G[tid]) * bs[tid];
     el[tid] = expf((float)(G[kC - 1] - G[tid]));
     if (tid == 0) ws_g[c.ws * heads + h] = expf((float)G[kC - 1]);
   }
@@ -384,83 +417,141 @@ delta_solve_kernel(float* __restrict__ ws_w, float* __restrict__ ws_k, float* __
 #pragma unroll
     for (int jt = 0; jt < 4; ++jt) {
       if (jt > wave) continue;
-      f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int s = 0; s < 4 * DKT; ++s) a = mma(kf[s], kb[(16 * jt + lo) * LDK + 4 * s + hi], a);
+      const float* kr = kb + (16 * jt + lo) * LDK + hi;
+      const f32x4 a = dot_steps<4 * DKT>([&](int s) { return kf[s]; }, [&](int s) { return kr[4 * s]; });
       const int j = 16 * jt + lo;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = 16 * wave + 4 * hi + r;
-        at[j * kPLD + i] = j < i ? bs[i] * a[r] * expf((float)(G[i] - G[j])) : 0.f;
+        ab[i * kPLD + j] = j < i ? bs[i] * a[r] * expf((float)(G[i] - G[j])) : 0.f;
       }
+    }
+  }
+  wave_lds_fence();
+  {
+    // the wave's own diagonal block: lane lo holds column lo of its inverse (the four quarters
+    // of the wave do the same work)
+    float* d = ab + 16 * wave * kPLD + 16 * wave;
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) x[i] = i == lo ? 1.f : 0.f;
+#pragma unroll
+    for (int j = 0; j < 15; ++j)
+#pragma unroll
+      for (int i = j + 1; i < 16; ++i) x[i] -= d[i * kPLD + j] * x[j];
+    wave_lds_fence();
+    if (hi == 0) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) d[i * kPLD + lo] = x[i];
     }
   }
   __syncthreads();
-  float* wk = ws_k + (c.ws * heads + h) * (long)DKP * kC;
-  for (int e = tid; e < DKP * kC; e += 256) {
-    const int d = e / kC, j = e % kC;
-    wk[e] = kb[j * LDK + d] * el[j];
-  }
-  float* ww = ws_w + (c.ws * heads + h) * (long)kC * DKP;
-  for (int col = tid; col < DKP + dv; col += 256) {
-    const bool is_w = col < DKP;
-    float x[kC];
-    if (is_w) {
+  // below the diagonal, one row of blocks after the other: T_ij = -T_ii sum_{j <= k < i} A_ik T_kj
 #pragma unroll
-      for (int i = 0; i < kC; ++i) x[i] = bs[i] * eg[i] * kb[i * LDK + col];
-    } else {
-      const float* vp = (const float*)in.v + c.row0 * in.v_stride + (long)h * dv + (col - DKP);
+  for (int i = 1; i < 4; ++i) {
+    f32x4 t = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int j = wave;
+    if (j < i) {
+      f32x4 m = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < kC; ++i) x[i] = i < c.cnt ? bs[i] * vp[i * in.v_stride] : 0.f;
-    }
+      for (int k = 0; k < i; ++k) {
+        if (k < j) continue;
 #pragma unroll
-    for (int j = 0; j < kC - 1; ++j) {
-      const float xj = x[j];
-#pragma unroll
-      for (int i4 = (j + 1) / 4; i4 < kC / 4; ++i4) {
-        const float4 a = *reinterpret_cast<const float4*>(&at[j * kPLD + 4 * i4]);
-        const float av[4] = {a.x, a.y, a.z, a.w};
-#pragma unroll
-        for (int u = 0; u < 4; ++u)
-          if (4 * i4 + u > j) x[4 * i4 + u] -= av[u] * xj;
+        for (int s = 0; s < 4; ++s)
+          m = mma(ab[(16 * i + lo) * kPLD + 16 * k + 4 * s + hi], ab[(16 * k + 4 * s + hi) * kPLD + 16 * j + lo], m);
       }
-    }
-    if (is_w) {
+      // m in accumulator layout is a right-hand operand with inner index 4 hi + r
 #pragma unroll
-      for (int i = 0; i < kC; ++i) ww[(long)i * DKP + col] = -x[i];
-    } else {
-#pragma unroll
-      for (int i = 0; i < kC; ++i)
-        if (i < c.cnt) ws_u[((c.row0 + i) * heads + h) * dv + (col - DKP)] = x[i];
+      for (int r = 0; r < 4; ++r) t = mma(-ab[(16 * i + lo) * kPLD + 16 * i + 4 * hi + r], m[r], t);
     }
+    __syncthreads();
+    if (j < i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ab[(16 * i + 4 * hi + r) * kPLD + 16 * j + lo] = t[r];
+    }
+    __syncthreads();
+  }
+  // [W | U] = T [beta e^G k | beta v], column tiles dealt out to the waves
+  float tf[4][16], fw[16], fu[16];
+#pragma unroll
+  for (int m = 0; m < 4; ++m)
+#pragma unroll
+    for (int s = 0; s < 4 * m + 4; ++s) tf[m][s] = ab[(16 * m + lo) * kPLD + 4 * s + hi];
+#pragma unroll
+  for (int s = 0; s < 16; ++s) {
+    fw[s] = eg[4 * s + hi];
+    fu[s] = bs[4 * s + hi];
+  }
+  // four row tiles of T b, or of its transpose (the operands in turn: their layouts are alike)
+  auto column = [&](const float (&b)[16], f32x4 (&x)[4], auto transposed) {
+#pragma unroll
+    for (int m = 0; m < 4; ++m) x[m] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < 16; ++s)
+#pragma unroll
+      for (int m = s / 4; m < 4; ++m)
+        x[m] = decltype(transposed)::value ? mma(b[s], tf[m][s], x[m]) : mma(tf[m][s], b[s], x[m]);
+  };
+  f32x4* ww = (f32x4*)ws_w + (c.ws * heads + h) * (long)(4 * DKT * 64);
+  for (int ct = wave; ct < DKT; ct += 4) {
+    float b[16];
+    f32x4 x[4];
+#pragma unroll
+    for (int s = 0; s < 16; ++s) b[s] = -fw[s] * kb[(4 * s + hi) * LDK + 16 * ct + lo];
+    column(b, x, std::integral_constant<bool, true>{});
+#pragma unroll
+    for (int m = 0; m < 4; ++m) ww[(m * DKT + ct) * 64 + lane] = x[m];
+  }
+  const int vtiles = (dv + 15) / 16;
+  f32x4* wu = (f32x4*)ws_u + (c.ws * heads + h) * (long)vtiles * 256;
+  for (int ct = wave; ct < vtiles; ct += 4) {
+    float b[16];
+    f32x4 x[4];
+    const int col = 16 * ct + lo;
+    const float* vp = (const float*)in.v + c.row0 * in.v_stride + (long)h * dv + min(col, dv - 1);
+#pragma unroll
+    for (int s = 0; s < 16; ++s) b[s] = fu[s] * vp[min(4 * s + hi, c.cnt - 1) * in.v_stride];   // beta is 0 past cnt
+    column(b, x, std::integral_constant<bool, false>{});
+#pragma unroll
+    for (int m = 0; m < 4; ++m) wu[(ct * 4 + m) * 64 + lane] = x[m];
+  }
+  f32x4* wk = (f32x4*)ws_k + (c.ws * heads + h) * (long)(4 * DKT * 64);
+  for (int e = wave; e < 4 * DKT; e += 4) {
+    const int i = e / 4, m = e % 4;
+    f32x4 x;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) x[r] = kb[(16 * m + 4 * hi + r) * LDK + 16 * i + lo] * el[16 * m + 4 * hi + r];
+    wk[e * 64 + lane] = x;
   }
 }
 
 // ---------------------------------------------------------------------------------
-// grid (ceil(dv / 16), heads, segments), four waves: the state's 16 columns, chunk after chunk.
+// grid (heads, ceil(dv / 16), segments), four waves: the state's 16 columns, chunk after chunk.
+// (Heads come first so that, 8 XCDs taking workgroups in turn, the column tiles of a head
+// tend to share one XCD's L2: they all read the same operands.)
 // Wave w holds the 16-row tiles w IT .. w IT + IT - 1 in accumulators; accumulator register r of
 // lane (hi, lo) is row 4 hi + r, column lo, which is also a right-hand operand whose inner index
 // 4 hi + r the left-hand operands (16-byte loads) follow.  Per chunk: every wave's part of
 // -W S for all 64 rows, the parts added through LDS (wave w adds U and owns rows 16 w ..), w left
 // in place of U, then S <- e^{G_last} S + K^T w.  Two register sets keep a chunk's operands
-// on their way while the chunk before is computed.
+// on their way while the chunk before is computed.  FULL (whole tiles: dk = 16 DKT, dv a multiple of
+// 16): no access is conditional, so nothing in the loop waits for more than it uses.
 // ---------------------------------------------------------------------------------
-template <int DKT>
+template <int DKT, bool FULL>
 __global__ void __launch_bounds__(256)
 delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, const float* __restrict__ ws_k,
                    float* __restrict__ ws_u, const float* __restrict__ ws_g, float* __restrict__ state,
                    const int* __restrict__ start, const int* __restrict__ pos0, const int* __restrict__ slot, int heads,
                    int dk, int dv, int num_slots, int min_rows) {
-  constexpr int DKP = 16 * DKT, IT = DKT < 4 ? 1 : DKT / 4;
+  constexpr int IT = DKT < 4 ? 1 : DKT / 4;
   __shared__ f32x4 part[4][4][64], whole[4][64];
   Chunk c;
   if (!find_chunk(c, 0, blockIdx.z, start, pos0, slot, min_rows, num_slots)) return;
-  const int h = blockIdx.y;
+  const int h = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lo = lane & 15, hi = lane >> 4;
-  const int n = start[blockIdx.z + 1] - start[blockIdx.z];
-  const int col = blockIdx.x * 16 + lo;
-  const bool live = col < dv;
-  const bool mine = wave * IT < DKT;                 // few tiles: some waves only add
+  const int col = blockIdx.y * 16 + lo;
+  const bool live = FULL || col < dv;
+  const bool mine = DKT >= 4 || wave * IT < DKT;     // few tiles: some waves only add
   float* sp = state + (((long)c.slot * heads + h) * dk) * dv + col;
   f32x4 S[IT];
 #pragma unroll
@@ -475,26 +566,23 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
     float g;
   };
   auto fetch = [&](Ops& f, int idx) {
-    if (idx >= c.num) return;
+    idx = min(idx, c.num - 1);         // past the end: loaded again, not used
     const long cs = (c.ws + idx) * heads + h;
-    const float* w = ws_w + cs * kC * DKP;
-    const float* k = ws_k + cs * DKP * kC;
+    const f32x4* w = (const f32x4*)ws_w + cs * (4 * DKT * 64) + lane;
+    const f32x4* k = (const f32x4*)ws_k + cs * (4 * DKT * 64) + lane;
     if (mine) {
 #pragma unroll
       for (int m = 0; m < 4; ++m)
 #pragma unroll
         for (int ii = 0; ii < IT; ++ii) {
           const int i = wave * IT + ii;
-          f.w[m][ii] = *reinterpret_cast<const f32x4*>(w + (16 * m + lo) * DKP + 16 * i + 4 * hi);
-          f.k[ii][m] = *reinterpret_cast<const f32x4*>(k + (16 * i + lo) * kC + 16 * m + 4 * hi);
+          f.w[m][ii] = w[(m * DKT + i) * 64];
+          f.k[ii][m] = k[(i * 4 + m) * 64];
         }
     }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = idx * kC + 16 * wave + 4 * hi + r;
-      f.u[r] = t < n && live ? ws_u[((c.row0 + t) * heads + h) * dv + col] : 0.f;
-    }
+    f.u = ((const f32x4*)ws_u)[((cs * gridDim.y + blockIdx.y) * 4 + wave) * 64 + lane];
     f.g = ws_g[cs];
+    asm volatile("" ::: "memory");     // the loads stay here: they are not moved to their uses, two chunks on
   };
   auto turn = [&](const Ops& f, int idx) {
     float* so = ws_s + (((c.ws + idx) * heads + h) * dk) * (long)dv + col;
@@ -504,42 +592,48 @@ delta_carry_kernel(float* __restrict__ ws_s, const float* __restrict__ ws_w, con
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int row = 16 * (wave * IT + ii) + 4 * hi + r;
-          if (row < dk) so[(long)row * dv] = S[ii][r];
+          if (FULL || row < dk) so[(long)row * dv] = S[ii][r];
         }
     }
+    f32x4 a[4];
 #pragma unroll
-    for (int m = 0; m < 4; ++m) {
-      f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-      if (mine) {
-#pragma unroll
-        for (int ii = 0; ii < IT; ++ii)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) a = mma(f.w[m][ii][r], S[ii][r], a);
-      }
-      part[m][wave][lane] = a;
-    }
-    __syncthreads();
-    f32x4 v = f.u;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) v += part[wave][w][lane];
-    whole[wave][lane] = v;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = idx * kC + 16 * wave + 4 * hi + r;
-      if (t < n && live) ws_u[((c.row0 + t) * heads + h) * dv + col] = v[r];
-    }
-    __syncthreads();
+    for (int m = 0; m < 4; ++m) a[m] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (mine) {
 #pragma unroll
-      for (int ii = 0; ii < IT; ++ii) S[ii] *= f.g;
+      for (int ii = 0; ii < IT; ++ii)
 #pragma unroll
-      for (int m = 0; m < 4; ++m) {
-        const f32x4 vm = whole[m][lane];
+        for (int r = 0; r < 4; ++r)
 #pragma unroll
-        for (int ii = 0; ii < IT; ++ii)
+          for (int m = 0; m < 4; ++m) a[m] = mma(f.w[m][ii][r], S[ii][r], a[m]);
+    }
 #pragma unroll
-          for (int r = 0; r < 4; ++r) S[ii] = mma(f.k[ii][m][r], vm[r], S[ii]);
+    for (int m = 0; m < 4; ++m) part[m][wave][lane] = a[m];
+    __syncthreads();
+    {
+      const f32x4 v0 = part[wave][0][lane], v1 = part[wave][1][lane], v2 = part[wave][2][lane], v3 = part[wave][3][lane];
+      a[0] = (f.u + v0) + (v1 + (v2 + v3));
+    }
+    const f32x4 v = a[0];
+    whole[wave][lane] = v;
+    ((f32x4*)ws_u)[((((c.ws + idx) * heads + h) * gridDim.y + blockIdx.y) * 4 + wave) * 64 + lane] = v;
+    __syncthreads();
+    if (mine) {
+      f32x4 vm[4], e[IT][2];             // two sums per tile in turn
+#pragma unroll
+      for (int m = 0; m < 4; ++m) vm[m] = whole[m][lane];
+#pragma unroll
+      for (int ii = 0; ii < IT; ++ii) {
+        e[ii][0] = S[ii] * f.g;
+        e[ii][1] = f32x4{0.f, 0.f, 0.f, 0.f};
       }
+#pragma unroll
+      for (int m = 0; m < 4; ++m)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int ii = 0; ii < IT; ++ii) e[ii][r & 1] = mma(f.k[ii][m][r], vm[m][r], e[ii][r & 1]);
+#pragma unroll
+      for (int ii = 0; ii < IT; ++ii) S[ii] = e[ii][0] + e[ii][1];
     }
   };
   Ops fa, fb;
@@ -636,16 +730,24 @@ extern "C" int mx_head_delta_chunks(float* o, const float* q, const float* k, co
   in.rep = heads / kv_heads;
   in.lg = lg;
   in.k_scale = 1.f;
-  const int vec = dk % 4 == 0 && dv % 4 == 0 && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)ws_u) % 16) == 0;
+  const int vec = dk % 4 == 0 && dv % 4 == 0 && (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v) % 16) == 0;
+  if (((uintptr_t)ws_w | (uintptr_t)ws_k | (uintptr_t)ws_u) % 16) return -3;
   const int chunks = (max_rows + kC - 1) / kC;
   if (heads > 65535 || (long)heads * ((dv + 63) / 64) > 65535 || num_segs > 65535) return -2;
   key_tiles(dk, [&](auto t) {
     hipLaunchKernelGGL((delta_solve_kernel<decltype(t)::value>), dim3(chunks, heads, num_segs), dim3(256), 0, s, ws_w,
                        ws_k, ws_u, ws_g, in, beta, start, pos0, slot, heads, dk, dv, num_slots, min_rows, vec);
-    hipLaunchKernelGGL((delta_carry_kernel<decltype(t)::value>), dim3((dv + 15) / 16, heads, num_segs), dim3(256), 0, s,
-                       ws_s, ws_w, ws_k, ws_u, ws_g, state, start, pos0, slot, heads, dk, dv, num_slots, min_rows);
+    constexpr int DKT = decltype(t)::value;
+    const dim3 cgrid(heads, (dv + 15) / 16, num_segs);
+    if (dk == 16 * DKT && dv % 16 == 0)
+      hipLaunchKernelGGL((delta_carry_kernel<DKT, true>), cgrid, dim3(256), 0, s, ws_s, ws_w, ws_k, ws_u, ws_g, state, start,
+                         pos0, slot, heads, dk, dv, num_slots, min_rows);
+    else
+      hipLaunchKernelGGL((delta_carry_kernel<DKT, false>), cgrid, dim3(256), 0, s, ws_s, ws_w, ws_k, ws_u, ws_g, state, start,
+                         pos0, slot, heads, dk, dv, num_slots, min_rows);
   });
   in.v = ws_u;                     // the solved rows take the values' place
+  in.v_frags = 1;
   launch_out<float>(o, in, ws_s, start, pos0, slot, dim3(chunks, heads * ((dv + 63) / 64), num_segs), heads, dk, dv,
                     num_slots, min_rows, vec, s);
   return (int)hipGetLastError();

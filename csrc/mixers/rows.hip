@@ -490,19 +490,61 @@ __global__ void gather_add_rows_kernel(float* __restrict__ out, const TY* __rest
   }
 }
 
+// Gated linear units on rows [gate (ff) | up (ff) | ...], activation by a functor; VEC: eight
+// neighbouring bf16 (four fp32) entries per thread, 16-byte accesses
+template <typename T> struct GluVec;
+template <> struct GluVec<float> { static constexpr int N = 4; };
+template <> struct GluVec<bf16_t> { static constexpr int N = 8; };
+
+__device__ __forceinline__ void load16(const float* p, float (&v)[4]) {
+  const float4 u = *reinterpret_cast<const float4*>(p);
+  v[0] = u.x; v[1] = u.y; v[2] = u.z; v[3] = u.w;
+}
+__device__ __forceinline__ void load16(const bf16_t* p, float (&v)[8]) { ft::load8(*reinterpret_cast<const uint4*>(p), v); }
+__device__ __forceinline__ void store16(float* p, const float (&v)[4]) {
+  *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+__device__ __forceinline__ void store16(bf16_t* p, const float (&v)[8]) {
+  *reinterpret_cast<uint4*>(p) =
+      make_uint4(ft::pack2(v[0], v[1]), ft::pack2(v[2], v[3]), ft::pack2(v[4], v[5]), ft::pack2(v[6], v[7]));
+}
+
+template <typename T, typename F>
+__device__ __forceinline__ void glu_rows(T* __restrict__ out, const T* __restrict__ gu, long gu_stride, long rows, int ff,
+                                         int vec, F act) {
+  constexpr int N = GluVec<T>::N;
+  const long step = (long)gridDim.x * blockDim.x, i0 = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (vec) {
+    const int per = ff / N;
+    for (long i = i0; i < rows * per; i += step) {
+      const long r = i / per;
+      const int c = (int)(i - r * per) * N;
+      float g[N], u[N];
+      load16(gu + r * gu_stride + c, g);
+      load16(gu + r * gu_stride + ff + c, u);
+#pragma unroll
+      for (int k = 0; k < N; ++k) g[k] = act(g[k], u[k]);
+      store16(out + r * ff + c, g);
+    }
+    return;
+  }
+  for (long i = i0; i < rows * ff; i += step) {
+    const long r = i / ff;
+    const int c = (int)(i % ff);
+    st(out, i, act(ld(gu, r * gu_stride + c), ld(gu, r * gu_stride + ff + c)));
+  }
+}
+
 // rows [gate (ff) | up (ff) | ...]: g = min(gate, limit), u = clamp(up, +-limit),
 // out = g * sigmoid(1.702 g) * (u + 1)
 template <typename T>
 __global__ void clamp_swiglu_kernel(T* __restrict__ out, const T* __restrict__ gu, long gu_stride,
-                                    long rows, int ff, float limit) {
-  const long n = rows * ff;
-  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
-    const long r = i / ff;
-    const int c = (int)(i % ff);
-    const float g = fminf(ld(gu, r * gu_stride + c), limit);
-    const float u = fminf(fmaxf(ld(gu, r * gu_stride + ff + c), -limit), limit);
-    st(out, i, g * sigmoidf_(1.702f * g) * (u + 1.0f));
-  }
+                                    long rows, int ff, float limit, int vec) {
+  glu_rows(out, gu, gu_stride, rows, ff, vec, [=](float g, float u) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * sigmoidf_(1.702f * g) * (u + 1.0f);
+  });
 }
 
 __device__ __forceinline__ float gelu_tanh_(float z) {
@@ -512,15 +554,10 @@ __device__ __forceinline__ float gelu_tanh_(float z) {
 // rows [gate (ff) | up (ff)]: out = act(gate) * up, act = gelu_tanh (0), relu (1) or silu (2)
 template <typename T>
 __global__ void act_glu_kernel(T* __restrict__ out, const T* __restrict__ gu, long gu_stride, long rows, int ff,
-                               int act) {
-  const long n = rows * ff;
-  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long)gridDim.x * blockDim.x) {
-    const long r = i / ff;
-    const int c = (int)(i % ff);
-    const float g = ld(gu, r * gu_stride + c);
-    const float a = act == 2 ? g * sigmoidf_(g) : act == 1 ? fmaxf(g, 0.f) : gelu_tanh_(g);
-    st(out, i, a * ld(gu, r * gu_stride + ff + c));
-  }
+                               int act, int vec) {
+  glu_rows(out, gu, gu_stride, rows, ff, vec, [=](float g, float u) {
+    return (act == 2 ? g * sigmoidf_(g) : act == 1 ? fmaxf(g, 0.f) : gelu_tanh_(g)) * u;
+  });
 }
 
 template <typename T>
@@ -661,6 +698,12 @@ static inline unsigned ew_grid(long n) {
   return (unsigned)(g < 1 ? 1 : g > 65535 ? 65535 : g);
 }
 
+// whole 16-byte pieces in every row of gate, up and out
+static inline int glu_vec(const void* out, const void* gu, int bf16, long gu_stride, int ff) {
+  const int n = bf16 ? 8 : 4;
+  return ff % n == 0 && gu_stride % n == 0 && ((uintptr_t)out | (uintptr_t)gu) % 16 == 0;
+}
+
 extern "C" int mx_tanh_cap(float* x, long n, float cap, hipStream_t s) {
   if (n <= 0) return 0;
   if (!(cap > 0.f)) return -1;
@@ -693,8 +736,9 @@ extern "C" int mx_gather_add_rows(float* out, const void* y, int y_bf16, const i
 extern "C" int mx_clamp_swiglu(void* out, const void* gu, int bf16, long gu_stride, long rows, int ff,
                                float limit, hipStream_t s) {
   if (rows * ff <= 0) return 0;
-  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((clamp_swiglu_kernel<T>), dim3(ew_grid(rows * ff)), dim3(256), 0,
-                                         s, (T*)out, (const T*)gu, gu_stride, rows, ff, limit));
+  const int vec = glu_vec(out, gu, bf16, gu_stride, ff);
+  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((clamp_swiglu_kernel<T>), dim3(ew_grid(vec ? rows * (ff / GluVec<T>::N) : rows * ff)),
+                                         dim3(256), 0, s, (T*)out, (const T*)gu, gu_stride, rows, ff, limit, vec));
   return (int)hipGetLastError();
 }
 
@@ -702,8 +746,9 @@ extern "C" int mx_act_glu(void* out, const void* gu, int bf16, long gu_stride, l
                           hipStream_t s) {
   if (rows * ff <= 0) return 0;
   if (act < 0 || act > 2) return -1;
-  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((act_glu_kernel<T>), dim3(ew_grid(rows * ff)), dim3(256), 0, s, (T*)out,
-                                         (const T*)gu, gu_stride, rows, ff, act));
+  const int vec = glu_vec(out, gu, bf16, gu_stride, ff);
+  MX_DISPATCH_T(bf16, hipLaunchKernelGGL((act_glu_kernel<T>), dim3(ew_grid(vec ? rows * (ff / GluVec<T>::N) : rows * ff)),
+                                         dim3(256), 0, s, (T*)out, (const T*)gu, gu_stride, rows, ff, act, vec));
   return (int)hipGetLastError();
 }
 
