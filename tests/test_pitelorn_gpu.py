@@ -187,6 +187,33 @@ def test_attention_kernels_multi_segment(dtype):
         _compare(run, dtype, ("q", "k cache", "v cache", "history", "attention", "weights"))
 
 
+@pytest.mark.parametrize("H,G,dk,dv,window", [(16, 4, 128, 128, 150), (6, 2, 24, 40, 100), (32, 8, 64, 64, 0), (5, 5, 16, 8, 1),
+                                              (24, 3, 40, 72, 64), (64, 8, 32, 32, 65), (2, 1, 256, 256, 0)])
+@pytest.mark.parametrize("sink", ["none", "one", "heads"])
+def test_plain_attention_on_key_tiles(H, G, dk, dv, window, sink):
+    """bf16 decode rows and short segments on the head-mixing attention's key tiles, without a mix:
+    window or every earlier key, cap, sinks, padding segments."""
+    from fasttalk_llm_microservice_amd.ops import mixers as M
+
+    g = torch.Generator().manual_seed(13)
+    page = 8
+    rows, pos0, slots = [1, 13, 5, 1], [270, 0, 30, 2], [2, 0, 3, 1]
+    seg, _, _, nb = _segments("cuda", rows, pos0, slots, page, pad=2)
+    T = sum(rows)
+    q = torch.randn(T, H * dk, generator=g)
+    kc = torch.randn(nb, page, G * dk, generator=g).bfloat16()
+    vc = (torch.randn(nb, page, G * dv, generator=g) * 0.5).bfloat16()
+    sinks = torch.randn(H, generator=g) * 3
+    for cap in (0.0, 4.0):
+        def run(dev):
+            s = {"none": None, "one": 1.5, "heads": sinks.to(dev)}[sink]
+            spec = M.WindowSpec(H, G, dk, dv, window, 1.5 * dk ** -0.5, softcap=cap, sink=s)
+            assert M._plain_tiles(spec, kc)
+            return (M.window_attention(q.to(dev), kc.to(dev), vc.to(dev), _on(seg, dev), spec),)
+
+        _compare(run, torch.float32, ("attention",), tol32=1e-4)
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_scaled_pair_rows_and_plain_add(dtype):
     from fasttalk_llm_microservice_amd.ops import mixers as M
