@@ -1,11 +1,12 @@
 """Sequence-mixer and mixture-of-experts ops: latent (low-rank KV) attention over a
 paged latent cache, windowed attention (softmax or sigmoid weights, distance bias,
-several score maps per head, capped scores, a sink in the softmax) over a paged key / value cache, attention that mixes its scores across the heads, the gated delta-rule
-recurrence (a decay per channel or per head), retention and the selective state-space scan
-over state slots, short causal convolutions (alone, or fused with per-head norms, rotation
-and the cache write, or with the delta rule's preparation), routing (grouped softmax top-k,
-or top-k on the logits with softmax or sigmoid weights, optionally limited to the best groups), clamped-GLU, silu-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product
-for many), and the fp32-residual norms (RMS pre/post norms, optionally with a token shift, layer
+several score maps per head, capped scores, a sink in the softmax) over a paged key / value
+cache, attention that mixes its scores across the heads, the gated delta-rule recurrence (a
+decay per channel or per head), retention and the selective state-space scan over state
+slots, short causal convolutions (alone, or fused with per-head norms, rotation and the cache
+write, or with the delta rule's preparation), routing (grouped softmax top-k, or top-k on the
+logits with softmax or sigmoid weights, optionally limited to the best groups), clamped-GLU,
+silu-GLU and relu^2 experts (per-pair kernels for few rows, a grouped product for many), and the fp32-residual norms (RMS pre/post norms, optionally with a token shift, layer
 norm with bias) that tie them together.
 
 GPU tensors run the gfx950 kernels of the ``_C_mixers`` extension (``csrc/mixers``),
@@ -939,8 +940,9 @@ def moe_top_sigmoid(z, top: int, scale: float, groups: int = 1, keep: int = 1):
 
 def moe_route_top_logits(h, router, bias, top: int, sigmoid: bool = False, scale: float = 1.0, groups: int = 1,
                          keep: int = 1):
-    """:func:`moe_top_logits` (or, ``sigmoid``, :func:`moe_top_sigmoid` with ``scale`` and groups) of z = router h + bias (fp32 router [E, width] and bias, h fp32
-    or bf16, fp32 accumulation) in one launch: the router of few rows (decode steps)."""
+    """:func:`moe_top_logits` (or, ``sigmoid``, :func:`moe_top_sigmoid` with ``scale`` and
+    groups) of z = router h + bias (fp32 router [E, width] and bias, h fp32 or bf16, fp32
+    accumulation) in one launch: the router of few rows (decode steps)."""
     if h.is_cuda:
         t = h.shape[0]
         idx = torch.empty(t, top, dtype=torch.int32, device=h.device)
